@@ -19,6 +19,9 @@
 extern "C" {
 #endif
 
+/* which two values of a head a rotation turns together: neighbours (2i, 2i + 1), or value i with value i + rot_dims / 2 */
+enum { PEGAINFER_ROT_PAIRS = 0, PEGAINFER_ROT_HALVES = 1 };
+
 /* ---- residual stream in fp32 ---- */
 /* out[t, :] = embed[token_ids[t], :] widened to fp32 */
 pegainfer_status_t pegainfer_embed_f32(const void* embed, const uint32_t* token_ids, float* out, int32_t width,
@@ -97,6 +100,36 @@ pegainfer_status_t pegainfer_latent_prep(const void* proj, int64_t proj_row_stri
                                          const int32_t* page_ids, void* cache, int64_t page_stride, int64_t layer_off,
                                          int32_t page_size, float* qc, int32_t heads, int32_t nope, int32_t rot,
                                          int32_t rank, int32_t n_tokens, int32_t dtype, pegainfer_stream_t stream);
+/* The same in parts, each optional (its pointer NULL), with a choice of the rotation's layout (PEGAINFER_ROT_*):
+ *   dkv rows [c: rank | kr: rot] -> cache entry as above (NULL: the layer reads another layer's entries and caches nothing);
+ *   ql rows [q_rank], a query latent -> ql_out packed rows of the storage type, ql / sqrt(mean(ql^2) + eps) * ql_norm_w;
+ *   q rows [heads][nope | rot] -> qc[t, h, rank:], rotated.
+ * A model with a query latent calls it twice: before the up-projection of the queries (dkv, ql) and after it (q). */
+typedef struct {
+  const void* dkv;
+  int64_t dkv_stride;
+  const void* c_norm_w;
+  const void* ql;
+  int64_t ql_stride;
+  const void* ql_norm_w;
+  void* ql_out;
+  int32_t q_rank;
+  const void* q;
+  int64_t q_stride;
+  float* qc;
+  float eps;
+  const float* inv_freq;
+  int32_t rot_dims, rot_layout;
+  const int32_t* positions;
+  const int32_t* token_req;
+  const int32_t* page_indptr;
+  const int32_t* page_ids;
+  void* cache;
+  int64_t page_stride, layer_off;
+  int32_t page_size;
+  int32_t heads, nope, rot, rank, n_tokens, dtype;
+} pegainfer_latent_prep_desc;
+pegainfer_status_t pegainfer_latent_prep_form(const pegainfer_latent_prep_desc* d, pegainfer_stream_t stream);
 /* Causal softmax attention of every (token, head) row over its request's cache entries 0 .. position:
  *   score_j = (qc[t, h, :] . entry_j) * scale;  o_lat[t, h, :] = sum_j softmax(score)_j * entry_j[:rank]
  * qc fp32 [T, heads, rank + rot], o_lat fp32 [T, heads, rank]; scores, running maxima / sums and accumulators in fp32.
@@ -116,6 +149,18 @@ pegainfer_status_t pegainfer_latent_attention(const float* qc, float* o_lat, con
                                               float scale, int32_t n_tokens, int32_t max_kv_len, int32_t split_keys,
                                               float* workspace, const int32_t* tile_row0, const int32_t* tile_rows,
                                               int32_t n_tiles, int32_t dtype, pegainfer_stream_t stream);
+
+/* The same with a row's keys dealt in tiles (32 keys, 256 in the plain form) to n_split workgroups in turn: the grid depends on the
+ * step's shape only, never on the contexts' lengths, so a recorded launch serves every later step of its shape.
+ * workspace: pegainfer_latent_attention_dealt_workspace(...) floats. */
+int64_t pegainfer_latent_attention_dealt_workspace(int32_t n_tokens, int32_t heads, int32_t rank, int32_t n_split);
+pegainfer_status_t pegainfer_latent_attention_dealt(const float* qc, float* o_lat, const void* cache, int64_t page_stride,
+                                                    int64_t layer_off, int32_t page_size, const int32_t* positions,
+                                                    const int32_t* token_req, const int32_t* page_indptr, const int32_t* page_ids,
+                                                    int32_t heads, int32_t rank, int32_t rot, float scale, int32_t n_tokens,
+                                                    int32_t n_split, float* workspace, const int32_t* tile_row0,
+                                                    const int32_t* tile_rows, int32_t n_tiles, int32_t dtype,
+                                                    pegainfer_stream_t stream);
 
 /* ---- routed experts ----
  * Router: z = W_r h (fp32 accumulation of the stored values), s = sigmoid(z), choice = s + correction (NULL = none).
@@ -259,6 +304,39 @@ pegainfer_status_t pegainfer_glu_rows(const void* gate, const void* up, int64_t 
 /* out[i] = cap * tanh(in[i] / cap) over n fp32 values (in place allowed) */
 pegainfer_status_t pegainfer_softcap_rows(const float* in, float* out, int64_t n, float cap, pegainfer_stream_t stream);
 
+/* ---- several residual streams with learned mixing (hyper-connections) ----
+ * A token's row holds its streams back to back: [rows][streams][d] fp32.  One launch between two sublayers; every part optional:
+ *   source   x_in rows (row_index: the source row of an output row, NULL = itself), or, with x_in NULL, embed[token_ids[row]] *
+ *            embed_scale in every stream;
+ *   y        (rows of dtype at y_row_stride, NULL = none)  X_t <- sum_s mix[s, t] X_s + mult * out_w[t] * y, all t from the old
+ *            streams; mix [streams][streams] is indexed [from][to];
+ *   x_out    the streams (may alias x_in unless row_index is given);  sum_out [rows][d]: their plain sum;
+ *   n_out    [rows][d] of dtype: u = sum_s read_w[s] X_s (read_w NULL: plain sum), normed: RMS u / sqrt(mean(u^2) + eps) * gain, or
+ *            LAYER (u - mean) / sqrt(mean((u - mean)^2) + eps) * gain.
+ * mix, out_w, read_w, gain of dtype.  streams <= 16, d <= 32768. */
+enum { PEGAINFER_NORM_RMS = 0, PEGAINFER_NORM_LAYER = 1 };
+typedef struct {
+  const float* x_in;
+  const void* embed;
+  const uint32_t* token_ids;
+  float embed_scale;
+  const int32_t* row_index;
+  const void* y;
+  int64_t y_row_stride;
+  const void* mix;
+  const void* out_w;
+  float mult;
+  float* x_out;
+  float* sum_out;
+  const void* read_w;
+  const void* gain;
+  void* n_out;
+  float eps;
+  int32_t norm_kind;
+  int32_t streams, d, rows, dtype;
+} pegainfer_stream_mix_desc;
+pegainfer_status_t pegainfer_stream_mix(const pegainfer_stream_mix_desc* q, pegainfer_stream_t stream);
+
 /* ---- recurrent matrix memories (state per (slot, head): S [dim][vdim] fp32, row-major) ----
  * Gated delta rule.  Per row, from qkv (fp32 [rows][qkv_stride]: q heads at 0, k heads at kv_heads * dim, v heads at
  * 2 * kv_heads * dim) and the projection row `proj` (dtype; beta logits at b_off, decay inputs at a_off, one per head):
@@ -304,6 +382,44 @@ pegainfer_status_t pegainfer_ssd_scan(const float* xbc, int64_t xbc_stride, cons
                                       float* o, int32_t heads, int32_t groups, int32_t n_state, int32_t vdim,
                                       const int32_t* entry_row0, const int32_t* entry_slot, int32_t n_entries, int32_t dtype,
                                       pegainfer_stream_t stream);
+/* Linear attention with a constant decay per head (state per (slot, head): S [dim][vdim] fp32, row-major, the heads back to back).
+ * Per row of `proj` (dtype): q at q_off, k at k_off (heads x dim), v at v_off (heads x vdim), each through silu when silu != 0:
+ *   S <- g_h S + k v^T;  y = S^T q                -> o (fp32 [rows][heads * vdim])
+ * decay_pow: fp32 [heads][pow_n], g_h^n for n = 0 .. pow_n - 1 (pow_n >= 2).  Everything in fp32.
+ * Two forms.  The scan walks an entry's tokens one by one (dim <= 256).  The chunk form takes chunks of <= 64 tokens side by side
+ * on fp32 matrix-core products: every chunk's sum of decayed k v^T, a walk over the chunks that leaves the state before each, then
+ * every chunk's outputs from that state and its own tokens.  It is taken for the entries of the tables when
+ * pegainfer_decay_attention_chunked_ok says the sizes fit; the scan then leaves alone the entries of more than scan_max rows.
+ *   chunk_row0 / chunk_rows / [n_chunks]: the chunks of all long entries, entry by entry;  long_chunk0 [n_long + 1]: the first
+ *   chunk of every long entry;  long_slot [n_long]: its state slot;  pow_n > the largest chunk_rows;
+ *   workspace: pegainfer_decay_attention_workspace(...) floats. */
+enum { PEGAINFER_DECAY_CHUNK = 64 };
+typedef struct {
+  const void* proj;
+  int64_t proj_stride, q_off, k_off, v_off;
+  int32_t silu;
+  const float* decay_pow;
+  int32_t pow_n;
+  float* state;
+  int64_t slot_stride;
+  float* o;
+  int32_t heads, dim, vdim;
+  const int32_t* entry_row0;
+  const int32_t* entry_slot;
+  int32_t n_entries;
+  int32_t scan_max;            /* 0: the scan takes every entry */
+  const int32_t* chunk_row0;
+  const int32_t* chunk_rows;
+  int32_t n_chunks;
+  const int32_t* long_chunk0;
+  const int32_t* long_slot;
+  int32_t n_long;
+  float* workspace;
+  int32_t dtype;
+} pegainfer_decay_attention_desc;
+int32_t pegainfer_decay_attention_chunked_ok(int32_t dim, int32_t vdim);
+int64_t pegainfer_decay_attention_workspace(int32_t n_chunks, int32_t heads, int32_t dim, int32_t vdim);
+pegainfer_status_t pegainfer_decay_attention(const pegainfer_decay_attention_desc* d, pegainfer_stream_t stream);
 /* Per-head RMS norm of a memory's read-out, a weight, a gate and a constant factor:
  *   out[row, h, :] = o[row, h, :] / sqrt(mean(o[row, h, :]^2) + eps) * w * act(gate[row, h, :]) * factor
  * w: [vdim] shared by the heads (w_per_head == 0) or [heads * vdim]; gate_kind 0 = silu, 1 = sigmoid; gate rows of dtype
@@ -354,7 +470,6 @@ pegainfer_status_t pegainfer_qk_prep_paged(const void* proj, int64_t proj_stride
  * heads of q (of k) before the rotation, times q_norm [heads * dim] / k_norm [kv_heads * dim].  rot_layout PAIRS: neighbours
  * (2i, 2i + 1) turn together; HALVES: value i with value i + rot_dims / 2, both by position * inv_freq[i].  dim <= 256. */
 enum { PEGAINFER_QKNORM_HEAD_WEIGHT = 0, PEGAINFER_QKNORM_HEAD_UNIT_AFTER = 1, PEGAINFER_QKNORM_ALL_WEIGHT = 2 };
-enum { PEGAINFER_ROT_PAIRS = 0, PEGAINFER_ROT_HALVES = 1 };
 pegainfer_status_t pegainfer_qk_prep_paged_form(const void* proj, int32_t proj_dtype, int64_t proj_stride, int64_t q_off,
                                                int64_t k_off, int64_t v_off, int32_t heads, int32_t kv_heads, int32_t dim,
                                                int32_t vdim, const void* q_norm, const void* k_norm, int32_t norm_kind, float eps,
@@ -415,6 +530,36 @@ pegainfer_status_t pegainfer_paged_attention_masked(const float* q, const void* 
                                                     int32_t keep_first, const float* dist_bias, int32_t n_dist, const void* gate,
                                                     int64_t gate_stride, int32_t gate_kind, int32_t n_split, float* workspace,
                                                     int32_t plain, int32_t dtype, pegainfer_stream_t stream);
+/* The same with the options in a struct (zeroed = plain causal softmax attention, unsplit; maps 0 counts as 1) and one more:
+ * dist_slope: fp32 [heads] (or NULL); dist_slope[h] * (i - j) is taken off the scaled, capped score of query head h - a bias that
+ * grows linearly with the distance, without a table and without a limit. */
+typedef struct {
+  int32_t maps;
+  float lambda;
+  int32_t block;
+  const void* sink;
+  int32_t head_norm;
+  float norm_eps;
+  float softcap;
+  int32_t window, keep_first;
+  const float* dist_bias;
+  int32_t n_dist;
+  const float* dist_slope;
+  const void* gate;
+  int64_t gate_stride;
+  int32_t gate_kind;
+  int32_t n_split;
+  float* workspace;
+  int32_t plain;
+} pegainfer_attn_options;
+pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cache, int64_t page_stride, int64_t k_cache_off,
+                                                 int64_t v_cache_off, int32_t page_size, const int32_t* positions,
+                                                 const int32_t* row_entry, const int32_t* page_indptr, const int32_t* page_ids,
+                                                 int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, float scale,
+                                                 float factor, const int32_t* tile_row0, const int32_t* tile_ntok,
+                                                 const int32_t* tile_qh0, const int32_t* tile_nqh, int32_t n_tiles, void* out,
+                                                 int64_t out_stride, const pegainfer_attn_options* opt, int32_t dtype,
+                                                 pegainfer_stream_t stream);
 /* fp32 values of scratch a launch with n_split > 1 needs (0 for n_split <= 1) */
 int64_t pegainfer_paged_attention_workspace(int32_t n_tiles, int32_t kv_heads, int32_t vdim, int32_t maps, int32_t n_split);
 /* out[row, :cols] = in[row, :cols] * factor; rows of in / out at their own strides (elements of dtype) */

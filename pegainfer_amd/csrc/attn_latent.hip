@@ -10,13 +10,13 @@
 // Scores, softmax weights, running maxima / sums and the output accumulators are fp32; the fp32 instance reads an fp32
 // cache, the bf16 instance widens bf16 entries exactly.
 //
-//   latent_prep_kernel        RMS-norm of the latent, rotation of the shared key part and of the query's rotated part,
-//                             cache write (one workgroup per token row)
+//   latent_prep_kernel        RMS-norm of the latent, rotation of the shared key part and of the query's rotated part (halves or
+//                             neighbours), cache write; RMS-norm of a query latent (each part optional)
 //   latent_attn_kernel        one workgroup per (token, head, key split): 256 keys per round, scores by one thread per
 //                             key, online softmax, value accumulation by one thread per latent dimension
 //   latent_attn_merge_kernel  combines the key splits of a row (log-sum-exp weights), fixed split order
-// A row's result depends on its own query, position and cache entries only: the split count is a function of the row's
-// key count alone, so batch composition and portion boundaries change nothing.
+// A row's result depends on its own query, position and cache entries only.  With contiguous splits the split count is a
+// function of the row's key count alone; with dealt splits it also depends on the step's shape (rounding only).
 #include "common.h"
 #include "typed.h"
 #include "pegainfer_kernels_blocks.h"
@@ -35,55 +35,83 @@ __device__ __forceinline__ float block_max256(float v, float* red) {
   return fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
 }
 
+// How a row's keys are cut into splits.  Contiguous: split z holds keys z * grain .. (z + 1) * grain - 1, and the number of splits
+// follows the context's length.  Dealt: runs of `grain` keys (one tile) go round the splits in turn - split z takes runs z,
+// z + n, ... - so the launch's grid does not depend on the contexts' lengths and a recorded launch serves every later step.
+struct LatentCut {
+  int grain, dealt;
+  __device__ __forceinline__ int splits_of(int n_keys, int max_splits) const { return min(max_splits, (n_keys + grain - 1) / grain); }
+  __device__ __forceinline__ int end_of(int split, int n_keys) const { return dealt ? n_keys : min(n_keys, (split + 1) * grain); }
+  __device__ __forceinline__ int step(int tile, int max_splits) const { return dealt ? tile * max_splits : tile; }
+};
+
 template <typename A>
 __device__ __forceinline__ const A* latent_entry(const A* cache, int64_t page_stride, int64_t layer_off, int page_size,
                                                  const int32_t* pages, int j, int E) {
   return cache + (int64_t)pages[j / page_size] * page_stride + layer_off + (int64_t)(j % page_size) * E;
 }
 
+// What one prep launch does to a token row; every part is optional (its pointer NULL).
 template <typename A>
-__global__ __launch_bounds__(256) void latent_prep_kernel(const A* __restrict__ proj, int64_t row_stride, int64_t dkv_off,
-                                                          const A* __restrict__ cw, float eps,
-                                                          const float* __restrict__ inv_freq, int rot_dims,
-                                                          const int32_t* __restrict__ positions,
+struct LatentPrep {
+  const A* dkv; int64_t dkv_stride; const A* c_norm;                      // [c: r | kr: dr] -> cache entry
+  const A* ql; int64_t ql_stride; const A* ql_norm; A* ql_out; int q_rank;  // query latent, RMS-normed with a weight -> packed rows
+  const A* q; int64_t q_stride; float* qc;                                // rotated parts of the heads' queries -> qc (fp32)
+};
+
+template <typename A>
+__global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrep<A> a, float eps, const float* __restrict__ inv_freq, int rot_dims,
+                                                          int pairs, const int32_t* __restrict__ positions,
                                                           const int32_t* __restrict__ token_req,
                                                           const int32_t* __restrict__ page_indptr,
                                                           const int32_t* __restrict__ page_ids, A* __restrict__ cache,
-                                                          int64_t page_stride, int64_t layer_off, int page_size,
-                                                          float* __restrict__ qc, int H, int dn, int dr, int r) {
+                                                          int64_t page_stride, int64_t layer_off, int page_size, int H, int dn,
+                                                          int dr, int r) {
   __shared__ float red[4];
   const int t = blockIdx.x, tid = threadIdx.x;
-  const A* row = proj + (int64_t)t * row_stride;
-  const A* dkv = row + dkv_off;
-  const int pos = positions[t], req = token_req[t];
+  const int pos = positions[t];
   const int E = r + dr;
-  A* entry = cache + (int64_t)page_ids[page_indptr[req] + pos / page_size] * page_stride + layer_off +
-             (int64_t)(pos % page_size) * E;
-  float ss = 0.f;
-  for (int i = tid; i < r; i += 256) { const float v = ld(dkv + i); ss += v * v; }
-  ss = block_sum<4>(ss, red);
-  const float inv = 1.0f / sqrtf(ss / (float)r + eps);
-  for (int i = tid; i < r; i += 256) st(entry + i, ld(dkv + i) * inv * ld(cw + i));
+  const A* dkv = a.dkv ? a.dkv + (int64_t)t * a.dkv_stride : nullptr;
+  A* entry = nullptr;
+  if (dkv) {
+    const int req = token_req[t];
+    entry = cache + (int64_t)page_ids[page_indptr[req] + pos / page_size] * page_stride + layer_off + (int64_t)(pos % page_size) * E;
+  }
+  // with several workgroups per row (few rows) the first norms the key latent, the last the query latent
+  if (dkv && blockIdx.y == 0) {
+    float ss = 0.f;
+    for (int i = tid; i < r; i += 256) { const float v = ld(dkv + i); ss += v * v; }
+    ss = block_sum<4>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)r + eps);
+    for (int i = tid; i < r; i += 256) st(entry + i, ld(dkv + i) * inv * ld(a.c_norm + i));
+  }
+  if (a.ql && blockIdx.y + 1 == gridDim.y) {
+    const A* ql = a.ql + (int64_t)t * a.ql_stride;
+    A* out = a.ql_out + (int64_t)t * a.q_rank;
+    float ss = 0.f;
+    for (int i = tid; i < a.q_rank; i += 256) { const float v = ld(ql + i); ss += v * v; }
+    ss = block_sum<4>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)a.q_rank + eps);
+    for (int i = tid; i < a.q_rank; i += 256) st(out + i, ld(ql + i) * inv * ld(a.ql_norm + i));
+  }
   const int half = rot_dims >> 1;
   const float fpos = (float)pos;
   // vector 0 = the shared key part (-> cache), vectors 1 .. H = the heads' rotated query parts (-> qc, fp32)
-  for (int w = tid; w < (H + 1) * dr; w += 256) {
+  const int w_end = (a.q ? H + 1 : 1) * dr;
+  for (int w = (dkv ? 0 : dr) + blockIdx.y * 256 + tid; w < w_end; w += 256 * gridDim.y) {
     const int vec = w / dr, i = w % dr;
-    const A* src = vec == 0 ? dkv + r : row + (int64_t)(vec - 1) * (dn + dr) + dn;
-    float out;
-    if (i < half) {
+    const A* src = vec == 0 ? dkv + r : a.q + (int64_t)t * a.q_stride + (int64_t)(vec - 1) * (dn + dr) + dn;
+    float out = ld(src + i);
+    if (i < rot_dims) {
       float sn, cs;
-      sincosf(fpos * inv_freq[i], &sn, &cs);
-      out = ld(src + i) * cs - ld(src + i + half) * sn;
-    } else if (i < rot_dims) {
-      float sn, cs;
-      sincosf(fpos * inv_freq[i - half], &sn, &cs);
-      out = ld(src + i) * cs + ld(src + i - half) * sn;
-    } else {
-      out = ld(src + i);
+      const int f = pairs ? i >> 1 : (i < half ? i : i - half);
+      const bool second = pairs ? (i & 1) : i >= half;
+      const float other = ld(src + (pairs ? i ^ 1 : second ? i - half : i + half));
+      sincosf(fpos * inv_freq[f], &sn, &cs);
+      out = second ? out * cs + other * sn : out * cs - other * sn;
     }
     if (vec == 0) st(entry + r + i, out);
-    else qc[((int64_t)t * H + (vec - 1)) * E + r + i] = out;
+    else a.qc[((int64_t)t * H + (vec - 1)) * E + r + i] = out;
   }
 }
 
@@ -96,15 +124,15 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const float* __restric
                                                           const int32_t* __restrict__ token_req,
                                                           const int32_t* __restrict__ page_indptr,
                                                           const int32_t* __restrict__ page_ids, int H, int r, int dr,
-                                                          float scale, float* __restrict__ partial, int max_splits, int split_keys) {
+                                                          float scale, float* __restrict__ partial, int max_splits, LatentCut cut) {
   extern __shared__ float smem[];
   __shared__ float red[4];
   const int t = blockIdx.x, h = blockIdx.y, split = blockIdx.z, tid = threadIdx.x;
   const int E = r + dr;
   const int n_keys = positions[t] + 1;
-  const int n_splits = (n_keys + split_keys - 1) / split_keys;
+  const int n_splits = cut.splits_of(n_keys, max_splits);
   if (split >= n_splits) return;
-  const int j_lo = split * split_keys, j_hi = min(n_keys, j_lo + split_keys);
+  const int j_lo = split * cut.grain, j_hi = cut.end_of(split, n_keys), j_step = cut.step(kLatKeys, max_splits);
   float* q = smem;            // [E]
   float* p = smem + E;        // [kLatKeys]
   const float* qrow = qc + ((int64_t)t * H + h) * E;
@@ -112,7 +140,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const float* __restric
   const int32_t* pages = page_ids + page_indptr[token_req[t]];
   float m = -INFINITY, l = 0.f, acc[kLatAcc] = {};
   __syncthreads();
-  for (int j0 = j_lo; j0 < j_hi; j0 += kLatKeys) {
+  for (int j0 = j_lo; j0 < j_hi; j0 += j_step) {
     const int j = j0 + tid;
     float s = -INFINITY;
     if (j < j_hi) {
@@ -159,11 +187,11 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const float* __restric
 
 __global__ __launch_bounds__(256) void latent_attn_merge_kernel(float* __restrict__ o_lat, const float* __restrict__ partial,
                                                                 const int32_t* __restrict__ positions, int H, int r,
-                                                                int max_splits, int split_keys) {
+                                                                int max_splits, LatentCut cut) {
   extern __shared__ float wsm[];   // [n_splits] weights exp(m_s - m) / l
   __shared__ float red[4];
   const int t = blockIdx.x, h = blockIdx.y;
-  const int n_splits = (positions[t] + split_keys) / split_keys;
+  const int n_splits = cut.splits_of(positions[t] + 1, max_splits);
   if (n_splits <= 1) return;
   const float* part = partial + ((int64_t)t * H + h) * max_splits * (r + 2);
   // the splits' maxima and sums are read in parallel (one thread each), combined in split order
@@ -211,7 +239,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const float* __re
                                                                const int32_t* __restrict__ tile_row0,
                                                                const int32_t* __restrict__ tile_rows, int H, int r, int dr,
                                                                float scale, float* __restrict__ partial, int max_splits,
-                                                               int split_keys) {
+                                                               LatentCut cut) {
   extern __shared__ __align__(16) uint8_t lat_smem[];
   typedef short v4s_t __attribute__((ext_vector_type(4)));
   const int E = r + dr, Epad = (E + 31) & ~31;
@@ -222,9 +250,9 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const float* __re
   const int row0 = tile_row0[blockIdx.x], cnt = tile_rows[blockIdx.x], split = blockIdx.y;
   const int t_first = row0 / H, t_last = (row0 + cnt - 1) / H;
   const int pmax = positions[t_last];
-  const int j_lo = split * split_keys;
+  const int j_lo = split * cut.grain;
   if (j_lo > pmax) return;
-  const int j_hi = min(pmax + 1, j_lo + split_keys);
+  const int j_hi = cut.end_of(split, pmax + 1), j_step = cut.step(kTileKeys, max_splits);
   const int32_t* pages = page_ids + page_indptr[token_req[t_first]];
   const int nchunk = E >> 3, tile_chunks = kTileKeys * nchunk;
   // this thread's chunks of a key tile: key kk, element offset ch * 8 - fixed for the whole loop, so the integer divisions
@@ -274,13 +302,13 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const float* __re
   float m = -INFINITY, l = 0.f;
   // per-lane element offset of the transposed reads inside the key tile: key row 4g + (l15 >> 2), dims 4 (l15 & 3) ..
   const int tr_off = (4 * g + (l15 >> 2)) * cs + 4 * (l15 & 3);
-  for (int j0 = j_lo; j0 < j_hi; j0 += kTileKeys) {
+  for (int j0 = j_lo; j0 < j_hi; j0 += j_step) {
     __syncthreads();                                                 // the previous tile's reads are done
 #pragma unroll
     for (int i = 0; i < kLatPrefetch; ++i)
       if (ck_kk[i] >= 0) *reinterpret_cast<u32x4*>(Ck + ck_kk[i] * cs + ck_el[i]) = pre[i];
     __syncthreads();
-    if (j0 + kTileKeys < j_hi) fetch(j0 + kTileKeys);
+    if (j0 + j_step < j_hi) fetch(j0 + j_step);
     if (!wave_live) continue;
     // two independent accumulator pairs over alternating k slices: with one wave per SIMD the LDS read -> MFMA -> MFMA chain
     // of a single pair would run at its latency
@@ -353,7 +381,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const float* __re
     }
   }
   if (my_row >= cnt) return;
-  const int own_splits = (pq + split_keys) / split_keys;
+  const int own_splits = cut.splits_of(pq + 1, max_splits);
   const int64_t grow = row0 + my_row;
   if (own_splits == 1) {
     if (split != 0) return;
@@ -379,7 +407,7 @@ static void latent_attn_mfma_launch(const float* qc, float* o_lat, const uint16_
                                     int page_size, const int32_t* positions, const int32_t* token_req,
                                     const int32_t* page_indptr, const int32_t* page_ids, const int32_t* tile_row0,
                                     const int32_t* tile_rows, int n_tiles, int H, int r, int dr, float scale, float* ws, int sp,
-                                    int split_keys, hipStream_t s) {
+                                    LatentCut cut, hipStream_t s) {
   const int Epad = (r + dr + 31) & ~31;
   const int lds = (kTileRows + kTileKeys) * (Epad + 8) * 2;
   auto kern = &latent_attn_mfma_kernel<ND>;
@@ -387,7 +415,7 @@ static void latent_attn_mfma_launch(const float* qc, float* o_lat, const uint16_
                                                 160 * 1024), true);
   (void)once;
   kern<<<dim3(n_tiles, sp), 256, lds, s>>>(qc, o_lat, cache, page_stride, layer_off, page_size, positions, token_req, page_indptr,
-                                           page_ids, tile_row0, tile_rows, H, r, dr, scale, ws, sp, split_keys);
+                                           page_ids, tile_row0, tile_rows, H, r, dr, scale, ws, sp, cut);
 }
 
 static inline int latent_split_keys(int split_keys) { return split_keys > 0 ? split_keys : kLatSplitKeys; }
@@ -407,15 +435,36 @@ pegainfer_status_t pegainfer_latent_prep(const void* proj, int64_t proj_row_stri
                                          const int32_t* page_ids, void* cache, int64_t page_stride, int64_t layer_off,
                                          int32_t page_size, float* qc, int32_t heads, int32_t nope, int32_t rot,
                                          int32_t rank, int32_t n_tokens, int32_t dtype, pegainfer_stream_t stream) {
-  if (n_tokens <= 0) return 0;
-  if (rot_dims < 0 || rot_dims > rot || (rot_dims & 1) || rank <= 0 || page_size <= 0)
+  pegainfer_latent_prep_desc d{};
+  const int64_t es = dtype == kDtF32 ? 4 : 2;
+  d.dkv = static_cast<const uint8_t*>(proj) + dkv_offset * es; d.dkv_stride = proj_row_stride; d.c_norm_w = c_norm_w;
+  d.q = proj; d.q_stride = proj_row_stride; d.qc = qc;
+  d.eps = eps; d.inv_freq = inv_freq; d.rot_dims = rot_dims; d.rot_layout = PEGAINFER_ROT_HALVES;
+  d.positions = positions; d.token_req = token_req; d.page_indptr = page_indptr; d.page_ids = page_ids;
+  d.cache = cache; d.page_stride = page_stride; d.layer_off = layer_off; d.page_size = page_size;
+  d.heads = heads; d.nope = nope; d.rot = rot; d.rank = rank; d.n_tokens = n_tokens; d.dtype = dtype;
+  return pegainfer_latent_prep_form(&d, stream);
+}
+
+pegainfer_status_t pegainfer_latent_prep_form(const pegainfer_latent_prep_desc* d, pegainfer_stream_t stream) {
+  if (!d) return (pegainfer_status_t)hipErrorInvalidValue;
+  if (d->n_tokens <= 0) return 0;
+  if (d->rot_dims < 0 || d->rot_dims > d->rot || (d->rot_dims & 1) || d->rank <= 0 || d->page_size <= 0 || d->heads < 0 || d->nope < 0 ||
+      (d->rot_dims > 0 && !d->inv_freq) || (d->rot_layout != PEGAINFER_ROT_PAIRS && d->rot_layout != PEGAINFER_ROT_HALVES) ||
+      (!d->dkv && !d->q && !d->ql) || (d->dkv && (!d->c_norm_w || !d->cache)) || (d->q && !d->qc) ||
+      (d->ql && (!d->ql_norm_w || !d->ql_out || d->q_rank <= 0)))
     return (pegainfer_status_t)hipErrorInvalidValue;
-  if (!by_dtype(dtype, [&](auto* t) {
+  if (!by_dtype(d->dtype, [&](auto* t) {
         using A = std::remove_pointer_t<decltype(t)>;
-        latent_prep_kernel<A><<<n_tokens, 256, 0, as_stream(stream)>>>(
-            static_cast<const A*>(proj), proj_row_stride, dkv_offset, static_cast<const A*>(c_norm_w), eps, inv_freq, rot_dims,
-            positions, token_req, page_indptr, page_ids, static_cast<A*>(cache), page_stride, layer_off, page_size, qc,
-            heads, nope, rot, rank);
+        LatentPrep<A> a{static_cast<const A*>(d->dkv), d->dkv_stride, static_cast<const A*>(d->c_norm_w),
+                        static_cast<const A*>(d->ql), d->ql_stride, static_cast<const A*>(d->ql_norm_w), static_cast<A*>(d->ql_out), d->q_rank,
+                        static_cast<const A*>(d->q), d->q_stride, d->qc};
+        // few rows (decoding): a row's rotated parts spread over several workgroups; many rows fill the chip alone
+        const int vals = (d->q ? d->heads + 1 : 1) * d->rot;
+        const int per_row = d->n_tokens >= 256 ? 1 : std::max(d->ql && d->dkv ? 2 : 1, std::min(8, (vals + 255) / 256));
+        latent_prep_kernel<A><<<dim3(d->n_tokens, per_row), 256, 0, as_stream(stream)>>>(
+            a, d->eps, d->inv_freq, d->rot_dims, d->rot_layout == PEGAINFER_ROT_PAIRS, d->positions, d->token_req, d->page_indptr,
+            d->page_ids, static_cast<A*>(d->cache), d->page_stride, d->layer_off, d->page_size, d->heads, d->nope, d->rot, d->rank);
       }))
     return (pegainfer_status_t)hipErrorInvalidValue;
   return (pegainfer_status_t)hipGetLastError();
@@ -433,15 +482,13 @@ int32_t pegainfer_latent_attention_tiled_ok(int32_t rank, int32_t rot, int64_t p
          kTileKeys * ((rank + rot) / 8) <= kLatPrefetch * 256 && (kTileRows + kTileKeys) * (Epad + 8) * 2 <= 160 * 1024;
 }
 
-pegainfer_status_t pegainfer_latent_attention(const float* qc, float* o_lat, const void* cache, int64_t page_stride,
-                                              int64_t layer_off, int32_t page_size, const int32_t* positions,
-                                              const int32_t* token_req, const int32_t* page_indptr,
-                                              const int32_t* page_ids, int32_t heads, int32_t rank, int32_t rot,
-                                              float scale, int32_t n_tokens, int32_t max_kv_len, int32_t split_keys,
-                                              float* workspace, const int32_t* tile_row0, const int32_t* tile_rows,
-                                              int32_t n_tiles, int32_t dtype, pegainfer_stream_t stream) {
-  if (n_tokens <= 0 || heads <= 0) return 0;
-  const int sk = latent_split_keys(split_keys), sp = latent_max_splits(max_kv_len, split_keys);
+// one launch (and its merge) with the keys cut as `cut` says into `sp` splits at most
+static pegainfer_status_t latent_attention_launch(const float* qc, float* o_lat, const void* cache, int64_t page_stride,
+                                                  int64_t layer_off, int32_t page_size, const int32_t* positions,
+                                                  const int32_t* token_req, const int32_t* page_indptr, const int32_t* page_ids,
+                                                  int32_t heads, int32_t rank, int32_t rot, float scale, int32_t n_tokens, int sp,
+                                                  pk::LatentCut cut, float* workspace, const int32_t* tile_row0,
+                                                  const int32_t* tile_rows, int32_t n_tiles, int32_t dtype, pegainfer_stream_t stream) {
   if (sp > 1 && !workspace) return (pegainfer_status_t)hipErrorInvalidValue;
   hipStream_t s = as_stream(stream);
   if (tile_row0) {
@@ -450,7 +497,7 @@ pegainfer_status_t pegainfer_latent_attention(const float* qc, float* o_lat, con
       return (pegainfer_status_t)hipErrorInvalidValue;
     const uint16_t* c = static_cast<const uint16_t*>(cache);
 #define LAT_LAUNCH(ND) latent_attn_mfma_launch<ND>(qc, o_lat, c, page_stride, layer_off, page_size, positions, token_req, page_indptr, \
-                                                   page_ids, tile_row0, tile_rows, n_tiles, heads, rank, rot, scale, workspace, sp, sk, s)
+                                                   page_ids, tile_row0, tile_rows, n_tiles, heads, rank, rot, scale, workspace, sp, cut, s)
     if (rank <= 64) LAT_LAUNCH(4);
     else if (rank <= 128) LAT_LAUNCH(8);
     else if (rank <= 256) LAT_LAUNCH(16);
@@ -465,12 +512,43 @@ pegainfer_status_t pegainfer_latent_attention(const float* qc, float* o_lat, con
           using A = std::remove_pointer_t<decltype(t)>;
           latent_attn_kernel<A><<<grid, 256, smem, s>>>(qc, o_lat, static_cast<const A*>(cache), page_stride, layer_off, page_size,
                                                         positions, token_req, page_indptr, page_ids, heads, rank, rot, scale,
-                                                        workspace, sp, sk);
+                                                        workspace, sp, cut);
         }))
       return (pegainfer_status_t)hipErrorInvalidValue;
   }
-  if (sp > 1) latent_attn_merge_kernel<<<dim3(n_tokens, heads), 256, (size_t)sp * sizeof(float), s>>>(o_lat, workspace, positions, heads, rank, sp, sk);
+  if (sp > 1) latent_attn_merge_kernel<<<dim3(n_tokens, heads), 256, (size_t)sp * sizeof(float), s>>>(o_lat, workspace, positions, heads, rank, sp, cut);
   return (pegainfer_status_t)hipGetLastError();
+}
+
+pegainfer_status_t pegainfer_latent_attention(const float* qc, float* o_lat, const void* cache, int64_t page_stride,
+                                              int64_t layer_off, int32_t page_size, const int32_t* positions,
+                                              const int32_t* token_req, const int32_t* page_indptr,
+                                              const int32_t* page_ids, int32_t heads, int32_t rank, int32_t rot,
+                                              float scale, int32_t n_tokens, int32_t max_kv_len, int32_t split_keys,
+                                              float* workspace, const int32_t* tile_row0, const int32_t* tile_rows,
+                                              int32_t n_tiles, int32_t dtype, pegainfer_stream_t stream) {
+  if (n_tokens <= 0 || heads <= 0) return 0;
+  const int sk = latent_split_keys(split_keys), sp = latent_max_splits(max_kv_len, split_keys);
+  return latent_attention_launch(qc, o_lat, cache, page_stride, layer_off, page_size, positions, token_req, page_indptr, page_ids, heads,
+                                 rank, rot, scale, n_tokens, sp, LatentCut{sk, 0}, workspace, tile_row0, tile_rows, n_tiles, dtype, stream);
+}
+
+int64_t pegainfer_latent_attention_dealt_workspace(int32_t n_tokens, int32_t heads, int32_t rank, int32_t n_split) {
+  return n_split <= 1 ? 0 : (int64_t)n_tokens * heads * n_split * (rank + 2);
+}
+
+pegainfer_status_t pegainfer_latent_attention_dealt(const float* qc, float* o_lat, const void* cache, int64_t page_stride,
+                                                    int64_t layer_off, int32_t page_size, const int32_t* positions,
+                                                    const int32_t* token_req, const int32_t* page_indptr, const int32_t* page_ids,
+                                                    int32_t heads, int32_t rank, int32_t rot, float scale, int32_t n_tokens,
+                                                    int32_t n_split, float* workspace, const int32_t* tile_row0,
+                                                    const int32_t* tile_rows, int32_t n_tiles, int32_t dtype,
+                                                    pegainfer_stream_t stream) {
+  if (n_tokens <= 0 || heads <= 0) return 0;
+  if (n_split < 1 || n_split > 1024) return (pegainfer_status_t)hipErrorInvalidValue;
+  return latent_attention_launch(qc, o_lat, cache, page_stride, layer_off, page_size, positions, token_req, page_indptr, page_ids, heads,
+                                 rank, rot, scale, n_tokens, n_split, LatentCut{tile_row0 ? kTileKeys : kLatKeys, 1}, workspace, tile_row0,
+                                 tile_rows, n_tiles, dtype, stream);
 }
 
 }  // extern "C"

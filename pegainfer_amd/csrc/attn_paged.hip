@@ -150,6 +150,7 @@ struct AttnForm {
   int keep_first = 0;          // tokens stay visible at their true positions)
   const float* dist_bias = nullptr;   // fp32 [n_dist][heads], added to the (scaled, capped) score of query head h by distance:
   int n_dist = 0;                     // dist_bias[min(i - j, n_dist - 1)][h]
+  const float* dist_slope = nullptr;  // fp32 [heads]: slope[h] * (i - j) is taken off the (scaled, capped) score
   const void* gate = nullptr;  // output gate logits (storage type), rows at gate_stride: the finished head is multiplied by
   int64_t gate_stride = 0;     // sigmoid(gate[row, h * vdim + c]) (gate_kind 1: one per value) or sigmoid(gate[row, h]) (2: one
   int gate_kind = 0;           // per head)
@@ -162,10 +163,12 @@ __device__ __forceinline__ int attn_row_lo(const AttnForm& form, int pos) {
   return lo;
 }
 // a raw dot product turned into the score of (query position rpos, key position kp, query head qh)
-__device__ __forceinline__ float attn_score(const AttnForm& form, float dot, float scale, int rpos, int kp, int qh, int H) {
+// slope: the head's entry of form.dist_slope, read once per row by the caller
+__device__ __forceinline__ float attn_score(const AttnForm& form, float dot, float scale, int rpos, int kp, int qh, int H, float slope) {
   float sc = dot * scale;
   if (form.softcap > 0.f) sc = form.softcap * tanhf(sc / form.softcap);
   if (form.dist_bias) sc += form.dist_bias[(int64_t)min(rpos - kp, form.n_dist - 1) * H + qh];
+  if (form.dist_slope) sc = fmaf(-slope, (float)(rpos - kp), sc);
   return sc;
 }
 
@@ -249,12 +252,14 @@ __global__ __launch_bounds__(256) void paged_attention_kernel(
   }
   float mrun[kAttRpw][MAPS], lrun[kAttRpw][MAPS], acc[kAttRpw][MAPS][4];
   int rpos[kAttRpw], rlo[kAttRpw], rqh[kAttRpw];
+  float rsl[kAttRpw];
 #pragma unroll
   for (int i = 0; i < kAttRpw; ++i) {
     const int lr = wave + 4 * i;
     rpos[i] = lr < nrows ? positions[row0 + lr / nqh] : -1;
     rlo[i] = rpos[i] >= 0 ? attn_row_lo(form, rpos[i]) : 0;
     rqh[i] = g * per_group + qh0 + (lr < nrows ? lr % nqh : 0);
+    rsl[i] = form.dist_slope ? form.dist_slope[rqh[i]] : 0.f;
 #pragma unroll
     for (int m = 0; m < MAPS; ++m) {
       mrun[i][m] = -INFINITY;
@@ -353,7 +358,7 @@ __global__ __launch_bounds__(256) void paged_attention_kernel(
         if (act[i]) {
           const int kp_ = k0 + lane;
           const bool seen = lane < nk && kp_ <= rpos[i] && (kp_ >= rlo[i] || kp_ < form.keep_first);
-          const float sc = seen ? attn_score(form, a[i], scale, rpos[i], kp_, rqh[i], H) : -INFINITY;
+          const float sc = seen ? attn_score(form, a[i], scale, rpos[i], kp_, rqh[i], H, rsl[i]) : -INFINITY;
           const float mnew = fmaxf(mrun[i][m], wave_max(sc));
           pv = sc == -INFINITY ? 0.f : expf(sc - mnew);
           corr[i] = mrun[i][m] == -INFINITY ? 0.f : expf(mrun[i][m] - mnew);
@@ -462,6 +467,7 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
   const int rpos = lrow < nrows ? positions[row0 + lrow / nqh] : -1;      // this lane's row (as a column of S^T)
   const int rlo = rpos >= 0 ? attn_row_lo(form, rpos) : 0;
   const int lqh = g * per_group + qh0 + (lrow < nrows ? lrow % nqh : 0);
+  const float lsl = form.dist_slope ? form.dist_slope[lqh] : 0.f;
   float mrun[MAPS], lrun[MAPS];
   f32x4 o[MAPS][NCB];
 #pragma unroll
@@ -526,7 +532,7 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int kp_ = k0 + kb + 4 * lgrp + r;
-        sv[r] = (kp_ <= rpos && (kp_ >= rlo || kp_ < form.keep_first)) ? attn_score(form, sv[r], scale, rpos, kp_, lqh, H) : -INFINITY;
+        sv[r] = (kp_ <= rpos && (kp_ >= rlo || kp_ < form.keep_first)) ? attn_score(form, sv[r], scale, rpos, kp_, lqh, H, lsl) : -INFINITY;
         tmax = fmaxf(tmax, sv[r]);
       }
       tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
@@ -797,9 +803,31 @@ pegainfer_status_t pegainfer_paged_attention_masked(const float* q, const void* 
                                                     int32_t keep_first, const float* dist_bias, int32_t n_dist, const void* gate,
                                                     int64_t gate_stride, int32_t gate_kind, int32_t n_split, float* workspace,
                                                     int32_t plain, int32_t dtype, pegainfer_stream_t stream) {
+  pegainfer_attn_options o{};
+  o.maps = maps; o.lambda = lambda; o.block = block; o.sink = sink; o.head_norm = head_norm; o.norm_eps = norm_eps;
+  o.softcap = softcap; o.window = window; o.keep_first = keep_first; o.dist_bias = dist_bias; o.n_dist = n_dist;
+  o.gate = gate; o.gate_stride = gate_stride; o.gate_kind = gate_kind; o.n_split = n_split; o.workspace = workspace; o.plain = plain;
+  return pegainfer_paged_attention_opt(q, cache, page_stride, k_cache_off, v_cache_off, page_size, positions, row_entry, page_indptr,
+                                          page_ids, heads, kv_heads, dim, vdim, scale, factor, tile_row0, tile_ntok, tile_qh0, tile_nqh,
+                                          n_tiles, out, out_stride, &o, dtype, stream);
+}
+
+pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cache, int64_t page_stride, int64_t k_cache_off,
+                                                 int64_t v_cache_off, int32_t page_size, const int32_t* positions,
+                                                 const int32_t* row_entry, const int32_t* page_indptr, const int32_t* page_ids,
+                                                 int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, float scale,
+                                                 float factor, const int32_t* tile_row0, const int32_t* tile_ntok,
+                                                 const int32_t* tile_qh0, const int32_t* tile_nqh, int32_t n_tiles, void* out,
+                                                 int64_t out_stride, const pegainfer_attn_options* opt, int32_t dtype,
+                                                 pegainfer_stream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (gate_kind < 0 || gate_kind > 2 || (gate_kind && !gate)) return PK_BAD;
-  if (window < 0 || keep_first < 0 || (keep_first > 0 && window <= 0) || softcap < 0.f || (dist_bias && n_dist < 1)) return PK_BAD;
+  if (!opt) return PK_BAD;
+  const int32_t maps = opt->maps > 0 ? opt->maps : 1, block = opt->block, window = opt->window, keep_first = opt->keep_first,
+                gate_kind = opt->gate_kind, plain = opt->plain;
+  int32_t n_split = opt->n_split;
+  float* workspace = opt->workspace;
+  if (gate_kind < 0 || gate_kind > 2 || (gate_kind && !opt->gate)) return PK_BAD;
+  if (window < 0 || keep_first < 0 || (keep_first > 0 && window <= 0) || opt->softcap < 0.f || (opt->dist_bias && opt->n_dist < 1)) return PK_BAD;
   if (n_split < 1) n_split = 1;
   if (n_split > 1 && (!workspace || n_split > 64)) return PK_BAD;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || dim <= 0 || (maps != 1 && maps != 2) || maps * dim > 256 || vdim <= 0 ||
@@ -810,17 +838,18 @@ pegainfer_status_t pegainfer_paged_attention_masked(const float* q, const void* 
   const dim3 grid(n_tiles, kv_heads, n_split);
   AttnForm form;
   form.block = block;
-  form.sink = sink;
-  form.lambda = lambda;
-  form.head_norm = head_norm;
-  form.norm_eps = norm_eps;
-  form.softcap = softcap;
+  form.sink = opt->sink;
+  form.lambda = opt->lambda;
+  form.head_norm = opt->head_norm;
+  form.norm_eps = opt->norm_eps;
+  form.softcap = opt->softcap;
   form.window = window;
   form.keep_first = window > 0 ? keep_first : 0;
-  form.dist_bias = dist_bias;
-  form.n_dist = n_dist;
-  form.gate = gate;
-  form.gate_stride = gate_stride;
+  form.dist_bias = opt->dist_bias;
+  form.n_dist = opt->n_dist;
+  form.dist_slope = opt->dist_slope;
+  form.gate = opt->gate;
+  form.gate_stride = opt->gate_stride;
   form.gate_kind = gate_kind;
   bool ok = true;
   if (dtype == kDtBf16 && !plain) {   // bf16 cache: the matrix-core kernel; same tiles, same splits, same merge

@@ -15,6 +15,7 @@
 #include "pegainfer_feruzen.h"
 #include "pegainfer_ramalix.h"
 #include "pegainfer_kukulorn.h"
+#include "pegainfer_zofadra.h"
 #include "pegainfer_scheduler.h"
 
 namespace psched {
@@ -305,6 +306,7 @@ PEGAINFER_STEP_API(DuguzenApi, pegainfer_duguzen);
 PEGAINFER_STEP_API(FeruzenApi, pegainfer_feruzen);
 PEGAINFER_STEP_API(RamalixApi, pegainfer_ramalix);
 PEGAINFER_STEP_API(KukulornApi, pegainfer_kukulorn);
+PEGAINFER_STEP_API(ZofadraApi, pegainfer_zofadra);
 
 template <class Api>
 struct StepExec {
@@ -371,6 +373,7 @@ using DuguzenExec = StepExec<DuguzenApi>;
 using FeruzenExec = StepExec<FeruzenApi>;
 using RamalixExec = StepExec<RamalixApi>;
 using KukulornExec = StepExec<KukulornApi>;
+using ZofadraExec = StepExec<ZofadraApi>;
 
 struct Scheduler {
   pegainfer_executor_vtbl ex;
@@ -380,6 +383,7 @@ struct Scheduler {
   FeruzenExec* owned_fz = nullptr;
   RamalixExec* owned_rx = nullptr;
   KukulornExec* owned_kk = nullptr;
+  ZofadraExec* owned_zf = nullptr;
   Rng rng;
   std::vector<Active> active;
   std::vector<Pending> deferred;
@@ -688,6 +692,19 @@ pegainfer_sched_t pegainfer_sched_create_kukulorn(void* model, uint64_t seed, co
   s->owned_kk = e;
   return s;
 }
+pegainfer_sched_t pegainfer_sched_create_zofadra(void* model, uint64_t seed, const uint32_t* stop_tokens, int32_t n_stop) {
+  if (!model) return nullptr;
+  auto* e = new psched::ZofadraExec();
+  e->model = model;
+  for (int i = 0; i < n_stop; ++i) e->stop.insert(stop_tokens[i]);
+  pegainfer_executor_vtbl v{sizeof(pegainfer_executor_vtbl), e, &psched::ZofadraExec::page_size, &psched::ZofadraExec::max_request_pages,
+                            &psched::ZofadraExec::available_pages, &psched::ZofadraExec::is_stop_token,
+                            &psched::ZofadraExec::drop_request, &psched::ZofadraExec::execute, &psched::ZofadraExec::last_error,
+                            &psched::ZofadraExec::max_batch_size, &psched::ZofadraExec::logprobs, nullptr, nullptr};
+  Scheduler* s = static_cast<Scheduler*>(pegainfer_sched_create(&v, seed));
+  s->owned_zf = e;
+  return s;
+}
 void pegainfer_sched_destroy(pegainfer_sched_t s) {
   if (!s) return;
   delete SC(s)->owned;
@@ -696,6 +713,7 @@ void pegainfer_sched_destroy(pegainfer_sched_t s) {
   delete SC(s)->owned_fz;
   delete SC(s)->owned_rx;
   delete SC(s)->owned_kk;
+  delete SC(s)->owned_zf;
   delete SC(s);
 }
 uint64_t pegainfer_sched_submit_ex(pegainfer_sched_t s, const uint32_t* prompt_tokens, int32_t n_tokens, int32_t max_tokens,

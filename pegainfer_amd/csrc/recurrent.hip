@@ -17,46 +17,13 @@
 // steps only moves where the state passes through HBM (exactly, it is fp32 either way).
 #include "common.h"
 #include "typed.h"
+#include "recurrent_core.h"
 #include "pegainfer_kernels_blocks.h"
 
 namespace pk {
 
-constexpr int kRecTokens = 16;   // tokens staged per round
-constexpr int kRecCols = 16;     // value columns per workgroup (four per wave)
-constexpr int kRecSlices = 16;   // lanes that share one column
-
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.0f ? x : log1pf(expf(x)); }
 __device__ __forceinline__ float logsigmoid_f(float x) { return fminf(x, 0.0f) - log1pf(expf(-fabsf(x))); }
-
-// One round's q | k | v values, fetched into registers (issue) and put into LDS later (land).  Thread t serves token t / 16
-// of the round: values t % 16, t % 16 + 16, ... of its query and key and column t % 16 of its value, so which register holds
-// what is known at compile time and neighbouring lanes read neighbouring addresses.
-template <int NS>
-struct RoundFetch {
-  static constexpr int DP = kRecSlices * NS;
-  float q[NS], k[NS], v;
-  template <typename LoadQ, typename LoadK, typename LoadV>
-  __device__ __forceinline__ void issue(int tc, int tid, int dim, LoadQ&& lq, LoadK&& lk, LoadV&& lv) {
-    const int tt = tid >> 4, part = tid & 15;
-    const bool live = tt < tc;
-#pragma unroll
-    for (int j = 0; j < NS; ++j) {
-      const int d = part + 16 * j;
-      q[j] = live && d < dim ? lq(tt, d) : 0.f;
-      k[j] = live && d < dim ? lk(tt, d) : 0.f;
-    }
-    v = live ? lv(tt, part) : 0.f;
-  }
-  __device__ __forceinline__ void land(int tid, float (*s_q)[DP], float (*s_k)[DP], float (*s_v)[kRecCols]) {
-    const int tt = tid >> 4, part = tid & 15;
-#pragma unroll
-    for (int j = 0; j < NS; ++j) {
-      s_q[tt][part + 16 * j] = q[j];
-      s_k[tt][part + 16 * j] = k[j];
-    }
-    s_v[tt][part] = v;
-  }
-};
 
 // Per row, before the recurrence: q and k heads made unit vectors in place (x / sqrt(sum(x^2) + 1e-6), q also * dim^-1/2),
 // gates[row] = [g: heads | beta: heads].  One workgroup per row, a wave per head.
@@ -375,17 +342,6 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(const float* __restrict__
     const int d = r * NS + i;
     if (d < dim && col < vdim) S_g[(int64_t)d * vdim + col] = S[i];
   }
-}
-
-template <typename F>
-inline bool by_slices(int dim, F&& fn) {
-  if (dim <= 16) fn(std::integral_constant<int, 1>());
-  else if (dim <= 32) fn(std::integral_constant<int, 2>());
-  else if (dim <= 64) fn(std::integral_constant<int, 4>());
-  else if (dim <= 128) fn(std::integral_constant<int, 8>());
-  else if (dim <= 256) fn(std::integral_constant<int, 16>());
-  else return false;
-  return true;
 }
 
 }  // namespace pk

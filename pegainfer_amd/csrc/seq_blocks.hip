@@ -147,15 +147,6 @@ __global__ __launch_bounds__(256) void time_conv_commit_kernel(const I* __restri
   }
 }
 
-// four consecutive values of a row, widened / rounded at the edges
-__device__ __forceinline__ void ld4(const float* p, float* o) { const f32x4 v = *reinterpret_cast<const f32x4*>(p); o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w; }
-__device__ __forceinline__ void ld4(const uint16_t* p, float* o) {
-  const u32x2 v = *reinterpret_cast<const u32x2*>(p);
-  o[0] = bf_lo(v.x); o[1] = bf_hi(v.x); o[2] = bf_lo(v.y); o[3] = bf_hi(v.y);
-}
-__device__ __forceinline__ void st4(float* p, const float* o) { *reinterpret_cast<f32x4*>(p) = f32x4{o[0], o[1], o[2], o[3]}; }
-__device__ __forceinline__ void st4(uint16_t* p, const float* o) { *reinterpret_cast<u32x2*>(p) = u32x2{pack_bf2(o[0], o[1]), pack_bf2(o[2], o[3])}; }
-
 // x_in, x_out and mix_out may name the same memory (the stream is updated in place): an element is read, then written, by
 // the same thread, and nothing else of those buffers is touched.  VEC: rows and groups are multiples of four values and every
 // pointer is 16-byte aligned - four values per load.
@@ -239,6 +230,31 @@ __global__ __launch_bounds__(256) void clamp_glu_rows_kernel(const A* __restrict
 }
 
 // one wave per (row, head)
+// The same for heads wider than a wave should walk alone (one norm over a whole row, say): a workgroup per (row, head).
+template <typename A>
+__global__ __launch_bounds__(256) void wide_rms_gate_kernel(const float* __restrict__ o, const A* __restrict__ w, int w_per_head,
+                                                            const A* __restrict__ gate, int64_t gate_stride, int gate_kind, float factor,
+                                                            float eps, A* __restrict__ out, int64_t out_stride, int heads, int vdim,
+                                                            int gate_first) {
+  __shared__ float red[4];
+  const int row = blockIdx.x, h = blockIdx.y;
+  const float* p = o + ((int64_t)row * heads + h) * vdim;
+  const A* gr = gate + (int64_t)row * gate_stride + (int64_t)h * vdim;
+  const A* wr = w + (w_per_head ? (int64_t)h * vdim : 0);
+  A* dst = out + (int64_t)row * out_stride + (int64_t)h * vdim;
+  auto act = [&](int i) {
+    const float z = ld(gr + i);
+    return gate_kind == 0 ? silu_f(z) : sigmoid_f(z);
+  };
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < vdim; i += 256) {
+    const float v = gate_first ? p[i] * act(i) : p[i];
+    ss = fmaf(v, v, ss);
+  }
+  const float sc = factor / sqrtf(block_sum<4>(ss, red) / (float)vdim + eps);
+  for (int i = threadIdx.x; i < vdim; i += 256) st(dst + i, p[i] * act(i) * sc * ld(wr + i));
+}
+
 template <typename A>
 __global__ __launch_bounds__(256) void head_rms_gate_kernel(const float* __restrict__ o, const A* __restrict__ w, int w_per_head,
                                                             const A* __restrict__ gate, int64_t gate_stride, int gate_kind,
@@ -685,6 +701,13 @@ pegainfer_status_t pegainfer_head_gate_rms(const float* o, const void* w, int32_
   const int blocks = ceil_div((long)rows * heads, 4);
   if (!by_dtype(dtype, [&](auto* t) {
         using A = std::remove_pointer_t<decltype(t)>;
+        if (vdim > 512 && heads <= 65535) {
+          wide_rms_gate_kernel<A><<<dim3(rows, heads), 256, 0, as_stream(stream)>>>(o, static_cast<const A*>(w), w_per_head,
+                                                                                   static_cast<const A*>(gate), gate_stride, gate_kind,
+                                                                                   factor, eps, static_cast<A*>(out), out_stride, heads,
+                                                                                   vdim, gate_first);
+          return;
+        }
         head_rms_gate_kernel<A><<<blocks, 256, 0, as_stream(stream)>>>(o, static_cast<const A*>(w), w_per_head,
                                                                        static_cast<const A*>(gate), gate_stride, gate_kind,
                                                                        factor, eps, static_cast<A*>(out), out_stride, heads,

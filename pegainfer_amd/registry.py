@@ -1,8 +1,8 @@
 """Model registry: which engine serves a model folder, decided by its config.json.
 
 Hugging Face style configurations name their family in ``model_type`` / ``architectures`` (Qwen3, Qwen3.5); Duguzen,
-Feruzen, Ramalix and Kukulorn name it in ``architecture``.  ``load_engine`` builds the engine with the weights of the folder; ``scheduler_for`` puts the
-continuous-batching scheduler (include/pegainfer_scheduler.h) on top of it.
+Feruzen, Ramalix, Kukulorn and Zofadra name it in ``architecture``.  ``load_engine`` builds the engine with the weights of the
+folder; ``scheduler_for`` puts the continuous-batching scheduler (include/pegainfer_scheduler.h) on top of it.
 """
 import json
 import os
@@ -47,6 +47,12 @@ def _kukulorn(model_dir, cfg, **kw):
                                           dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
 
 
+def _zofadra(model_dir, cfg, **kw):
+    from .zofadra import ZofadraEngine
+    return ZofadraEngine.from_pretrained(model_dir, max_tokens=kw.get("max_tokens", 4096), max_requests=kw.get("max_requests", 8),
+                                         dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
+
+
 # family -> (loader, dtypes it can be served in)
 REGISTRY = {
     "qwen3": (_qwen3, ("bfloat16",)),
@@ -55,12 +61,13 @@ REGISTRY = {
     "feruzen": (_feruzen, ("bfloat16", "float32")),
     "ramalix": (_ramalix, ("bfloat16", "float32")),
     "kukulorn": (_kukulorn, ("bfloat16", "float32")),
+    "zofadra": (_zofadra, ("bfloat16", "float32")),
 }
 
 
 def family_of(cfg):
     """the registry key of a parsed config.json, or None"""
-    if str(cfg.get("architecture", "")).lower() in ("duguzen", "feruzen", "ramalix", "kukulorn"):
+    if str(cfg.get("architecture", "")).lower() in ("duguzen", "feruzen", "ramalix", "kukulorn", "zofadra"):
         return str(cfg["architecture"]).lower()
     names = [str(cfg.get("model_type", ""))] + [str(a) for a in cfg.get("architectures", [])]
     low = " ".join(names).lower()
