@@ -497,3 +497,123 @@ def ssd_scan(xbc_f32, proj, dt_off, A_log, dt_bias, D, state, heads, groups, n_s
                                       _p(state), state.stride(0), _p(y), heads, groups, n_state, vdim, _p(rg.entry_row0), _p(rg.entry_slot),
                                       rg.n, _dt(proj), _stream()), "ssd_scan")
     return y
+
+
+# ---- several residual streams, latent attention with a query latent, a linear distance bias, constant decays ----
+def _struct(name, fields):
+    kinds = {"p": ctypes.c_void_p, "i": ctypes.c_int32, "l": ctypes.c_int64, "f": ctypes.c_float}
+    return type(name, (ctypes.Structure,), {"_fields_": [(n, kinds[k]) for k, ns in fields for n in ns.split()]})
+
+
+AttnOptions = _struct("AttnOptions", [("i", "maps"), ("f", "lambda_"), ("i", "block"), ("p", "sink"), ("i", "head_norm"), ("f", "norm_eps softcap"),
+                                      ("i", "window keep_first"), ("p", "dist_bias"), ("i", "n_dist"), ("p", "dist_slope gate"),
+                                      ("l", "gate_stride"), ("i", "gate_kind n_split"), ("p", "workspace"), ("i", "plain")])
+LatentPrepDesc = _struct("LatentPrepDesc", [("p", "dkv"), ("l", "dkv_stride"), ("p", "c_norm_w ql"), ("l", "ql_stride"), ("p", "ql_norm_w ql_out"),
+                                            ("i", "q_rank"), ("p", "q"), ("l", "q_stride"), ("p", "qc"), ("f", "eps"), ("p", "inv_freq"),
+                                            ("i", "rot_dims rot_layout"), ("p", "positions token_req page_indptr page_ids cache"),
+                                            ("l", "page_stride layer_off"), ("i", "page_size heads nope rot rank n_tokens dtype")])
+StreamMixDesc = _struct("StreamMixDesc", [("p", "x_in embed token_ids"), ("f", "embed_scale"), ("p", "row_index y"), ("l", "y_row_stride"),
+                                          ("p", "mix out_w"), ("f", "mult"), ("p", "x_out sum_out read_w gain n_out"), ("f", "eps"),
+                                          ("i", "norm_kind streams d rows dtype")])
+DecayAttentionDesc = _struct("DecayAttentionDesc", [("p", "proj"), ("l", "proj_stride q_off k_off v_off"), ("i", "silu"), ("p", "decay_pow"),
+                                                    ("i", "pow_n"), ("p", "state"), ("l", "slot_stride"), ("p", "o"), ("i", "heads dim vdim"),
+                                                    ("p", "entry_row0 entry_slot"), ("i", "n_entries scan_max"), ("p", "chunk_row0 chunk_rows"),
+                                                    ("i", "n_chunks"), ("p", "long_chunk0 long_slot"), ("i", "n_long"), ("p", "workspace"),
+                                                    ("i", "dtype")])
+
+
+def paged_attention_opt(q, cache, page_stride, k_off, v_off, page_size, rg, page_indptr, page_ids, kv_heads, vdim, scale, window=0,
+                        dist_slope=None, softcap=0.0, n_split=1, plain=False):
+    """q fp32 [rows, heads, dim]; dist_slope fp32 [heads]: slope * distance is taken off the scores"""
+    T, H, dim = q.shape
+    out = torch.empty((T, H * vdim), dtype=cache.dtype, device=q.device)
+    t = attention_tiles(rg.lens, H // kv_heads, q.device)
+    ws = None
+    if n_split > 1:
+        ws = torch.empty(ffi.lib().pegainfer_paged_attention_workspace(t[0].numel(), kv_heads, vdim, 1, n_split), dtype=torch.float32,
+                         device=q.device)
+    o = AttnOptions(window=int(window), dist_slope=_p(dist_slope), softcap=float(softcap), n_split=int(n_split), workspace=_p(ws),
+                    plain=int(bool(plain)))
+    _chk(ffi.lib().pegainfer_paged_attention_opt(_p(q), _p(cache), page_stride, k_off, v_off, page_size, _p(rg.positions), _p(rg.row_entry),
+                                                 _p(page_indptr), _p(page_ids), H, kv_heads, dim, vdim, float(scale), 1.0, _p(t[0]), _p(t[1]),
+                                                 _p(t[2]), _p(t[3]), t[0].numel(), _p(out), out.stride(0), ctypes.addressof(o), _dt(cache),
+                                                 _stream()), "paged_attention_opt")
+    return out
+
+
+def latent_prep_form(rg, page_indptr, page_ids, cache, page_stride, layer_off, page_size, heads, nope, rot, rank, eps, inv_freq, pairs,
+                     dkv=None, c_norm_w=None, ql=None, ql_norm_w=None, q=None, qc=None):
+    """dkv [rows, rank + rot] -> cache; ql [rows, q_rank] -> returned normed; q [rows, heads * (nope + rot)] -> qc[:, :, rank:]"""
+    T = rg.positions.numel()
+    out = torch.empty((T, ql.shape[1]), dtype=cache.dtype, device=cache.device) if ql is not None else None
+    d = LatentPrepDesc(eps=float(eps), inv_freq=_p(inv_freq), rot_dims=rot, rot_layout=0 if pairs else 1, positions=_p(rg.positions),
+                       token_req=_p(rg.row_entry), page_indptr=_p(page_indptr), page_ids=_p(page_ids), cache=_p(cache),
+                       page_stride=page_stride, layer_off=layer_off, page_size=page_size, heads=heads, nope=nope, rot=rot, rank=rank,
+                       n_tokens=T, dtype=_dt(cache))
+    if dkv is not None:
+        d.dkv, d.dkv_stride, d.c_norm_w = _p(dkv), dkv.stride(0), _p(c_norm_w)
+    if ql is not None:
+        d.ql, d.ql_stride, d.ql_norm_w, d.ql_out, d.q_rank = _p(ql), ql.stride(0), _p(ql_norm_w), _p(out), ql.shape[1]
+    if q is not None:
+        d.q, d.q_stride, d.qc = _p(q), q.stride(0), _p(qc)
+    _chk(ffi.lib().pegainfer_latent_prep_form(ctypes.addressof(d), _stream()), "latent_prep_form")
+    return out
+
+
+def latent_attention_dealt(qc, cache, page_stride, layer_off, page_size, rg, page_indptr, page_ids, rank, rot, scale, n_split=1, tiles=None):
+    """qc fp32 [T, heads, rank + rot] -> o_lat fp32 [T, heads, rank]; the keys dealt to n_split workgroups per row (tile)"""
+    T, H, _ = qc.shape
+    o = torch.empty((T, H, rank), dtype=torch.float32, device=qc.device)
+    ws = torch.empty(max(1, int(ffi.lib().pegainfer_latent_attention_dealt_workspace(T, H, rank, n_split))), dtype=torch.float32, device=qc.device)
+    t0, tr = tiles if tiles is not None else (None, None)
+    _chk(ffi.lib().pegainfer_latent_attention_dealt(_p(qc), _p(o), _p(cache), page_stride, layer_off, page_size, _p(rg.positions),
+                                                    _p(rg.row_entry), _p(page_indptr), _p(page_ids), H, rank, rot, float(scale), T, n_split,
+                                                    _p(ws), _p(t0), _p(tr), 0 if t0 is None else t0.numel(), _dt(cache), _stream()),
+         "latent_attention_dealt")
+    return o
+
+
+def stream_mix(x, streams, d, dtype, y=None, mix=None, out_w=None, mult=1.0, read_w=None, gain=None, eps=1e-5, layer_norm=True, embed=None,
+               token_ids=None, embed_scale=1.0, row_index=None, want_sum=False, keep=True):
+    """x fp32 [rows, streams, d] or None (then embed[token_ids] * embed_scale) -> (new streams or None, normed row or None, sum or None)"""
+    rows = row_index.numel() if row_index is not None else (token_ids.numel() if x is None else x.shape[0])
+    new = torch.empty((rows, streams, d), dtype=torch.float32, device="cuda") if keep else None
+    n = torch.empty((rows, d), dtype=dtype, device="cuda") if gain is not None else None
+    sm = torch.empty((rows, d), dtype=torch.float32, device="cuda") if want_sum else None
+    q = StreamMixDesc(x_in=_p(x), embed=_p(embed), token_ids=_p(token_ids), embed_scale=float(embed_scale), row_index=_p(row_index), y=_p(y),
+                      y_row_stride=y.stride(0) if y is not None else 0, mix=_p(mix), out_w=_p(out_w), mult=float(mult), x_out=_p(new),
+                      sum_out=_p(sm), read_w=_p(read_w), gain=_p(gain), n_out=_p(n), eps=float(eps), norm_kind=int(bool(layer_norm)),
+                      streams=streams, d=d, rows=rows, dtype=0 if dtype == torch.bfloat16 else 1)
+    _chk(ffi.lib().pegainfer_stream_mix(ctypes.addressof(q), _stream()), "stream_mix")
+    return new, n, sm
+
+
+def decay_attention(proj, offs, decay, state, heads, dim, vdim, rg, silu=True, scan_max=0):
+    """proj rows [.. q at offs[0] | k at offs[1] | v at offs[2] ..]; decay: one number per head; state fp32 [slots, heads * dim * vdim];
+    scan_max > 0: entries of more rows take the chunk form -> fp32 [rows, heads * vdim]"""
+    C = 64
+    pw = torch.tensor([[float(g) ** n for n in range(C + 1)] for g in decay], dtype=torch.float32, device=proj.device)
+    o = torch.empty((proj.shape[0], heads * vdim), dtype=torch.float32, device=proj.device)
+    d = DecayAttentionDesc(proj=_p(proj), proj_stride=proj.stride(0), q_off=offs[0], k_off=offs[1], v_off=offs[2], silu=int(bool(silu)),
+                           decay_pow=_p(pw), pow_n=C + 1, state=_p(state), slot_stride=state.stride(0), o=_p(o), heads=heads, dim=dim,
+                           vdim=vdim, entry_row0=_p(rg.entry_row0), entry_slot=_p(rg.entry_slot), n_entries=len(rg.lens), dtype=_dt(proj))
+    keep = []
+    if scan_max > 0:
+        row0, rows, first, slot, at = [], [], [0], [], 0
+        slots = rg.entry_slot.tolist()
+        for i, n in enumerate(rg.lens):
+            if n > scan_max:
+                for k in range(0, n, C):
+                    row0.append(at + k)
+                    rows.append(min(C, n - k))
+                first.append(len(row0))
+                slot.append(slots[i])
+            at += n
+        if slot:
+            keep = [torch.tensor(v, dtype=torch.int32, device=proj.device) for v in (row0, rows, first, slot)]
+            keep.append(torch.empty(int(ffi.lib().pegainfer_decay_attention_workspace(len(row0), heads, dim, vdim)), dtype=torch.float32,
+                                    device=proj.device))
+            d.scan_max, d.chunk_row0, d.chunk_rows, d.n_chunks = scan_max, _p(keep[0]), _p(keep[1]), len(row0)
+            d.long_chunk0, d.long_slot, d.n_long, d.workspace = _p(keep[2]), _p(keep[3]), len(slot), _p(keep[4])
+    _chk(ffi.lib().pegainfer_decay_attention(ctypes.addressof(d), _stream()), "decay_attention")
+    return o
