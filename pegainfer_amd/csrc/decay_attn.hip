@@ -55,15 +55,15 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(DecayIn<A> in, const fl
   auto fetch = [&](int t0) {
     const A* base = in.proj + (int64_t)(row0 + t0) * in.stride;
     const A *qb = base + in.q_off + (int64_t)h * dim, *kb = base + in.k_off + (int64_t)h * dim, *vb = base + in.v_off + (int64_t)h * vdim + col0;
-    nxt.issue(min(kRecTokens, len - t0), tid, dim, [=](int tt, int d) { return in.act(ld(qb + (int64_t)tt * in.stride + d)); },
-              [=](int tt, int d) { return in.act(ld(kb + (int64_t)tt * in.stride + d)); },
-              [=](int tt, int c) { return col0 + c < vdim ? in.act(ld(vb + (int64_t)tt * in.stride + c)) : 0.f; });
+    nxt.issue(min(kRecTokens, len - t0), tid, dim, [=](int tt, int d) { return ld(qb + (int64_t)tt * in.stride + d); },
+              [=](int tt, int d) { return ld(kb + (int64_t)tt * in.stride + d); },
+              [=](int tt, int c) { return col0 + c < vdim ? ld(vb + (int64_t)tt * in.stride + c) : 0.f; });
   };
   fetch(0);
   for (int t0 = 0; t0 < len; t0 += kRecTokens) {
     const int tc = min(kRecTokens, len - t0);
     __syncthreads();
-    nxt.land(tid, s_q, s_k, s_v);
+    nxt.land(tid, s_q, s_k, s_v, [=](float x) { return in.act(x); });
     __syncthreads();
     if (t0 + kRecTokens < len) fetch(t0 + kRecTokens);
     float okeep = 0.f;
@@ -92,27 +92,37 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(DecayIn<A> in, const fl
   }
 }
 
-// A chunk's rows of one head into LDS (fp32, activated), rows past `n` and columns past `dim` as zeros; four threads per row.
-template <typename A>
+// A chunk's rows of one head into LDS (fp32, activated), rows past `n` and columns past `dim` as zeros; TPR threads per row, four
+// loads of eight values in flight per thread.
+template <int TPR, typename A>
 __device__ __forceinline__ void stage_rows(const DecayIn<A>& in, int64_t off, int row0, int n, int dim, int padded, float* dst, int stride,
                                            const float* row_factor, int tid) {
-  const int j = tid >> 2, sub = tid & 3;
-  const A* src = in.proj + (int64_t)(row0 + j) * in.stride + off;
-  const float f = j < n && row_factor ? row_factor[j] : 1.0f;
+  const int j = tid / TPR, sub = tid % TPR;
+  const A* src = in.proj + (int64_t)(row0 + min(j, n - 1)) * in.stride + off;
+  const float f = j < n ? (row_factor ? row_factor[j] : 1.0f) : 0.f;
   const bool vec = (dim & 7) == 0 && (off & 7) == 0 && (in.stride & 7) == 0 && aligned16(in.proj);
   float* d = dst + j * stride;
-  for (int c = sub * 8; c < padded; c += 32) {
-    float t[8];
-    if (j < n && vec && c < dim) {
-      Vec8<A>::load(src + c, t);
+  for (int c0 = sub * 8; c0 < padded; c0 += 32 * TPR) {
+    float t[4][8];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) t[u] = in.act(t[u]) * f;
-    } else {
+    for (int k = 0; k < 4; ++k) {
+      const int c = c0 + 8 * TPR * k;
+      if (vec) {
+        Vec8<A>::load(src + (c < dim ? c : 0), t[k]);      // always in bounds; what lies past dim or n becomes zero below
+      } else {
 #pragma unroll
-      for (int u = 0; u < 8; ++u) t[u] = j < n && c + u < dim ? in.act(ld(src + c + u)) * f : 0.f;
+        for (int u = 0; u < 8; ++u) t[k][u] = ld(src + (c + u < dim ? c + u : 0));
+      }
     }
-    *reinterpret_cast<f32x4*>(d + c) = f32x4{t[0], t[1], t[2], t[3]};
-    *reinterpret_cast<f32x4*>(d + c + 4) = f32x4{t[4], t[5], t[6], t[7]};
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int c = c0 + 8 * TPR * k;
+      if (c >= padded) break;
+#pragma unroll
+      for (int u = 0; u < 8; ++u) t[k][u] = j < n && c + u < dim ? in.act(t[k][u]) * f : 0.f;
+      *reinterpret_cast<f32x4*>(d + c) = f32x4{t[k][0], t[k][1], t[k][2], t[k][3]};
+      *reinterpret_cast<f32x4*>(d + c + 4) = f32x4{t[k][4], t[k][5], t[k][6], t[k][7]};
+    }
   }
 }
 
@@ -121,10 +131,12 @@ __device__ __forceinline__ void stage_rows(const DecayIn<A>& in, int64_t off, in
 __host__ __device__ constexpr int pad16(int n) { return (n + 15) & ~15; }
 __host__ __device__ constexpr int stride_rows4(int n) { return pad16(n) % 32 == 0 ? pad16(n) + 16 : pad16(n); }
 __host__ __device__ constexpr int stride_rows16(int n) { return pad16(n) + 4; }
+// value columns of the workspace and of the staged values: what the kernels' 16-column blocks cover
+__host__ __device__ constexpr int pad_values(int vdim) { return vdim <= 32 ? 32 : vdim <= 64 ? 64 : vdim <= 128 ? 128 : 256; }
 
-// U_c[d][col] = sum_i g^(n-1-i) k_i[d] v_i[col]; one workgroup per (chunk, head), a wave per 16 rows of U, four column blocks at a time
-template <typename A>
-__global__ __launch_bounds__(256) void decay_chunk_sum_kernel(DecayIn<A> in, const float* __restrict__ decay_pow, int pow_n,
+// U_c[d][col] = sum_i g^(n-1-i) k_i[d] v_i[col]; one workgroup per (chunk, head), a wave per block of 16 rows x (16 NB) columns of U
+template <typename A, int NB>
+__global__ __launch_bounds__(512) void decay_chunk_sum_kernel(DecayIn<A> in, const float* __restrict__ decay_pow, int pow_n,
                                                               float* __restrict__ ws, int H, int dim, int vdim,
                                                               const int32_t* __restrict__ chunk_row0,
                                                               const int32_t* __restrict__ chunk_rows) {
@@ -132,32 +144,32 @@ __global__ __launch_bounds__(256) void decay_chunk_sum_kernel(DecayIn<A> in, con
   __shared__ float s_f[kDecayChunk];
   const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
   const int row0 = chunk_row0[c], n = chunk_rows[c];
-  const int dp = pad16(dim), vp = pad16(vdim), sk = stride_rows4(dim), sv = stride_rows4(vdim);
+  const int dp = pad16(dim), vp = pad_values(vdim), sk = stride_rows4(dim), sv = stride_rows4(vp);
   float *s_k = sm, *s_v = sm + kDecayChunk * sk;
   if (tid < kDecayChunk) s_f[tid] = tid < n ? decay_pow[(int64_t)h * pow_n + n - 1 - tid] : 0.f;
   __syncthreads();
-  stage_rows(in, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sk, s_f, tid);
-  stage_rows(in, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid);
+  stage_rows<8>(in, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sk, s_f, tid);
+  stage_rows<8>(in, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid);
   __syncthreads();
   float* U = ws + ((int64_t)c * H + h) * dp * vp;
-  const int steps = (n + 3) >> 2;
-  for (int d0 = wave * 16; d0 < dp; d0 += 64)
-    for (int c0 = 0; c0 < vp; c0 += 64) {
-      f32x4 acc[4];
+  const int steps = (n + 3) >> 2, col_blocks = vp / (16 * NB), blocks = (dp >> 4) * col_blocks;
+  for (int blk = wave; blk < blocks; blk += 8) {
+    const int d0 = (blk / col_blocks) * 16, c0 = (blk % col_blocks) * 16 * NB;
+    f32x4 acc[NB];
 #pragma unroll
-      for (int b = 0; b < 4; ++b) acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
-      for (int i = 0; i < steps; ++i) {
-        const float a = s_k[(4 * i + lg) * sk + d0 + l15];
+    for (int b = 0; b < NB; ++b) acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const float *ka = s_k + lg * sk + d0 + l15, *vb = s_v + lg * sv + c0 + l15;
+#pragma unroll 2
+    for (int i = 0; i < steps; ++i) {
+      const float a = ka[4 * i * sk];
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
-          if (c0 + 16 * b < vp) acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, s_v[(4 * i + lg) * sv + c0 + 16 * b + l15], acc[b], 0, 0, 0);
-      }
-#pragma unroll
-      for (int b = 0; b < 4; ++b)
-        if (c0 + 16 * b < vp)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) U[(int64_t)(d0 + 4 * lg + r) * vp + c0 + 16 * b + l15] = acc[b][r];
+      for (int b = 0; b < NB; ++b) acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, vb[4 * i * sv + 16 * b], acc[b], 0, 0, 0);
     }
+#pragma unroll
+    for (int b = 0; b < NB; ++b)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) U[(int64_t)(d0 + 4 * lg + r) * vp + c0 + 16 * b + l15] = acc[b][r];
+  }
 }
 
 // One thread per element of the state: through the entry's chunks, the state before each left in U's place.
@@ -168,7 +180,7 @@ __global__ __launch_bounds__(256) void decay_chunk_state_kernel(const float* __r
                                                                 const int32_t* __restrict__ long_slot) {
   const int e = blockIdx.z, h = blockIdx.y, i = blockIdx.x * 256 + threadIdx.x;
   if (i >= dim * vdim) return;
-  const int dp = pad16(dim), vp = pad16(vdim);
+  const int dp = pad16(dim), vp = pad_values(vdim);
   float* sp = state + (int64_t)long_slot[e] * slot_stride + (int64_t)h * dim * vdim + i;
   const int64_t cs = (int64_t)H * dp * vp;
   float* u = ws + (int64_t)h * dp * vp + (int64_t)(i / vdim) * vp + i % vdim;
@@ -188,68 +200,79 @@ __global__ __launch_bounds__(256) void decay_chunk_state_kernel(const float* __r
   *sp = S;
 }
 
-// NB: 16-column blocks of the values (vdim <= 16 NB); a wave owns 16 of the chunk's rows
+// Eight waves: wave w takes 16 rows of the chunk and half of the value columns (NB blocks of 16); the two halves take the row blocks
+// in opposite order, so that the two waves of a SIMD have the same number of key blocks between them.
 template <typename A, int NB>
-__global__ __launch_bounds__(256) void decay_chunk_out_kernel(DecayIn<A> in, const float* __restrict__ decay_pow, int pow_n,
+__global__ __launch_bounds__(512) void decay_chunk_out_kernel(DecayIn<A> in, const float* __restrict__ decay_pow, int pow_n,
                                                               const float* __restrict__ ws, float* __restrict__ o, int H, int dim,
                                                               int vdim, const int32_t* __restrict__ chunk_row0,
                                                               const int32_t* __restrict__ chunk_rows) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   __shared__ float s_pow[kDecayChunk + 1];
+  constexpr int vp = 32 * NB, sv = stride_rows16(vp);
   const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
   const int row0 = chunk_row0[c], n = chunk_rows[c];
-  const int dp = pad16(dim), vp = pad16(vdim), sq = stride_rows16(dim), sv = stride_rows16(vdim);
+  const int dp = pad16(dim), sq = stride_rows16(dim);
   float *s_q = sm, *s_k = s_q + kDecayChunk * sq, *s_v = s_k + kDecayChunk * sq;
+  const int half = wave >> 2, rb = half ? 3 - (wave & 3) : wave & 3, i0 = rb * 16, c0 = half * 16 * NB;
   if (tid <= kDecayChunk) s_pow[tid] = tid <= n ? decay_pow[(int64_t)h * pow_n + tid] : 0.f;
-  stage_rows(in, in.q_off + (int64_t)h * dim, row0, n, dim, dp, s_q, sq, nullptr, tid);
-  stage_rows(in, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sq, nullptr, tid);
-  stage_rows(in, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid);
+  stage_rows<8>(in, in.q_off + (int64_t)h * dim, row0, n, dim, dp, s_q, sq, nullptr, tid);
+  stage_rows<8>(in, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sq, nullptr, tid);
+  stage_rows<8>(in, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid);
   __syncthreads();
-  const int i0 = wave * 16;
   if (i0 >= n) return;                               // no barrier follows
   const int my_i = i0 + l15;                         // the query this lane holds scores of
   f32x4 acc[NB];
 #pragma unroll
   for (int b = 0; b < NB; ++b) acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
   const float* qr = s_q + my_i * sq + lg;
-  {   // what the tokens before the chunk left
+  {   // what the tokens before the chunk left; rows dim .. dp - 1 and columns vdim .. vp - 1 of the state before a chunk are zeros
     const float f = s_pow[min(my_i + 1, n)];         // rows past n are not stored
-    const float* S = ws + ((int64_t)c * H + h) * dp * vp + (int64_t)lg * vp + l15;
-    for (int d0 = 0; d0 < dp; d0 += 16) {            // rows dim .. dp - 1 of the state before a chunk are zeros
-      float sv4[4][NB];
+    const float* S = ws + ((int64_t)c * H + h) * dp * vp + (int64_t)lg * vp + c0 + l15;
+    constexpr int U = NB <= 4 ? 4 : 2;               // steps whose state values are fetched together, one group ahead of its use
+    float cur[U][NB], nxt[U][NB];
+    auto fetch = [&](int d0, float (*t)[NB]) {
 #pragma unroll
-      for (int u = 0; u < 4; ++u)
+      for (int u = 0; u < U; ++u)
 #pragma unroll
-        for (int b = 0; b < NB; ++b) sv4[u][b] = 16 * b < vp ? S[(int64_t)(d0 + 4 * u) * vp + 16 * b] : 0.f;
+        for (int b = 0; b < NB; ++b) t[u][b] = S[(int64_t)(d0 + 4 * u) * vp + 16 * b];
+    };
+    fetch(0, cur);
+    for (int d0 = 0; d0 < dp; d0 += 4 * U) {
+      fetch(min(d0 + 4 * U, dp - 4 * U), nxt);
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
+      for (int u = 0; u < U; ++u) {
         const float a = qr[d0 + 4 * u] * f;
 #pragma unroll
-        for (int b = 0; b < NB; ++b)
-          if (16 * b < vp) acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, sv4[u][b], acc[b], 0, 0, 0);
+        for (int b = 0; b < NB; ++b) acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, cur[u][b], acc[b], 0, 0, 0);
       }
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int b = 0; b < NB; ++b) cur[u][b] = nxt[u][b];
     }
   }
-  for (int jb = 0; jb <= wave; ++jb) {               // the chunk's own tokens, 16 keys at a time
-    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+  for (int jb = 0; jb <= rb; ++jb) {                 // the chunk's own tokens, 16 keys at a time
+    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0, s2 = s0, s3 = s0;
     const float* kr = s_k + (jb * 16 + l15) * sq + lg;
-    for (int d = 0; d < dp; d += 8) {
+    for (int d = 0; d < dp; d += 16) {
       s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[d], qr[d], s0, 0, 0, 0);
       s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[d + 4], qr[d + 4], s1, 0, 0, 0);
+      s2 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[d + 8], qr[d + 8], s2, 0, 0, 0);
+      s3 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[d + 12], qr[d + 12], s3, 0, 0, 0);
     }
-    s0 += s1;
+    s0 = (s0 + s1) + (s2 + s3);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int j = jb * 16 + 4 * lg + r;
       const float p = j <= my_i ? s0[r] * s_pow[min(my_i - j, n)] : 0.f;
 #pragma unroll
-      for (int b = 0; b < NB; ++b)
-        if (16 * b < vp) acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(p, s_v[j * sv + 16 * b + l15], acc[b], 0, 0, 0);
+      for (int b = 0; b < NB; ++b) acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(p, s_v[j * sv + c0 + 16 * b + l15], acc[b], 0, 0, 0);
     }
   }
 #pragma unroll
   for (int b = 0; b < NB; ++b) {
-    const int col = 16 * b + l15;
+    const int col = c0 + 16 * b + l15;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = i0 + 4 * lg + r;
@@ -258,8 +281,8 @@ __global__ __launch_bounds__(256) void decay_chunk_out_kernel(DecayIn<A> in, con
   }
 }
 
-static size_t decay_sum_lds(int dim, int vdim) { return (size_t)kDecayChunk * (stride_rows4(dim) + stride_rows4(vdim)) * sizeof(float); }
-static size_t decay_out_lds(int dim, int vdim) { return (size_t)kDecayChunk * (2 * stride_rows16(dim) + stride_rows16(vdim)) * sizeof(float); }
+static size_t decay_sum_lds(int dim, int vdim) { return (size_t)kDecayChunk * (stride_rows4(dim) + stride_rows4(pad_values(vdim))) * sizeof(float); }
+static size_t decay_out_lds(int dim, int vdim) { return (size_t)kDecayChunk * (2 * stride_rows16(dim) + stride_rows16(pad_values(vdim))) * sizeof(float); }
 constexpr size_t kLdsMost = 159 * 1024;              // beside the kernels' static tables
 
 }  // namespace pk
@@ -272,7 +295,7 @@ int32_t pegainfer_decay_attention_chunked_ok(int32_t dim, int32_t vdim) {
 }
 
 int64_t pegainfer_decay_attention_workspace(int32_t n_chunks, int32_t heads, int32_t dim, int32_t vdim) {
-  return (int64_t)n_chunks * heads * pad16(dim) * pad16(vdim);
+  return (int64_t)n_chunks * heads * pad16(dim) * pad_values(vdim);
 }
 
 pegainfer_status_t pegainfer_decay_attention(const pegainfer_decay_attention_desc* q, pegainfer_stream_t stream) {
@@ -303,18 +326,22 @@ pegainfer_status_t pegainfer_decay_attention(const pegainfer_decay_attention_des
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
       return bytes;
     };
-    decay_chunk_sum_kernel<A><<<dim3(q->n_chunks, H), 256, lds(decay_chunk_sum_kernel<A>, decay_sum_lds(dim, vdim)), st>>>(
-        in, q->decay_pow, q->pow_n, q->workspace, H, dim, vdim, q->chunk_row0, q->chunk_rows);
+    auto sums = [&](auto kern) {
+      kern<<<dim3(q->n_chunks, H), 512, lds(kern, decay_sum_lds(dim, vdim)), st>>>(in, q->decay_pow, q->pow_n, q->workspace, H, dim, vdim,
+                                                                                  q->chunk_row0, q->chunk_rows);
+    };
+    if (vdim <= 32) sums(decay_chunk_sum_kernel<A, 2>);
+    else sums(decay_chunk_sum_kernel<A, 4>);
     decay_chunk_state_kernel<<<dim3(ceil_div((long)dim * vdim, 256), H, q->n_long), 256, 0, st>>>(
         q->decay_pow, q->pow_n, q->workspace, q->state, q->slot_stride, H, dim, vdim, q->chunk_rows, q->long_chunk0, q->long_slot);
     auto out = [&](auto kern) {
-      kern<<<dim3(q->n_chunks, H), 256, lds(kern, decay_out_lds(dim, vdim)), st>>>(in, q->decay_pow, q->pow_n, q->workspace, q->o, H, dim, vdim,
+      kern<<<dim3(q->n_chunks, H), 512, lds(kern, decay_out_lds(dim, vdim)), st>>>(in, q->decay_pow, q->pow_n, q->workspace, q->o, H, dim, vdim,
                                                                                   q->chunk_row0, q->chunk_rows);
     };
-    if (vdim <= 32) out(decay_chunk_out_kernel<A, 2>);
-    else if (vdim <= 64) out(decay_chunk_out_kernel<A, 4>);
-    else if (vdim <= 128) out(decay_chunk_out_kernel<A, 8>);
-    else out(decay_chunk_out_kernel<A, 16>);
+    if (vdim <= 32) out(decay_chunk_out_kernel<A, 1>);
+    else if (vdim <= 64) out(decay_chunk_out_kernel<A, 2>);
+    else if (vdim <= 128) out(decay_chunk_out_kernel<A, 4>);
+    else out(decay_chunk_out_kernel<A, 8>);
   });
   return known && ok ? (pegainfer_status_t)hipGetLastError() : bad;
 }

@@ -30,13 +30,18 @@ struct RoundFetch {
     v = live ? lv(tt, part) : 0.f;
   }
   __device__ __forceinline__ void land(int tid, float (*s_q)[DP], float (*s_k)[DP], float (*s_v)[kRecCols]) {
+    land(tid, s_q, s_k, s_v, [](float x) { return x; });
+  }
+  // act: applied to every value on its way into LDS, when the loads have long arrived (act(0) = 0)
+  template <typename Act>
+  __device__ __forceinline__ void land(int tid, float (*s_q)[DP], float (*s_k)[DP], float (*s_v)[kRecCols], Act&& act) {
     const int tt = tid >> 4, part = tid & 15;
 #pragma unroll
     for (int j = 0; j < NS; ++j) {
-      s_q[tt][part + 16 * j] = q[j];
-      s_k[tt][part + 16 * j] = k[j];
+      s_q[tt][part + 16 * j] = act(q[j]);
+      s_k[tt][part + 16 * j] = act(k[j]);
     }
-    s_v[tt][part] = v;
+    s_v[tt][part] = act(v);
   }
 };
 

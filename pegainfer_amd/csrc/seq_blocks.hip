@@ -229,9 +229,10 @@ __global__ __launch_bounds__(256) void clamp_glu_rows_kernel(const A* __restrict
   st(out + (int64_t)row * I + i, g * sigmoid_f(alpha * g) * (u + 1.0f));
 }
 
-// one wave per (row, head)
-// The same for heads wider than a wave should walk alone (one norm over a whole row, say): a workgroup per (row, head).
-template <typename A>
+// The norm-and-gate below for heads wider than a wave should walk alone (one norm over a whole row, say): a workgroup per (row, head).
+// VEC: rows, strides and pointers allow four values per load.
+constexpr int kWideKeep = 4;
+template <typename A, bool VEC>
 __global__ __launch_bounds__(256) void wide_rms_gate_kernel(const float* __restrict__ o, const A* __restrict__ w, int w_per_head,
                                                             const A* __restrict__ gate, int64_t gate_stride, int gate_kind, float factor,
                                                             float eps, A* __restrict__ out, int64_t out_stride, int heads, int vdim,
@@ -242,19 +243,64 @@ __global__ __launch_bounds__(256) void wide_rms_gate_kernel(const float* __restr
   const A* gr = gate + (int64_t)row * gate_stride + (int64_t)h * vdim;
   const A* wr = w + (w_per_head ? (int64_t)h * vdim : 0);
   A* dst = out + (int64_t)row * out_stride + (int64_t)h * vdim;
-  auto act = [&](int i) {
-    const float z = ld(gr + i);
-    return gate_kind == 0 ? silu_f(z) : sigmoid_f(z);
+  auto act = [&](float z) { return gate_kind == 0 ? silu_f(z) : sigmoid_f(z); };
+  constexpr int V = VEC ? 4 : 1;
+  auto load = [&](const auto* q, float* t) {
+    if constexpr (VEC) ld4(q, t); else t[0] = ld(q);
   };
+  // the first kWideKeep groups of a thread stay in registers between the sum and the output
+  float v[kWideKeep][V], z[kWideKeep][V], wv[kWideKeep][V];
+#pragma unroll
+  for (int k = 0; k < kWideKeep; ++k) {
+    const int i = (threadIdx.x + 256 * k) * V;
+    if (i < vdim) { load(p + i, v[k]); load(gr + i, z[k]); load(wr + i, wv[k]); }
+  }
   float ss = 0.f;
-  for (int i = threadIdx.x; i < vdim; i += 256) {
-    const float v = gate_first ? p[i] * act(i) : p[i];
-    ss = fmaf(v, v, ss);
+#pragma unroll
+  for (int k = 0; k < kWideKeep; ++k) {
+    const int i = (threadIdx.x + 256 * k) * V;
+    if (i < vdim)
+#pragma unroll
+      for (int u = 0; u < V; ++u) {
+        z[k][u] = act(z[k][u]);
+        const float t = gate_first ? v[k][u] * z[k][u] : v[k][u];
+        ss = fmaf(t, t, ss);
+      }
+  }
+  for (int i = (threadIdx.x + 256 * kWideKeep) * V; i < vdim; i += 256 * V) {
+    float a[V], b[V];
+    load(p + i, a);
+    load(gr + i, b);
+#pragma unroll
+    for (int u = 0; u < V; ++u) {
+      const float t = gate_first ? a[u] * act(b[u]) : a[u];
+      ss = fmaf(t, t, ss);
+    }
   }
   const float sc = factor / sqrtf(block_sum<4>(ss, red) / (float)vdim + eps);
-  for (int i = threadIdx.x; i < vdim; i += 256) st(dst + i, p[i] * act(i) * sc * ld(wr + i));
+  auto store = [&](int i, const float* a, const float* g, const float* b) {
+    float r[V];
+#pragma unroll
+    for (int u = 0; u < V; ++u) r[u] = a[u] * g[u] * sc * b[u];
+    if constexpr (VEC) st4(dst + i, r); else st(dst + i, r[0]);
+  };
+#pragma unroll
+  for (int k = 0; k < kWideKeep; ++k) {
+    const int i = (threadIdx.x + 256 * k) * V;
+    if (i < vdim) store(i, v[k], z[k], wv[k]);
+  }
+  for (int i = (threadIdx.x + 256 * kWideKeep) * V; i < vdim; i += 256 * V) {
+    float a[V], g[V], b[V];
+    load(p + i, a);
+    load(gr + i, g);
+    load(wr + i, b);
+#pragma unroll
+    for (int u = 0; u < V; ++u) g[u] = act(g[u]);
+    store(i, a, g, b);
+  }
 }
 
+// one wave per (row, head)
 template <typename A>
 __global__ __launch_bounds__(256) void head_rms_gate_kernel(const float* __restrict__ o, const A* __restrict__ w, int w_per_head,
                                                             const A* __restrict__ gate, int64_t gate_stride, int gate_kind,
@@ -702,10 +748,15 @@ pegainfer_status_t pegainfer_head_gate_rms(const float* o, const void* w, int32_
   if (!by_dtype(dtype, [&](auto* t) {
         using A = std::remove_pointer_t<decltype(t)>;
         if (vdim > 512 && heads <= 65535) {
-          wide_rms_gate_kernel<A><<<dim3(rows, heads), 256, 0, as_stream(stream)>>>(o, static_cast<const A*>(w), w_per_head,
-                                                                                   static_cast<const A*>(gate), gate_stride, gate_kind,
-                                                                                   factor, eps, static_cast<A*>(out), out_stride, heads,
-                                                                                   vdim, gate_first);
+          const bool vec = vdim % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && host_aligned16(o) && host_aligned16(w) &&
+                           host_aligned16(gate) && host_aligned16(out);
+          auto wide = [&](auto kern) {
+            kern<<<dim3(rows, heads), 256, 0, as_stream(stream)>>>(o, static_cast<const A*>(w), w_per_head, static_cast<const A*>(gate),
+                                                                   gate_stride, gate_kind, factor, eps, static_cast<A*>(out), out_stride,
+                                                                   heads, vdim, gate_first);
+          };
+          if (vec) wide(wide_rms_gate_kernel<A, true>);
+          else wide(wide_rms_gate_kernel<A, false>);
           return;
         }
         head_rms_gate_kernel<A><<<blocks, 256, 0, as_stream(stream)>>>(o, static_cast<const A*>(w), w_per_head,

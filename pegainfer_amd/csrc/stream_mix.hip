@@ -33,25 +33,19 @@ struct StreamMix {
   int layer_norm;              // 0: RMS norm
 };
 
-// MS: the streams a thread's registers hold (S <= MS).  VEC: d, strides and pointers allow four values per load.
-template <typename A, int MS, bool VEC>
-__global__ __launch_bounds__(256) void stream_mix_kernel(StreamMix<A> p, int S, int d) {
+// MS: the streams a thread's registers hold (S <= MS).  VEC: d, strides and pointers allow four values per load.  WAVES: of the
+// workgroup - a step of few rows (decoding) spreads a row over more of them.
+template <typename A, int MS, bool VEC, int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void stream_mix_kernel(StreamMix<A> p, int S, int d) {
   extern __shared__ __attribute__((aligned(16))) float s_u[];   // [d] when a norm follows
-  __shared__ float s_mix[MS * MS], s_out[MS], s_read[MS], red[4];
-  constexpr int V = VEC ? 4 : 1;
+  __shared__ float s_mix[MS * MS], s_out[MS], s_read[MS], red[WAVES];
+  constexpr int V = VEC ? 4 : 1, N = 64 * WAVES;
   const int row = blockIdx.x, tid = threadIdx.x;
   const int64_t src = p.row_index ? p.row_index[row] : row;
   const float* xr = p.x_in ? p.x_in + src * S * d : nullptr;
   const A* er = p.x_in ? nullptr : p.embed + (int64_t)p.ids[src] * d;
-  if (p.y) {
-    for (int i = tid; i < S * S; i += 256) s_mix[i] = ld(p.mix + i);
-    if (tid < S) s_out[tid] = p.mult * ld(p.out_w + tid);
-  }
-  if (tid < S) s_read[tid] = p.read_w ? ld(p.read_w + tid) : 1.0f;
-  __syncthreads();
-  float total = 0.f;
-  for (int i = tid * V; i < d; i += 256 * V) {
-    float x[MS][V], n[MS][V];
+  float x[MS][V], y[V];
+  auto load = [&](int i) {
     if (xr) {
 #pragma unroll
       for (int s = 0; s < MS; ++s)
@@ -67,9 +61,22 @@ __global__ __launch_bounds__(256) void stream_mix_kernel(StreamMix<A> p, int S, 
         for (int u = 0; u < V; ++u) x[s][u] = e[u] * p.embed_scale;
     }
     if (p.y) {
-      float y[V];
       const A* yr = p.y + (int64_t)row * p.y_stride;
       if constexpr (VEC) ld4(yr + i, y); else y[0] = ld(yr + i);
+    }
+  };
+  if (tid * V < d) load(tid * V);            // in flight while the coefficients arrive
+  if (p.y) {
+    for (int i = tid; i < S * S; i += N) s_mix[i] = ld(p.mix + i);
+    if (tid < S) s_out[tid] = p.mult * ld(p.out_w + tid);
+  }
+  if (tid < S) s_read[tid] = p.read_w ? ld(p.read_w + tid) : 1.0f;
+  __syncthreads();
+  float total = 0.f;
+  for (int i = tid * V; i < d; i += N * V) {
+    float n[MS][V];
+    if (i != tid * V) load(i);
+    if (p.y) {
 #pragma unroll
       for (int t = 0; t < MS; ++t)
         if (t < S) {
@@ -116,21 +123,21 @@ __global__ __launch_bounds__(256) void stream_mix_kernel(StreamMix<A> p, int S, 
     }
   }
   if (!p.n_out) return;                      // uniform over the grid
-  total = block_sum<4>(total, red);
+  total = block_sum<WAVES>(total, red);
   float mean = 0.f, var = total / (float)d;
   if (p.layer_norm) {
     mean = total / (float)d;
     float sq = 0.f;
-    for (int i = tid * V; i < d; i += 256 * V)
+    for (int i = tid * V; i < d; i += N * V)
 #pragma unroll
       for (int u = 0; u < V; ++u) {
         const float z = s_u[i + u] - mean;
         sq = fmaf(z, z, sq);
       }
-    var = block_sum<4>(sq, red) / (float)d;
+    var = block_sum<WAVES>(sq, red) / (float)d;
   }
   const float inv = 1.0f / sqrtf(var + p.eps);
-  for (int i = tid * V; i < d; i += 256 * V) {
+  for (int i = tid * V; i < d; i += N * V) {
     float g[V], o[V];
     if constexpr (VEC) ld4(p.gain + i, g); else g[0] = ld(p.gain + i);
 #pragma unroll
@@ -163,19 +170,22 @@ pegainfer_status_t pegainfer_stream_mix(const pegainfer_stream_mix_desc* q, pega
                          host_aligned16(q->y) && host_aligned16(q->x_out) && host_aligned16(q->sum_out) && host_aligned16(q->gain) &&
                          host_aligned16(q->n_out);
         const size_t lds = q->n_out ? (size_t)d * sizeof(float) : 0;
-        auto launch = [&](auto kern) {
+        auto launch = [&](auto kern, int threads) {
           if (lds > 48 * 1024)
             (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-          kern<<<q->rows, 256, lds, as_stream(stream)>>>(p, S, d);
+          kern<<<q->rows, threads, lds, as_stream(stream)>>>(p, S, d);
         };
-        auto by_streams = [&](auto v) {
+        auto by_streams = [&](auto v, auto waves) {
           constexpr bool VEC = decltype(v)::value;
-          if (S <= 2) launch(stream_mix_kernel<A, 2, VEC>);
-          else if (S <= 4) launch(stream_mix_kernel<A, 4, VEC>);
-          else launch(stream_mix_kernel<A, 16, VEC>);
+          constexpr int W = decltype(waves)::value;
+          if (S <= 2) launch(stream_mix_kernel<A, 2, VEC, W>, 64 * W);
+          else if (S <= 4) launch(stream_mix_kernel<A, 4, VEC, W>, 64 * W);
+          else launch(stream_mix_kernel<A, 16, VEC, 4>, 256);   // its registers fit four waves only
         };
-        if (vec) by_streams(std::true_type());
-        else by_streams(std::false_type());
+        const bool wide = q->rows < 128 && d > 1024;
+        if (vec && wide) by_streams(std::true_type(), std::integral_constant<int, 16>());
+        else if (vec) by_streams(std::true_type(), std::integral_constant<int, 4>());
+        else by_streams(std::false_type(), std::integral_constant<int, 4>());
       }))
     return bad;
   return (pegainfer_status_t)hipGetLastError();

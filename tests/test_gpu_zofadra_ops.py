@@ -42,7 +42,7 @@ def states(n, d, seed):
 
 # ------------------------------------------------------------------ streams
 @BOTH
-@pytest.mark.parametrize("streams,d", [(1, 50), (2, 256), (2, 1030), (3, 1024), (4, 77), (5, 300), (16, 64), (3, 13000)])
+@pytest.mark.parametrize("streams,d", [(1, 50), (2, 256), (2, 1030), (3, 1024), (4, 77), (5, 300), (16, 64), (3, 13000), (4, 2048), (6, 2048)])
 def test_output_joins_the_mixed_streams_and_the_next_norm_reads_them(dtype, streams, d):
     g = torch.Generator().manual_seed(streams * d)
     rows, eps = 5, 1e-3
@@ -61,6 +61,9 @@ def test_output_joins_the_mixed_streams_and_the_next_norm_reads_them(dtype, stre
     new, n, sm = B().stream_mix(X.cuda(), streams, d, DT[dtype], **kw)                       # no norm follows
     close(new, ref.permute(1, 0, 2), "float32", tol32=3e-6)
     assert n is None and sm is None
+    many = X.repeat(40, 1, 1)                                                                # enough rows for the narrow workgroups
+    n2 = B().stream_mix(many.cuda(), streams, d, DT[dtype], read_w=dev(a, dtype), gain=dev(gain, dtype), **dict(kw, y=dev(y.repeat(40, 1), dtype)))[1]
+    close(n2, R.layer_norm(u, gain.double(), eps).repeat(40, 1), dtype, tol16=1e-2)
     # the end: a plain sum, some rows only, in another order
     idx = torch.tensor([3, 0, 3], dtype=torch.int32, device="cuda")
     _, n, _ = B().stream_mix(X.cuda(), streams, d, DT[dtype], gain=dev(gain, dtype), eps=eps, row_index=idx, keep=False)
