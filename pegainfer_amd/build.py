@@ -27,6 +27,13 @@ KERNEL_LIB = os.path.join(LIBDIR, "libpegainfer_kernels_hip.so")
 HOST_LIB = os.path.join(LIBDIR, "libpegainfer_qwen3.so")
 
 
+# What the step runtime of a family needs of csrc/*.hip and csrc/host/*.cpp (build_family); the link refuses a missing symbol.
+FAMILY_SOURCES = {
+    "zofadra": (("attn_latent", "attn_paged", "decay_attn", "elementwise", "gemm_strided", "linear", "norm", "sampling", "seq_blocks", "stream_mix"),
+                ("logprobs", "zofadra_runtime")),
+}
+
+
 def _hipcc():
     for c in (os.environ.get("HIPCC"), shutil.which("hipcc"), "/opt/rocm/bin/hipcc"):
         if c and os.path.exists(c):
@@ -58,6 +65,35 @@ def _compile(src, extra, headers, objdir=None):
     return obj
 
 
+def _headers():
+    headers = [os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith(".h")]
+    headers += [os.path.join(ROOT, "include", f) for f in os.listdir(os.path.join(ROOT, "include"))]
+    return headers, [os.path.join(HOST, f) for f in os.listdir(HOST) if f.endswith(".h")]
+
+
+def build_family(family, libdir=None):
+    """The two libraries with ONE family's sources, in pegainfer_amd/lib_<family> (PEGAINFER_LIB_DIR selects it): enough to load that
+    family's engine, in a fraction of the whole build's time.  Objects are shared with the whole build.  Returns the folder."""
+    ksrcs, hsrcs = FAMILY_SOURCES[family]
+    libdir = libdir or os.path.join(PKG, "lib_" + family)
+    kernel_lib, host_lib = os.path.join(libdir, os.path.basename(KERNEL_LIB)), os.path.join(libdir, os.path.basename(HOST_LIB))
+    os.makedirs(libdir, exist_ok=True)
+    os.makedirs(OBJDIR, exist_ok=True)
+    headers, hheaders = _headers()
+    with cf.ThreadPoolExecutor(max_workers=min(8, os.cpu_count() or 4)) as ex:
+        kfut = [ex.submit(_compile, os.path.join(CSRC, s + ".hip"), [], headers) for s in ksrcs]
+        hfut = [ex.submit(_compile, os.path.join(HOST, s + ".cpp"), ["-x", "hip", "-I", HOST], headers + hheaders) for s in hsrcs]
+        kobjs, hobjs = [f.result() for f in kfut], [f.result() for f in hfut]
+    link = [_hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", "-Wl,--no-undefined", "-o"]
+    if _newer(kobjs, kernel_lib):
+        _run(link + [kernel_lib] + kobjs)
+    if _newer(hobjs + [kernel_lib], host_lib):
+        _run(link + [host_lib] + hobjs + ["-L", libdir, "-lpegainfer_kernels_hip", "-Wl,-rpath,$ORIGIN"])
+    with open(os.path.join(libdir, "FAMILY"), "w") as f:      # tells ffi.py that other families' symbols are absent on purpose
+        f.write(family + "\n")
+    return libdir
+
+
 def build(verbose=False, force=False, variant=None, extra_flags=()):
     """variant: build the same sources with `extra_flags` into pegainfer_amd/lib_<variant> (objects in build_<variant>) for a
     same-box A/B against the default build (PEGAINFER_LIB_DIR selects it at load time); the default build takes no flags."""
@@ -71,13 +107,9 @@ def build(verbose=False, force=False, variant=None, extra_flags=()):
         for f in os.listdir(objdir):
             if os.path.isfile(os.path.join(objdir, f)):
                 os.remove(os.path.join(objdir, f))
-    headers = [os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith(".h")]
-    headers += [os.path.join(ROOT, "include", f) for f in os.listdir(os.path.join(ROOT, "include"))]
+    headers, hheaders = _headers()
     ksrcs = sorted(os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith(".hip"))
-    hsrcs, hheaders = [], []
-    if os.path.isdir(HOST):
-        hsrcs = sorted(os.path.join(HOST, f) for f in os.listdir(HOST) if f.endswith(".cpp"))
-        hheaders = [os.path.join(HOST, f) for f in os.listdir(HOST) if f.endswith(".h")]
+    hsrcs = sorted(os.path.join(HOST, f) for f in os.listdir(HOST) if f.endswith(".cpp"))
     with cf.ThreadPoolExecutor(max_workers=min(8, os.cpu_count() or 4)) as ex:
         kfut = [ex.submit(_compile, s, extra_flags, headers, objdir) for s in ksrcs]
         hfut = [ex.submit(_compile, s, ["-x", "hip", "-I", HOST] + extra_flags, headers + hheaders, objdir) for s in hsrcs]

@@ -84,7 +84,10 @@ class _Lib:
         self.protos = {}
         for header in headers:
             self.protos.update(parse_header(os.path.join(INCLUDE, header)))
+        one_family = os.path.exists(os.path.join(LIBDIR, "FAMILY"))   # build.build_family: other families' symbols are absent
         for name, (res, args) in self.protos.items():
+            if one_family and not hasattr(self.cdll, name):
+                continue               # using one raises AttributeError
             fn = getattr(self.cdll, name)  # AttributeError if a declared symbol is not exported
             fn.restype = res
             fn.argtypes = args

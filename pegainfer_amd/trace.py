@@ -13,6 +13,18 @@ import os
 import sys
 
 
+def model_family(argv):
+    """the family of the model folder that `argv` names, or None; needs no native library"""
+    ap = argparse.ArgumentParser(add_help=False)
+    ap.add_argument("--model")
+    a, _ = ap.parse_known_args(argv)
+    from . import registry
+    try:
+        return registry.family_of(registry.read_config(a.model)) if a.model else None
+    except (OSError, ValueError):
+        return None
+
+
 def main(argv=None):
     ap = argparse.ArgumentParser(prog="trace_run", description=__doc__.split("\n")[0])
     ap.add_argument("--model", required=True, help="folder with config.json and model.safetensors")

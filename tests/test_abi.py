@@ -43,6 +43,16 @@ def test_reference_ffi_names_are_kept(built_libs):
     assert not [s for s in must if s not in exp]
 
 
+def test_one_familys_libraries_link_without_the_other_families(built_libs, tmp_path):
+    """what a fresh checkout compiles for one model: every symbol of that family resolves inside its two libraries"""
+    from pegainfer_amd import build
+    for family in build.FAMILY_SOURCES:
+        libdir = build.build_family(family, str(tmp_path / family))
+        exp = _exported(os.path.join(libdir, "libpegainfer_qwen3.so"))
+        assert set(ffi.declared_symbols("pegainfer_%s.h" % family)) <= exp and "pegainfer_qwen3_decode" not in exp
+        assert os.path.exists(os.path.join(libdir, "FAMILY"))
+
+
 def test_gfx950_code_object_present(built_libs):
     """The .so must carry a gfx950 code object (single target arch, no dual build)."""
     data = open(built_libs[0], "rb").read()
