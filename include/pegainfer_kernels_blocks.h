@@ -55,7 +55,7 @@ pegainfer_status_t pegainfer_silu_mul_rows(const void* gate_up, void* out, int32
  * kernel (bf16 weights with contiguous k in 16-byte chunks; an fp32 x is rounded to bf16 as it is staged) and a few-rows
  * form that streams the weights once (<= 8 rows per tile: decode).  In each the k order of an output is fixed, so a row's
  * result does not depend on what else is in the launch; which kernel runs depends on the launch's shape. */
-enum { PEGAINFER_EPI_NONE = 0, PEGAINFER_EPI_RELU_SQ = 1, PEGAINFER_EPI_SIGMOID_GATE = 2 };
+enum { PEGAINFER_EPI_NONE = 0, PEGAINFER_EPI_RELU_SQ = 1, PEGAINFER_EPI_SIGMOID_GATE = 2, PEGAINFER_EPI_GELU_ERF = 3 };
 typedef struct {
   const void* x;
   const void* w;
@@ -72,7 +72,7 @@ typedef struct {
   int32_t max_tiles;
   const int32_t* x_row_index;
   const int32_t* y_row_index;
-  int32_t epilogue;          /* SIGMOID_GATE: y *= sigmoid(gate[row * gate_row_stride + g]) */
+  int32_t epilogue;          /* RELU_SQ, GELU_ERF: an activation of y; SIGMOID_GATE: y *= sigmoid(gate[row * gate_row_stride + g]) */
   const void* gate;
   int32_t gate_dtype;
   int64_t gate_row_stride;
@@ -259,6 +259,24 @@ pegainfer_status_t pegainfer_route_from_logits_ex(const float* logits, int64_t l
                                                   int32_t* out_expert, float* out_weight, int32_t experts, int32_t n_groups,
                                                   int32_t keep_groups, int32_t top, int32_t rows, int32_t score_kind,
                                                   int32_t group_kind, int32_t renorm, int32_t dtype, pegainfer_stream_t stream);
+/* Selection and, with sort_experts > 0, the sort of pegainfer_route_sort behind it, from router logits in fp32 (one launch for up to 16
+ * rows).  As pegainfer_route_from_logits_ex, with the weights times `factor` at the end.  Only expert numbers below sort_experts get
+ * positions: numbers from there on are identity experts, whose output is the feed-forward's own input
+ * (pegainfer_route_combine_same). */
+typedef struct {
+  const float* logits;
+  int64_t logits_stride;
+  const void* correction;
+  int32_t* out_expert;
+  float* out_weight;
+  int32_t experts, n_groups, keep_groups, top, rows, score_kind, group_kind, renorm;
+  float factor;
+  int32_t sort_experts;
+  int32_t *pos_pair, *pos_row, *tile_group, *tile_row0, *tile_rows, *n_tiles;
+  int32_t max_tiles, rows_per_tile;
+  int32_t dtype;
+} pegainfer_route_plan_desc;
+pegainfer_status_t pegainfer_route_plan(const pegainfer_route_plan_desc* q, pegainfer_stream_t stream);
 /* pegainfer_route_combine plus a row every token gets (a shared expert's output, [rows, d] of dtype; NULL = none) */
 pegainfer_status_t pegainfer_route_combine_add(const float* y_pairs, const float* weight, const void* add, void* out, int32_t d,
                                                int32_t top, int32_t rows, int32_t dtype, pegainfer_stream_t stream);
@@ -268,6 +286,13 @@ pegainfer_status_t pegainfer_route_combine_add(const float* y_pairs, const float
 pegainfer_status_t pegainfer_route_combine_gated(const float* y_pairs, const float* weight, const void* add,
                                                  const float* add_gate, int64_t add_gate_stride, void* out, int32_t d,
                                                  int32_t top, int32_t rows, int32_t dtype, pegainfer_stream_t stream);
+
+/* pegainfer_route_combine_gated in which a pair whose expert[row * top + c] is same_from or more takes the row of `same` ([rows, d] of
+ * dtype at same_stride; NULL = no such pairs) instead of its y_pairs row: identity experts */
+pegainfer_status_t pegainfer_route_combine_same(const float* y_pairs, const float* weight, const int32_t* expert, int32_t same_from,
+                                                const void* same, int64_t same_stride, const void* add, const float* add_gate,
+                                                int64_t add_gate_stride, void* out, int32_t d, int32_t top, int32_t rows, int32_t dtype,
+                                                pegainfer_stream_t stream);
 
 /* Residual sum with a constant factor, then an RMS norm whose gain is ONE number (gain: a one-element tensor of dtype):
  *   r = x_in + mult * (y + bias) + add_rows + add_vec          -> x_out (fp32; may alias x_in)
@@ -296,9 +321,36 @@ typedef struct {
 pegainfer_status_t pegainfer_terms_rms_add(const float* x_in, const pegainfer_sum_term* terms, int32_t n_terms, float* x_out,
                                            const void* gain, float eps, void* n_out, int32_t n_dtype, int32_t d, int32_t rows,
                                            int32_t dtype, pegainfer_stream_t stream);
+/* The same with its options in a struct (zeroed = as above):
+ *   gain_offset  is added to every norm weight, the terms' and the gain: 1 for weights stored around zero;
+ *   row_index    x_in's row of an output row (x_out must then be another buffer);
+ *   embed        with x_in NULL the stream starts as embed[token_ids[row]] * embed_scale, plus, when pair_table ([buckets + 1][d]) is
+ *                given, its row (prev_ids[row] * mul_prev + token_ids[row] * mul_cur) mod buckets - row `buckets` where prev_ids is
+ *                negative (a sequence's first token).  embed and pair_table of dtype. */
+typedef struct {
+  const float* x_in;
+  const int32_t* row_index;
+  const void* embed;
+  const uint32_t* token_ids;
+  float embed_scale;
+  const void* pair_table;
+  const int32_t* prev_ids;
+  int64_t mul_prev, mul_cur, buckets;
+  const pegainfer_sum_term* terms;
+  int32_t n_terms;
+  float* x_out;
+  const void* gain;
+  float eps, gain_offset;
+  void* n_out;
+  int32_t n_dtype, d, rows, dtype;
+} pegainfer_terms_rms_desc;
+pegainfer_status_t pegainfer_terms_rms(const pegainfer_terms_rms_desc* q, pegainfer_stream_t stream);
 /* out[row, i] = act(gate[row, i]) * up[row, i], i < I; gate and up are column ranges of rows with stride in_row_stride (elements of
- * dtype).  act 0 = silu, 1 = relu, 2 = gelu (tanh form) */
-enum { PEGAINFER_ACT_SILU = 0, PEGAINFER_ACT_RELU = 1, PEGAINFER_ACT_GELU_TANH = 2 };
+ * dtype).  act 0 = silu, 1 = relu, 2 = gelu (tanh form), 3 = gelu (exact form) */
+enum { PEGAINFER_ACT_SILU = 0, PEGAINFER_ACT_RELU = 1, PEGAINFER_ACT_GELU_TANH = 2, PEGAINFER_ACT_GELU_ERF = 3 };
+/* out[row, i] = act(in[row, i]), i < I (in place allowed) */
+pegainfer_status_t pegainfer_act_rows(const void* in, int64_t in_row_stride, void* out, int64_t out_row_stride, int32_t I, int32_t rows,
+                                      int32_t act, int32_t dtype, pegainfer_stream_t stream);
 pegainfer_status_t pegainfer_glu_rows(const void* gate, const void* up, int64_t in_row_stride, void* out, int64_t out_row_stride,
                                       int32_t I, int32_t rows, int32_t act, int32_t dtype, pegainfer_stream_t stream);
 /* out[i] = cap * tanh(in[i] / cap) over n fp32 values (in place allowed) */
@@ -420,6 +472,39 @@ typedef struct {
 int32_t pegainfer_decay_attention_chunked_ok(int32_t dim, int32_t vdim);
 int64_t pegainfer_decay_attention_workspace(int32_t n_chunks, int32_t heads, int32_t dim, int32_t vdim);
 pegainfer_status_t pegainfer_decay_attention(const pegainfer_decay_attention_desc* d, pegainfer_stream_t stream);
+/* Gated linear attention: the same state with a decay per (head, key channel) and token that acts on the rows of S.
+ * Per row of `proj` (dtype): q at q_off, k at k_off (heads x dim), v at v_off (heads x vdim);  z: fp32 [rows][heads * dim] at z_stride,
+ * z_bias [heads * dim] of dtype or NULL:
+ *   a = sigmoid(z + z_bias)^(1 / tau);  S <- diag(a) S + k v^T;  y = S^T (q * q_scale)          -> o (fp32 [rows][heads * vdim])
+ * Scan and chunk form, tables and scan_max as pegainfer_decay_attention (pegainfer_gated_linear_chunked_ok, ..._workspace). */
+typedef struct {
+  const void* proj;
+  int64_t proj_stride, q_off, k_off, v_off;
+  float q_scale;
+  const float* z;
+  int64_t z_stride;
+  const void* z_bias;
+  float tau;
+  float* state;
+  int64_t slot_stride;
+  float* o;
+  int32_t heads, dim, vdim;
+  const int32_t* entry_row0;
+  const int32_t* entry_slot;
+  int32_t n_entries;
+  int32_t scan_max;
+  const int32_t* chunk_row0;
+  const int32_t* chunk_rows;
+  int32_t n_chunks;
+  const int32_t* long_chunk0;
+  const int32_t* long_slot;
+  int32_t n_long;
+  float* workspace;
+  int32_t dtype;
+} pegainfer_gated_linear_desc;
+int32_t pegainfer_gated_linear_chunked_ok(int32_t dim, int32_t vdim);
+int64_t pegainfer_gated_linear_workspace(int32_t n_chunks, int32_t heads, int32_t dim, int32_t vdim);
+pegainfer_status_t pegainfer_gated_linear(const pegainfer_gated_linear_desc* d, pegainfer_stream_t stream);
 /* Per-head RMS norm of a memory's read-out, a weight, a gate and a constant factor:
  *   out[row, h, :] = o[row, h, :] / sqrt(mean(o[row, h, :]^2) + eps) * w * act(gate[row, h, :]) * factor
  * w: [vdim] shared by the heads (w_per_head == 0) or [heads * vdim]; gate_kind 0 = silu, 1 = sigmoid; gate rows of dtype
@@ -479,6 +564,33 @@ pegainfer_status_t pegainfer_qk_prep_paged_form(const void* proj, int32_t proj_d
                                                const int32_t* page_ids, void* cache, int64_t page_stride, int64_t k_cache_off,
                                                int64_t v_cache_off, int32_t page_size, float* q_out, void* q_out_stored,
                                                int32_t n_rows, int32_t dtype, pegainfer_stream_t stream);
+/* The same with its parameters in a struct and two more: rot_amp multiplies every cosine and sine of the rotation (1 = none; a
+ * long-context scaling's amplitude); shared_tail > 0 leaves the last shared_tail values of a key out of the cache's key part, whose
+ * rows are then [kv_heads][dim - shared_tail] - for values projected as keys (v_off = k_off, vdim = dim), whose rows hold those
+ * values already because the rotation does not reach them. */
+typedef struct {
+  const void* proj;
+  int32_t proj_dtype;
+  int64_t proj_stride, q_off, k_off, v_off;
+  int32_t heads, kv_heads, dim, vdim;
+  const void *q_norm, *k_norm;
+  int32_t norm_kind;
+  float eps;
+  const void *q_bias, *k_bias, *v_bias;
+  float qt_coef;
+  int32_t qt_every;
+  const float* inv_freq;
+  int32_t rot_dims, rot_layout;
+  float rot_amp;
+  const int32_t *positions, *row_entry, *page_indptr, *page_ids;
+  void* cache;
+  int64_t page_stride, k_cache_off, v_cache_off;
+  int32_t page_size, shared_tail;
+  float* q_out;
+  void* q_out_stored;
+  int32_t n_rows, dtype;
+} pegainfer_qk_prep_desc;
+pegainfer_status_t pegainfer_qk_prep(const pegainfer_qk_prep_desc* p, pegainfer_stream_t stream);
 /* Causal softmax attention, scores and weights in fp32:  out[row, h, :] = factor * sum_{j <= position} softmax_j(q . k_j * scale) v_j.
  * The rows are cut by the caller into tiles that stay inside one entry: tile i covers rows tile_row0[i] .. + tile_ntok[i] - 1
  * and, of each key/value group's query heads, tile_qh0[i] .. + tile_nqh[i] - 1, with ntok * nqh <= 16.  dim, vdim <= 256.
@@ -551,6 +663,7 @@ typedef struct {
   int32_t n_split;
   float* workspace;
   int32_t plain;
+  int32_t shared_tail;       /* > 0: the last shared_tail values of a key are its value's (see pegainfer_qk_prep); one map, vdim == dim */
 } pegainfer_attn_options;
 pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cache, int64_t page_stride, int64_t k_cache_off,
                                                  int64_t v_cache_off, int32_t page_size, const int32_t* positions,

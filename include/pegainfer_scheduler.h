@@ -109,6 +109,8 @@ pegainfer_sched_t pegainfer_sched_create_ramalix(void* model, uint64_t seed, con
 pegainfer_sched_t pegainfer_sched_create_kukulorn(void* model, uint64_t seed, const uint32_t* stop_tokens, int32_t n_stop);
 /* the same over the Zofadra runtime (pegainfer_zofadra.h): `model` is a pegainfer_zofadra_t */
 pegainfer_sched_t pegainfer_sched_create_zofadra(void* model, uint64_t seed, const uint32_t* stop_tokens, int32_t n_stop);
+/* the same over the Sopanex runtime (pegainfer_sopanex.h): `model` is a pegainfer_sopanex_t */
+pegainfer_sched_t pegainfer_sched_create_sopanex(void* model, uint64_t seed, const uint32_t* stop_tokens, int32_t n_stop);
 void pegainfer_sched_destroy(pegainfer_sched_t s);
 
 /* EngineHandle::submit: returns the RequestId the events carry (ids count up from 0 in submission order) */

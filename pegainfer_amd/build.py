@@ -31,6 +31,8 @@ HOST_LIB = os.path.join(LIBDIR, "libpegainfer_qwen3.so")
 FAMILY_SOURCES = {
     "zofadra": (("attn_latent", "attn_paged", "decay_attn", "elementwise", "gemm_strided", "linear", "norm", "sampling", "seq_blocks", "stream_mix"),
                 ("logprobs", "zofadra_runtime")),
+    "sopanex": (("attn_paged", "elementwise", "gated_linear", "gemm_strided", "linear", "moe_route", "norm", "sampling", "seq_blocks"),
+                ("logprobs", "sopanex_runtime")),
 }
 
 

@@ -28,6 +28,8 @@ struct PrepForm {
                         // rotation, no weight (unit root mean square); 2: over ALL heads of the projection at once before the
                         // rotation, times a weight [heads * dim] / [kv_heads * dim]
   int rot_halves = 0;   // 0: neighbours (2i, 2i + 1) are rotated together; 1: value i with value i + rot_dims / 2
+  float rot_amp = 1.f;  // factor of every cosine and sine
+  int k_keep = 0;       // leading values of a key that go to the key part of the cache (dim unless the rest is the value's)
 };
 
 // I: type of the projection rows read (the storage type, or float for rows that an fp32 stage such as a convolution left)
@@ -100,11 +102,11 @@ __global__ __launch_bounds__(256) void qk_prep_paged_kernel(
           if (pf.rot_halves) {
             const int f = i < half ? i : i - half;
             const float ang = (float)pos * inv_freq[f];
-            const float cs = cosf(ang), sn = sinf(ang);
+            const float cs = cosf(ang) * pf.rot_amp, sn = sinf(ang) * pf.rot_amp;
             out = i < half ? buf[i] * cs - buf[i + half] * sn : buf[i] * cs + buf[i - half] * sn;
           } else {
             const float ang = (float)pos * inv_freq[i >> 1];
-            const float cs = cosf(ang), sn = sinf(ang);
+            const float cs = cosf(ang) * pf.rot_amp, sn = sinf(ang) * pf.rot_amp;
             out = (i & 1) ? buf[i] * cs + buf[i - 1] * sn : buf[i] * cs - buf[i + 1] * sn;
           }
         }
@@ -121,8 +123,8 @@ __global__ __launch_bounds__(256) void qk_prep_paged_kernel(
       if (is_q) {
         if (q_out_stored) st(q_out_stored + ((int64_t)row * H + hh) * dim + i, out);
         else q_out[((int64_t)row * H + hh) * dim + i] = out;
-      } else
-        st(cache + page * page_stride + k_cache_off + ((int64_t)slot * G + hd) * dim + i, out);
+      } else if (i < pf.k_keep)
+        st(cache + page * page_stride + k_cache_off + ((int64_t)slot * G + hd) * pf.k_keep + i, out);
     }
     __builtin_amdgcn_wave_barrier();
   }
@@ -154,6 +156,8 @@ struct AttnForm {
   const void* gate = nullptr;  // output gate logits (storage type), rows at gate_stride: the finished head is multiplied by
   int64_t gate_stride = 0;     // sigmoid(gate[row, h * vdim + c]) (gate_kind 1: one per value) or sigmoid(gate[row, h]) (2: one
   int gate_kind = 0;           // per head)
+  int k_keep = 0;              // values of a key in the cache's key part; the key's values from there on are its value's (MAPS == 1, the
+                               // whole key unless values are projected as keys and only a part of a key is rotated)
 };
 
 // first position of the run of keys that position `pos` sees (besides the kept first tokens)
@@ -233,8 +237,10 @@ __global__ __launch_bounds__(256) void paged_attention_kernel(
   float* s_q = s_v + kAttKeys * vdim;                 // [16][qd]
   float* s_p = s_q + kAttRows * qd;                   // [4 waves][MAPS][64 keys][4 rows of the wave]
   // 16-byte loads from the cache: every key / value row of the request starts at a multiple of eight values
-  const bool vec_k = (qd & 7) == 0 && (page_stride & 7) == 0 && (k_cache_off & 7) == 0 && aligned16(cache);
-  const bool vec_v = (vdim & 7) == 0 && (page_stride & 7) == 0 && (v_cache_off & 7) == 0 && aligned16(cache);
+  const int kw = form.k_keep;                         // values of a head in the cache's key part
+  const bool tail = kw < qd;                          // the others are staged with the values
+  const bool vec_k = (kw & 7) == 0 && (page_stride & 7) == 0 && (k_cache_off & 7) == 0 && aligned16(cache);
+  const bool vec_v = (vdim & 7) == 0 && (kw & 7) == 0 && (page_stride & 7) == 0 && (v_cache_off & 7) == 0 && aligned16(cache);
   const int tile = blockIdx.x, g = blockIdx.y;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int row0 = tile_row0[tile], ntok = tile_ntok[tile], qh0 = tile_qh0[tile], nqh = tile_nqh[tile];
@@ -280,19 +286,19 @@ __global__ __launch_bounds__(256) void paged_attention_kernel(
       if (j < nk) {
         const int p = k0 + j;
         const int64_t pg = (int64_t)pages[p / page_size] * page_stride;
-        const A* kp = cache + pg + k_cache_off + ((int64_t)(p % page_size) * G + g) * qd;
+        const A* kp = cache + pg + k_cache_off + ((int64_t)(p % page_size) * G + g) * kw;
         const A* vp = cache + pg + v_cache_off + ((int64_t)(p % page_size) * G + g) * vdim;
         float* dk = s_k + j * kd;
         float* dv = s_v + j * vdim;
         if (vec_k) {
-          for (int d = sub * 8; d < qd; d += 32) {
+          for (int d = sub * 8; d < kw; d += 32) {
             float t[8];
             Vec8<A>::load(kp + d, t);
 #pragma unroll
             for (int u = 0; u < 8; ++u) dk[d + u] = t[u];
           }
         } else {
-          for (int d = sub; d < qd; d += 4) dk[d] = ld(kp + d);
+          for (int d = sub; d < kw; d += 4) dk[d] = ld(kp + d);
         }
         if (vec_v) {
           for (int d = sub * 8; d < vdim; d += 32) {
@@ -300,9 +306,17 @@ __global__ __launch_bounds__(256) void paged_attention_kernel(
             Vec8<A>::load(vp + d, t);
 #pragma unroll
             for (int u = 0; u < 8; ++u) dv[d + u] = t[u];
+            if (tail && d >= kw) {
+#pragma unroll
+              for (int u = 0; u < 8; ++u) dk[d + u] = t[u];
+            }
           }
         } else {
-          for (int d = sub; d < vdim; d += 4) dv[d] = ld(vp + d);
+          for (int d = sub; d < vdim; d += 4) {
+            const float t = ld(vp + d);
+            dv[d] = t;
+            if (tail && d >= kw) dk[d] = t;
+          }
         }
       }
     }
@@ -477,8 +491,10 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
 #pragma unroll
     for (int cb = 0; cb < NCB; ++cb) o[m][cb] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  const bool vec_k = (dim & 7) == 0 && (page_stride & 7) == 0 && (k_cache_off & 7) == 0 && aligned16(cache);
-  const bool vec_v = (vdim & 7) == 0 && (page_stride & 7) == 0 && (v_cache_off & 7) == 0 && aligned16(cache);
+  const int kw = form.k_keep;                       // values of a head in the cache's key part
+  const bool tail = kw < qd;                        // the others are staged with the values (one map then)
+  const bool vec_k = (dim & 7) == 0 && (kw & 7) == 0 && (page_stride & 7) == 0 && (k_cache_off & 7) == 0 && aligned16(cache);
+  const bool vec_v = (vdim & 7) == 0 && (kw & 7) == 0 && (page_stride & 7) == 0 && (v_cache_off & 7) == 0 && aligned16(cache);
   for (int k0 = kfirst + (int)blockIdx.z * kAttKeys; k0 < kmax; k0 += kAttKeys * nsplit) {
     const int nk = min(kAttKeys, kmax - k0);
     if (k0 >= form.keep_first && k0 + kAttKeys <= lo0) continue;   // seen by no row of the tile (uniform over the workgroup)
@@ -488,18 +504,18 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
       if (j < nk) {
         const int p = k0 + j;
         const int64_t pg = (int64_t)pages[p / page_size] * page_stride;
-        const uint16_t* kp = cache + pg + k_cache_off + ((int64_t)(p % page_size) * G + g) * qd;
+        const uint16_t* kp = cache + pg + k_cache_off + ((int64_t)(p % page_size) * G + g) * kw;
         const uint16_t* vp = cache + pg + v_cache_off + ((int64_t)(p % page_size) * G + g) * vdim;
         uint16_t* dk = s_k + j * ks;
         if (vec_k) {
-          for (int c = sub * 8; c < qd; c += 32) {
+          for (int c = sub * 8; c < kw; c += 32) {
             const u32x4 t = *reinterpret_cast<const u32x4*>(kp + c);
             uint16_t* dst = dk + (c / dim) * dp + c % dim;           // 8-byte aligned (ks * 2 is a multiple of 8 only)
             *reinterpret_cast<u32x2*>(dst) = u32x2{t.x, t.y};
             *reinterpret_cast<u32x2*>(dst + 4) = u32x2{t.z, t.w};
           }
         } else {
-          for (int c = sub; c < qd; c += 4) dk[(c / dim) * dp + c % dim] = kp[c];
+          for (int c = sub; c < kw; c += 4) dk[(c / dim) * dp + c % dim] = kp[c];
         }
         if (vec_v) {
           for (int c = sub * 8; c < vdim; c += 32) {
@@ -510,9 +526,17 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
               s_vt[(c + 2 * u) * kMfVs + j] = (uint16_t)(w[u] & 0xFFFFu);
               s_vt[(c + 2 * u + 1) * kMfVs + j] = (uint16_t)(w[u] >> 16);
             }
+            if (tail && c >= kw) {
+              *reinterpret_cast<u32x2*>(dk + c) = u32x2{t.x, t.y};
+              *reinterpret_cast<u32x2*>(dk + c + 4) = u32x2{t.z, t.w};
+            }
           }
         } else {
-          for (int c = sub; c < vdim; c += 4) s_vt[c * kMfVs + j] = vp[c];
+          for (int c = sub; c < vdim; c += 4) {
+            const uint16_t t = vp[c];
+            s_vt[c * kMfVs + j] = t;
+            if (tail && c >= kw) dk[c] = t;
+          }
         }
       }
     }
@@ -738,26 +762,45 @@ pegainfer_status_t pegainfer_qk_prep_paged_form(const void* proj, int32_t proj_d
                                                const int32_t* page_ids, void* cache, int64_t page_stride, int64_t k_cache_off,
                                                int64_t v_cache_off, int32_t page_size, float* q_out, void* q_out_stored,
                                                int32_t n_rows, int32_t dtype, pegainfer_stream_t stream) {
-  if (n_rows <= 0) return 0;
-  if (heads <= 0 || kv_heads <= 0 || dim <= 0 || dim > 256 || vdim <= 0 || rot_dims < 0 || rot_dims > dim || (rot_dims & 1) ||
-      page_size <= 0 || (rot_dims > 0 && !inv_freq) || (!q_norm) != (!k_norm) || norm_kind < 0 || norm_kind > 2 ||
-      (norm_kind == PEGAINFER_QKNORM_ALL_WEIGHT && !q_norm) || (rot_layout != PEGAINFER_ROT_PAIRS && rot_layout != PEGAINFER_ROT_HALVES))
+  pegainfer_qk_prep_desc p{};
+  p.proj = proj; p.proj_dtype = proj_dtype; p.proj_stride = proj_stride; p.q_off = q_off; p.k_off = k_off; p.v_off = v_off;
+  p.heads = heads; p.kv_heads = kv_heads; p.dim = dim; p.vdim = vdim;
+  p.q_norm = q_norm; p.k_norm = k_norm; p.norm_kind = norm_kind; p.eps = eps;
+  p.q_bias = q_bias; p.k_bias = k_bias; p.v_bias = v_bias; p.qt_coef = qt_coef; p.qt_every = qt_every;
+  p.inv_freq = inv_freq; p.rot_dims = rot_dims; p.rot_layout = rot_layout; p.rot_amp = 1.0f;
+  p.positions = positions; p.row_entry = row_entry; p.page_indptr = page_indptr; p.page_ids = page_ids;
+  p.cache = cache; p.page_stride = page_stride; p.k_cache_off = k_cache_off; p.v_cache_off = v_cache_off; p.page_size = page_size;
+  p.q_out = q_out; p.q_out_stored = q_out_stored; p.n_rows = n_rows; p.dtype = dtype;
+  return pegainfer_qk_prep(&p, stream);
+}
+
+pegainfer_status_t pegainfer_qk_prep(const pegainfer_qk_prep_desc* p, pegainfer_stream_t stream) {
+  if (!p) return PK_BAD;
+  if (p->n_rows <= 0) return 0;
+  const int heads = p->heads, kv_heads = p->kv_heads, dim = p->dim;
+  if (heads <= 0 || kv_heads <= 0 || dim <= 0 || dim > 256 || p->vdim <= 0 || p->rot_dims < 0 || p->rot_dims > dim || (p->rot_dims & 1) ||
+      p->page_size <= 0 || (p->rot_dims > 0 && !p->inv_freq) || (!p->q_norm) != (!p->k_norm) || p->norm_kind < 0 || p->norm_kind > 2 ||
+      (p->norm_kind == PEGAINFER_QKNORM_ALL_WEIGHT && !p->q_norm) ||
+      (p->rot_layout != PEGAINFER_ROT_PAIRS && p->rot_layout != PEGAINFER_ROT_HALVES) || p->shared_tail < 0 || p->shared_tail > dim)
     return PK_BAD;
   PrepForm pf;
-  pf.norm_kind = norm_kind;
-  pf.rot_halves = rot_layout == PEGAINFER_ROT_HALVES;
+  pf.norm_kind = p->norm_kind;
+  pf.rot_halves = p->rot_layout == PEGAINFER_ROT_HALVES;
+  pf.rot_amp = p->rot_amp;
+  pf.k_keep = dim - p->shared_tail;
   bool ok = true;
-  const bool known = by_dtype(dtype, [&](auto* t) {
+  const bool known = by_dtype(p->dtype, [&](auto* t) {
     using A = std::remove_pointer_t<decltype(t)>;
-    ok = by_dtype(proj_dtype, [&](auto* ti) {
+    ok = by_dtype(p->proj_dtype, [&](auto* ti) {
       using I = std::remove_pointer_t<decltype(ti)>;
       // few rows (decoding): the heads of a row spread over several workgroups, four heads each; many rows fill the chip alone
-      const int per_row = n_rows >= 512 ? 1 : std::min(16, ceil_div(heads + kv_heads, 4));
-      qk_prep_paged_kernel<A, I><<<dim3(n_rows, per_row), 256, (size_t)4 * dim * sizeof(float), as_stream(stream)>>>(
-          static_cast<const I*>(proj), proj_stride, q_off, k_off, v_off, heads, kv_heads, dim, vdim, static_cast<const A*>(q_norm),
-          static_cast<const A*>(k_norm), eps, inv_freq, rot_dims, positions, row_entry, page_indptr, page_ids, static_cast<A*>(cache),
-          page_stride, k_cache_off, v_cache_off, page_size, q_out, static_cast<A*>(q_out_stored), static_cast<const A*>(q_bias),
-          static_cast<const A*>(k_bias), static_cast<const A*>(v_bias), qt_coef, qt_every, pf);
+      const int per_row = p->n_rows >= 512 ? 1 : std::min(16, ceil_div(heads + kv_heads, 4));
+      qk_prep_paged_kernel<A, I><<<dim3(p->n_rows, per_row), 256, (size_t)4 * dim * sizeof(float), as_stream(stream)>>>(
+          static_cast<const I*>(p->proj), p->proj_stride, p->q_off, p->k_off, p->v_off, heads, kv_heads, dim, p->vdim,
+          static_cast<const A*>(p->q_norm), static_cast<const A*>(p->k_norm), p->eps, p->inv_freq, p->rot_dims, p->positions, p->row_entry,
+          p->page_indptr, p->page_ids, static_cast<A*>(p->cache), p->page_stride, p->k_cache_off, p->v_cache_off, p->page_size, p->q_out,
+          static_cast<A*>(p->q_out_stored), static_cast<const A*>(p->q_bias), static_cast<const A*>(p->k_bias),
+          static_cast<const A*>(p->v_bias), p->qt_coef, p->qt_every, pf);
     });
   });
   return known && ok ? (pegainfer_status_t)hipGetLastError() : PK_BAD;
@@ -831,7 +874,8 @@ pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cac
   if (n_split < 1) n_split = 1;
   if (n_split > 1 && (!workspace || n_split > 64)) return PK_BAD;
   if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || dim <= 0 || (maps != 1 && maps != 2) || maps * dim > 256 || vdim <= 0 ||
-      vdim > 256 || page_size <= 0 || kv_heads > 65535 || block < 0)
+      vdim > 256 || page_size <= 0 || kv_heads > 65535 || block < 0 || opt->shared_tail < 0 || opt->shared_tail > dim ||
+      (opt->shared_tail > 0 && (maps != 1 || vdim != dim)))
     return PK_BAD;
   const int qd = maps * dim;
   const size_t smem = ((size_t)kAttKeys * (qd + 1) + (size_t)kAttKeys * vdim + (size_t)kAttRows * qd + 4 * maps * 64 * kAttRpw) * sizeof(float);
@@ -851,6 +895,7 @@ pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cac
   form.gate = opt->gate;
   form.gate_stride = opt->gate_stride;
   form.gate_kind = gate_kind;
+  form.k_keep = qd - opt->shared_tail;
   bool ok = true;
   if (dtype == kDtBf16 && !plain) {   // bf16 cache: the matrix-core kernel; same tiles, same splits, same merge
     const int ncb = vdim <= 32 ? 2 : vdim <= 64 ? 4 : vdim <= 128 ? 8 : 16;

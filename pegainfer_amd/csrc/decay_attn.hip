@@ -16,11 +16,10 @@
 #include "common.h"
 #include "typed.h"
 #include "recurrent_core.h"
+#include "chunk_core.h"
 #include "pegainfer_kernels_blocks.h"
 
 namespace pk {
-
-constexpr int kDecayChunk = PEGAINFER_DECAY_CHUNK;
 
 template <typename A>
 struct DecayIn {
@@ -92,48 +91,6 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(DecayIn<A> in, const fl
   }
 }
 
-// A chunk's rows of one head into LDS (fp32, activated), rows past `n` and columns past `dim` as zeros; TPR threads per row, four
-// loads of eight values in flight per thread.
-template <int TPR, typename A>
-__device__ __forceinline__ void stage_rows(const DecayIn<A>& in, int64_t off, int row0, int n, int dim, int padded, float* dst, int stride,
-                                           const float* row_factor, int tid) {
-  const int j = tid / TPR, sub = tid % TPR;
-  const A* src = in.proj + (int64_t)(row0 + min(j, n - 1)) * in.stride + off;
-  const float f = j < n ? (row_factor ? row_factor[j] : 1.0f) : 0.f;
-  const bool vec = (dim & 7) == 0 && (off & 7) == 0 && (in.stride & 7) == 0 && aligned16(in.proj);
-  float* d = dst + j * stride;
-  for (int c0 = sub * 8; c0 < padded; c0 += 32 * TPR) {
-    float t[4][8];
-#pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      const int c = c0 + 8 * TPR * k;
-      if (vec) {
-        Vec8<A>::load(src + (c < dim ? c : 0), t[k]);      // always in bounds; what lies past dim or n becomes zero below
-      } else {
-#pragma unroll
-        for (int u = 0; u < 8; ++u) t[k][u] = ld(src + (c + u < dim ? c + u : 0));
-      }
-    }
-#pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      const int c = c0 + 8 * TPR * k;
-      if (c >= padded) break;
-#pragma unroll
-      for (int u = 0; u < 8; ++u) t[k][u] = j < n && c + u < dim ? in.act(t[k][u]) * f : 0.f;
-      *reinterpret_cast<f32x4*>(d + c) = f32x4{t[k][0], t[k][1], t[k][2], t[k][3]};
-      *reinterpret_cast<f32x4*>(d + c + 4) = f32x4{t[k][4], t[k][5], t[k][6], t[k][7]};
-    }
-  }
-}
-
-// LDS row strides (floats, multiples of 4): a fragment read of 4 rows x 16 columns wants rows 16 banks apart, one of 16 rows x 4
-// columns (and one of rows 4 apart x 16 columns) wants an odd multiple of 4
-__host__ __device__ constexpr int pad16(int n) { return (n + 15) & ~15; }
-__host__ __device__ constexpr int stride_rows4(int n) { return pad16(n) % 32 == 0 ? pad16(n) + 16 : pad16(n); }
-__host__ __device__ constexpr int stride_rows16(int n) { return pad16(n) + 4; }
-// value columns of the workspace and of the staged values: what the kernels' 16-column blocks cover
-__host__ __device__ constexpr int pad_values(int vdim) { return vdim <= 32 ? 32 : vdim <= 64 ? 64 : vdim <= 128 ? 128 : 256; }
-
 // U_c[d][col] = sum_i g^(n-1-i) k_i[d] v_i[col]; one workgroup per (chunk, head), a wave per block of 16 rows x (16 NB) columns of U
 template <typename A, int NB>
 __global__ __launch_bounds__(512) void decay_chunk_sum_kernel(DecayIn<A> in, const float* __restrict__ decay_pow, int pow_n,
@@ -146,10 +103,11 @@ __global__ __launch_bounds__(512) void decay_chunk_sum_kernel(DecayIn<A> in, con
   const int row0 = chunk_row0[c], n = chunk_rows[c];
   const int dp = pad16(dim), vp = pad_values(vdim), sk = stride_rows4(dim), sv = stride_rows4(vp);
   float *s_k = sm, *s_v = sm + kDecayChunk * sk;
+  auto act = [=](float x) { return in.act(x); };
   if (tid < kDecayChunk) s_f[tid] = tid < n ? decay_pow[(int64_t)h * pow_n + n - 1 - tid] : 0.f;
   __syncthreads();
-  stage_rows<8>(in, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sk, s_f, tid);
-  stage_rows<8>(in, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid);
+  stage_rows<8>(in.proj, in.stride, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sk, s_f, tid, act);
+  stage_rows<8>(in.proj, in.stride, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid, act);
   __syncthreads();
   float* U = ws + ((int64_t)c * H + h) * dp * vp;
   const int steps = (n + 3) >> 2, col_blocks = vp / (16 * NB), blocks = (dp >> 4) * col_blocks;
@@ -215,10 +173,11 @@ __global__ __launch_bounds__(512) void decay_chunk_out_kernel(DecayIn<A> in, con
   const int dp = pad16(dim), sq = stride_rows16(dim);
   float *s_q = sm, *s_k = s_q + kDecayChunk * sq, *s_v = s_k + kDecayChunk * sq;
   const int half = wave >> 2, rb = half ? 3 - (wave & 3) : wave & 3, i0 = rb * 16, c0 = half * 16 * NB;
+  auto act = [=](float x) { return in.act(x); };
   if (tid <= kDecayChunk) s_pow[tid] = tid <= n ? decay_pow[(int64_t)h * pow_n + tid] : 0.f;
-  stage_rows<8>(in, in.q_off + (int64_t)h * dim, row0, n, dim, dp, s_q, sq, nullptr, tid);
-  stage_rows<8>(in, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sq, nullptr, tid);
-  stage_rows<8>(in, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid);
+  stage_rows<8>(in.proj, in.stride, in.q_off + (int64_t)h * dim, row0, n, dim, dp, s_q, sq, nullptr, tid, act);
+  stage_rows<8>(in.proj, in.stride, in.k_off + (int64_t)h * dim, row0, n, dim, dp, s_k, sq, nullptr, tid, act);
+  stage_rows<8>(in.proj, in.stride, in.v_off + (int64_t)h * vdim, row0, n, vdim, vp, s_v, sv, nullptr, tid, act);
   __syncthreads();
   if (i0 >= n) return;                               // no barrier follows
   const int my_i = i0 + l15;                         // the query this lane holds scores of
@@ -283,7 +242,6 @@ __global__ __launch_bounds__(512) void decay_chunk_out_kernel(DecayIn<A> in, con
 
 static size_t decay_sum_lds(int dim, int vdim) { return (size_t)kDecayChunk * (stride_rows4(dim) + stride_rows4(pad_values(vdim))) * sizeof(float); }
 static size_t decay_out_lds(int dim, int vdim) { return (size_t)kDecayChunk * (2 * stride_rows16(dim) + stride_rows16(pad_values(vdim))) * sizeof(float); }
-constexpr size_t kLdsMost = 159 * 1024;              // beside the kernels' static tables
 
 }  // namespace pk
 
@@ -321,13 +279,8 @@ pegainfer_status_t pegainfer_decay_attention(const pegainfer_decay_attention_des
             in, q->decay_pow, q->pow_n, q->state, q->slot_stride, q->o, H, dim, vdim, q->entry_row0, q->entry_slot, chunks ? q->scan_max : 0);
       });
     if (!ok || !chunks) return;
-    auto lds = [&](auto kern, size_t bytes) {
-      if (bytes > 48 * 1024)
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
-      return bytes;
-    };
     auto sums = [&](auto kern) {
-      kern<<<dim3(q->n_chunks, H), 512, lds(kern, decay_sum_lds(dim, vdim)), st>>>(in, q->decay_pow, q->pow_n, q->workspace, H, dim, vdim,
+      kern<<<dim3(q->n_chunks, H), 512, with_lds(kern, decay_sum_lds(dim, vdim)), st>>>(in, q->decay_pow, q->pow_n, q->workspace, H, dim, vdim,
                                                                                   q->chunk_row0, q->chunk_rows);
     };
     if (vdim <= 32) sums(decay_chunk_sum_kernel<A, 2>);
@@ -335,7 +288,7 @@ pegainfer_status_t pegainfer_decay_attention(const pegainfer_decay_attention_des
     decay_chunk_state_kernel<<<dim3(ceil_div((long)dim * vdim, 256), H, q->n_long), 256, 0, st>>>(
         q->decay_pow, q->pow_n, q->workspace, q->state, q->slot_stride, H, dim, vdim, q->chunk_rows, q->long_chunk0, q->long_slot);
     auto out = [&](auto kern) {
-      kern<<<dim3(q->n_chunks, H), 512, lds(kern, decay_out_lds(dim, vdim)), st>>>(in, q->decay_pow, q->pow_n, q->workspace, q->o, H, dim, vdim,
+      kern<<<dim3(q->n_chunks, H), 512, with_lds(kern, decay_out_lds(dim, vdim)), st>>>(in, q->decay_pow, q->pow_n, q->workspace, q->o, H, dim, vdim,
                                                                                   q->chunk_row0, q->chunk_rows);
     };
     if (vdim <= 32) out(decay_chunk_out_kernel<A, 1>);

@@ -89,6 +89,7 @@ __global__ __launch_bounds__(256) void gemm_strided_kernel(pegainfer_gemm_desc d
       if (m0 + tm + j >= d.m) continue;
       float v = acc[i][j];
       if (d.epilogue == PEGAINFER_EPI_RELU_SQ) { v = fmaxf(v, 0.f); v *= v; }
+      else if (d.epilogue == PEGAINFER_EPI_GELU_ERF) v = gelu_erf_f(v);
       else if (d.epilogue == PEGAINFER_EPI_SIGMOID_GATE) v *= scale;
       st(Y + (int64_t)dst * d.y_row_stride + m0 + tm + j, v);
     }
@@ -208,6 +209,7 @@ __global__ __launch_bounds__(256) void gemm_strided_mfma_kernel(pegainfer_gemm_d
         if (m >= d.m) continue;
         float v = acc[i][j][e];
         if (d.epilogue == PEGAINFER_EPI_RELU_SQ) { v = fmaxf(v, 0.f); v *= v; }
+        else if (d.epilogue == PEGAINFER_EPI_GELU_ERF) v = gelu_erf_f(v);
         else if (d.epilogue == PEGAINFER_EPI_SIGMOID_GATE) v *= scale;
         st(Y + (int64_t)dst * d.y_row_stride + m, v);
       }
@@ -322,6 +324,7 @@ __global__ __launch_bounds__(256) void gemm_strided_rows_kernel(pegainfer_gemm_d
           if (yrow[r] < 0) continue;
           float v = acc[n][q][r];
           if (d.epilogue == PEGAINFER_EPI_RELU_SQ) { v = fmaxf(v, 0.f); v *= v; }
+          else if (d.epilogue == PEGAINFER_EPI_GELU_ERF) v = gelu_erf_f(v);
           else if (d.epilogue == PEGAINFER_EPI_SIGMOID_GATE)
             v *= sigmoid_f(ld(static_cast<const TG*>(d.gate) + (int64_t)xrow[r] * d.gate_row_stride + g));
           st(Y + (int64_t)yrow[r] * d.y_row_stride + m, v);

@@ -16,6 +16,7 @@
 #include "pegainfer_ramalix.h"
 #include "pegainfer_kukulorn.h"
 #include "pegainfer_zofadra.h"
+#include "pegainfer_sopanex.h"
 #include "pegainfer_scheduler.h"
 
 namespace psched {
@@ -307,6 +308,7 @@ PEGAINFER_STEP_API(FeruzenApi, pegainfer_feruzen);
 PEGAINFER_STEP_API(RamalixApi, pegainfer_ramalix);
 PEGAINFER_STEP_API(KukulornApi, pegainfer_kukulorn);
 PEGAINFER_STEP_API(ZofadraApi, pegainfer_zofadra);
+PEGAINFER_STEP_API(SopanexApi, pegainfer_sopanex);
 
 template <class Api>
 struct StepExec {
@@ -374,6 +376,7 @@ using FeruzenExec = StepExec<FeruzenApi>;
 using RamalixExec = StepExec<RamalixApi>;
 using KukulornExec = StepExec<KukulornApi>;
 using ZofadraExec = StepExec<ZofadraApi>;
+using SopanexExec = StepExec<SopanexApi>;
 
 struct Scheduler {
   pegainfer_executor_vtbl ex;
@@ -384,6 +387,7 @@ struct Scheduler {
   RamalixExec* owned_rx = nullptr;
   KukulornExec* owned_kk = nullptr;
   ZofadraExec* owned_zf = nullptr;
+  SopanexExec* owned_sx = nullptr;
   Rng rng;
   std::vector<Active> active;
   std::vector<Pending> deferred;
@@ -705,6 +709,19 @@ pegainfer_sched_t pegainfer_sched_create_zofadra(void* model, uint64_t seed, con
   s->owned_zf = e;
   return s;
 }
+pegainfer_sched_t pegainfer_sched_create_sopanex(void* model, uint64_t seed, const uint32_t* stop_tokens, int32_t n_stop) {
+  if (!model) return nullptr;
+  auto* e = new psched::SopanexExec();
+  e->model = model;
+  for (int i = 0; i < n_stop; ++i) e->stop.insert(stop_tokens[i]);
+  pegainfer_executor_vtbl v{sizeof(pegainfer_executor_vtbl), e, &psched::SopanexExec::page_size, &psched::SopanexExec::max_request_pages,
+                            &psched::SopanexExec::available_pages, &psched::SopanexExec::is_stop_token,
+                            &psched::SopanexExec::drop_request, &psched::SopanexExec::execute, &psched::SopanexExec::last_error,
+                            &psched::SopanexExec::max_batch_size, &psched::SopanexExec::logprobs, nullptr, nullptr};
+  Scheduler* s = static_cast<Scheduler*>(pegainfer_sched_create(&v, seed));
+  s->owned_sx = e;
+  return s;
+}
 void pegainfer_sched_destroy(pegainfer_sched_t s) {
   if (!s) return;
   delete SC(s)->owned;
@@ -714,6 +731,7 @@ void pegainfer_sched_destroy(pegainfer_sched_t s) {
   delete SC(s)->owned_rx;
   delete SC(s)->owned_kk;
   delete SC(s)->owned_zf;
+  delete SC(s)->owned_sx;
   delete SC(s);
 }
 uint64_t pegainfer_sched_submit_ex(pegainfer_sched_t s, const uint32_t* prompt_tokens, int32_t n_tokens, int32_t max_tokens,

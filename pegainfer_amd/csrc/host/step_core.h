@@ -1,9 +1,10 @@
-// What a host runtime with ONE batched step function needs besides its layers (include/pegainfer_zofadra.h is the first user; the
-// runtimes beside it carry their own copies): device memory, checkpoint tensors waiting to be uploaded, request slots over the
+// What a host runtime with ONE batched step function needs besides its layers (include/pegainfer_zofadra.h and include/pegainfer_sopanex.h
+// use it; the older runtimes beside them carry their own copies): device memory, checkpoint tensors waiting to be uploaded, request slots over the
 // shared PagePool (kv_pool.h) and the fp32 state arena (seq_state.h), the step's packed metadata block with the tile tables its
 // attention launches read, decode steps captured as hipGraphs, logits, sampling, logprobs, the per-layer stream tap - and the
 // C entry points over all of that (PEGAINFER_STEP_ENTRIES).  A model derives from StepModel, parses its own layers and provides
 //   parse(config)      sizes; add_cache() / state_layout.reserve() for what a request holds; *_tiles() for its launches' tables
+//   resolve_sizes(f)   sizes that only the checkpoint's tensors tell (optional)
 //   tensor_list()      names and shapes of the checkpoint
 //   synthetic(...)     one weight of a seeded random model
 //   build_weights()    staged tensors -> device
@@ -18,6 +19,7 @@
 #include <cstdio>
 #include <cstdlib>
 #include <cstring>
+#include <functional>
 #include <map>
 #include <string>
 #include <vector>
@@ -95,6 +97,7 @@ struct StepCtx {
   int T = 0, n = 0, W = 0;         // token rows, entries, wanted rows
   bool single = false;             // every entry brings one token: decoding
   const uint32_t* tokens = nullptr;
+  const int32_t* prev = nullptr;   // a row's previous token in its sequence, -1 for the first
   const int32_t *pos = nullptr, *entry = nullptr, *row0 = nullptr, *slot = nullptr, *page_indptr = nullptr, *want = nullptr, *pages = nullptr;
   std::vector<TileTable> group_tiles, flat_tiles;
   ChunkTable chunks;
@@ -109,6 +112,7 @@ class StepModel {
   std::string err;
   PagePool pool{0};
   std::vector<KvState> requests;
+  std::vector<int32_t> last_token;     // of every request slot, -1 before its first
   pq::StateLayout state_layout;
   int64_t weight_bytes = 0;
   float last_step_ms = 0.f;
@@ -132,6 +136,9 @@ class StepModel {
   virtual const char* architecture() const = 0;
   virtual int parse(const Json& config) = 0;
   virtual int layer_runs() const = 0;
+  // sizes the configuration leaves to the tensors: numel_of gives a tensor's element count, 0 while it is unknown (a model of
+  // synthetic weights then picks a size of its own).  Called before tensor_list() is used and before the weights are built.
+  virtual int resolve_sizes(const std::function<int64_t(const std::string&)>&) { return 0; }
   virtual TensorList tensor_list() const = 0;
   virtual float synthetic(const std::string& name, float z, float std) const = 0;   // z: a draw of unit variance
   virtual int build_weights() = 0;
@@ -158,6 +165,7 @@ class StepModel {
     num_pages = std::max(1, (max_tokens + kPageSize - 1) / kPageSize);
     pool = PagePool(num_pages);
     requests.assign((size_t)max_requests, KvState());
+    last_token.assign((size_t)max_requests, -1);
     if (dalloc_a(&cache, (size_t)num_pages * (size_t)page_stride)) return -1;
     if (dalloc(&state, (size_t)max_requests * (size_t)std::max<int64_t>(1, state_layout.floats_per_slot()))) return -1;
     return dalloc(&probs_scratch, (size_t)V) || dalloc(&top1_value, 1) || dalloc(&row_states, 1024 * 1024) ||
@@ -181,6 +189,7 @@ class StepModel {
       const float u = (float)(z & 0xFFFF) + (float)((z >> 16) & 0xFFFF) + (float)((z >> 32) & 0xFFFF) + (float)(z >> 48);
       return (u * (1.0f / 65536.0f) - 2.0f) * 1.7320508f;
     };
+    if (resolve_sizes([](const std::string&) { return (int64_t)0; })) return -1;
     for (auto& t : tensor_list()) {
       std::vector<uint16_t>& v = staged[t.first];
       v.resize((size_t)numel(t.second));
@@ -192,6 +201,8 @@ class StepModel {
     pst::Checkpoint ck;
     std::string e;
     if (!ck.open(path, &e)) return set_error(e);
+    if (resolve_sizes([&ck](const std::string& n) { const pst::TensorView* v = ck.find(n); return v ? (int64_t)v->numel() : (int64_t)0; }))
+      return -1;
     for (auto& t : tensor_list()) {
       const pst::TensorView* v = ck.find(t.first);
       if (!v) return set_error("checkpoint has no tensor " + t.first);
@@ -211,6 +222,8 @@ class StepModel {
   }
   int finalize() {
     if (finalized) return 0;
+    if (resolve_sizes([this](const std::string& n) { const auto it = staged.find(n); return it == staged.end() ? (int64_t)0 : (int64_t)it->second.size(); }))
+      return -1;
     if (build_weights()) return -1;
     staged.clear();
     finalized = true;
@@ -225,6 +238,7 @@ class StepModel {
         if (n) PSTEP_HIP(hipMemsetAsync(state + i * n, 0, n * sizeof(float), stream));   // a request's state starts from zero
         requests[i].live = true;
         requests[i].seq_len = 0;
+        last_token[i] = -1;
         return (int)i;
       }
     return set_error("no free request slot");
@@ -276,7 +290,7 @@ class StepModel {
     std::vector<int32_t>& mb = meta;
     mb.clear();
     auto open = [&](size_t len) { const size_t at = mb.size(); mb.resize(at + len); return at; };
-    const size_t o_tok = open(T), o_pos = open(T), o_ent = open(T), o_row0 = open((size_t)n + 1), o_slot = open((size_t)n),
+    const size_t o_tok = open(T), o_prev = open(T), o_pos = open(T), o_ent = open(T), o_row0 = open((size_t)n + 1), o_slot = open((size_t)n),
                  o_ind = open((size_t)n + 1), o_want = open((size_t)std::max(1, W));
     StepCtx c;
     c.T = (int)T; c.n = n; c.W = W;
@@ -292,6 +306,7 @@ class StepModel {
         pg += st.pages.size();
         for (int k = 0; k < lens[i]; ++k, ++t) {
           mb[o_tok + t] = (int32_t)tokens[t];
+          mb[o_prev + t] = k ? (int32_t)tokens[t - 1] : last_token[ids[i]];
           mb[o_pos + t] = st.seq_len + k;
           mb[o_ent + t] = i;
         }
@@ -313,7 +328,7 @@ class StepModel {
     PSTEP_HIP(hipMemcpyAsync(meta_dev, meta_host, mb.size() * 4, hipMemcpyHostToDevice, stream));
     const int32_t* md = reinterpret_cast<const int32_t*>(meta_dev);
     c.tokens = reinterpret_cast<const uint32_t*>(md + o_tok);
-    c.pos = md + o_pos; c.entry = md + o_ent; c.row0 = md + o_row0; c.slot = md + o_slot; c.page_indptr = md + o_ind;
+    c.prev = md + o_prev; c.pos = md + o_pos; c.entry = md + o_ent; c.row0 = md + o_row0; c.slot = md + o_slot; c.page_indptr = md + o_ind;
     c.want = md + o_want; c.pages = md + o_pages;
     for (auto& g : group_at) c.group_tiles.push_back(TileTable{md + g.first, g.second});
     for (auto& f : flat_at) c.flat_tiles.push_back(TileTable{md + f.first, f.second});
@@ -359,7 +374,11 @@ class StepModel {
     if (W > 0 && out_tokens) PSTEP_HIP(hipMemcpyAsync(out_tokens, tokens_d, (size_t)W * 4, hipMemcpyDeviceToHost, stream));
     PSTEP_HIP(hipStreamSynchronize(stream));
     (void)hipEventElapsedTime(&last_step_ms, ev0, ev1);
-    for (int i = 0; i < n; ++i) requests[ids[i]].seq_len += lens[i];
+    for (int i = 0, t = 0; i < n; ++i) {
+      t += lens[i];
+      requests[ids[i]].seq_len += lens[i];
+      last_token[ids[i]] = (int32_t)tokens[t - 1];
+    }
     return 0;
   }
 
@@ -485,6 +504,16 @@ class StepModel {
     }
     return upload(out, st.data(), st.size());
   }
+  // [rows, cols_i] tensors side by side, each part's first column at the given column (Part.rows = its columns), zeros between and after
+  int up_beside(void** out, const std::vector<Part>& parts, int64_t rows, int64_t total_cols) {
+    std::vector<uint16_t> st((size_t)(rows * total_cols), 0);
+    for (auto& p : parts) {
+      const auto* v = need(p.name, rows * p.rows);
+      if (!v) return -1;
+      for (int64_t r = 0; r < rows; ++r) std::memcpy(&st[(size_t)(r * total_cols + p.at)], v->data() + r * p.rows, (size_t)p.rows * 2);
+    }
+    return upload(out, st.data(), st.size());
+  }
   // [groups][rows][cols] transposed group by group to [groups][cols][rows]
   int up_transposed(void** out, const std::string& name, int groups, int rows, int cols) {
     const auto* v = need(name, (int64_t)groups * rows * cols);
@@ -501,6 +530,37 @@ class StepModel {
     for (int k = 0; k < dims / 2; ++k) f[k] = (float)std::pow(base, -2.0 * k / (double)dims);
     return f;
   }
+  // Long-context scaling by a ramp over the dimensions: pairs whose wave turns more than `fast` times over `original` positions keep
+  // their frequency, those that turn fewer than `slow` times have it divided by `factor`, the ones between are mixed linearly; every
+  // cosine and sine is multiplied by amplitude().
+  struct RampScaling {
+    bool on = false;
+    double factor = 1.0, original = 1.0, fast = 1.0, slow = 1.0;
+    bool ok() const { return factor > 0.0 && original > 0.0 && fast > 0.0 && slow > 0.0; }
+    float amplitude() const { return on ? (float)(0.1 * std::log(factor) + 1.0) : 1.0f; }
+  };
+  static RampScaling parse_ramp(const Json* j) {
+    RampScaling r;
+    r.on = j && j->kind == Json::Obj;
+    if (r.on) {
+      r.factor = j->number_or("factor", 1.0);
+      r.original = j->number_or("original", 0.0);
+      r.fast = j->number_or("fast", 32.0);
+      r.slow = j->number_or("slow", 1.0);
+    }
+    return r;
+  }
+  static std::vector<float> rotation_frequencies(double base, int dims, const RampScaling& r) {
+    if (!r.on) return rotation_frequencies(base, dims);
+    auto dim_of = [&](double turns) { return dims * std::log(r.original / (2.0 * M_PI * turns)) / (2.0 * std::log(base)); };
+    const double lo = std::max(std::floor(dim_of(r.fast)), 0.0), hi = std::min(std::ceil(dim_of(r.slow)), (double)dims - 1.0);
+    std::vector<float> f((size_t)std::max(1, dims / 2));
+    for (int k = 0; k < dims / 2; ++k) {
+      const double w = std::pow(base, -2.0 * k / (double)dims), t = std::min(std::max((k - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+      f[k] = (float)(w / r.factor * t + w * (1.0 - t));
+    }
+    return f;
+  }
 
   // Y[T, M] = X[T, K] W[M, K]^T in the model's storage type
   int linear(const void* W, const void* X, void* Y, int M, int T, int K) {
@@ -511,12 +571,14 @@ class StepModel {
     return linear_strided(W, X, dtype, K, Y, dtype, M, T, K);
   }
   // the same through the strided GEMM: operands that are columns of a wider matrix, outputs that stay in fp32
-  int linear_strided(const void* W, const void* X, int x_dtype, int64_t x_stride, void* Y, int y_dtype, int M, int T, int K) {
+  int linear_strided(const void* W, const void* X, int x_dtype, int64_t x_stride, void* Y, int y_dtype, int M, int T, int K,
+                     int epilogue = PEGAINFER_EPI_NONE) {
     pegainfer_gemm_desc d{};
     d.x = X; d.w = W; d.y = Y;
     d.x_dtype = x_dtype; d.w_dtype = dtype; d.y_dtype = y_dtype;
     d.m = M; d.k = K; d.rows = T; d.groups = 1;
     d.x_row_stride = x_stride; d.w_m_stride = K; d.w_k_stride = 1; d.y_row_stride = M;
+    d.epilogue = epilogue;
     d.plain = plain_kernels;
     PSTEP_K(pegainfer_gemm_strided(&d, S()));
     return 0;

@@ -11,7 +11,9 @@
 //   combine_kernel  out[row] = sum over the row's choices, in choice order, of weight * expert output (fp32 sum), plus a row
 //                   every token gets (a shared expert), optionally times the sigmoid of a per-row gate logit.
 // Options of the selection: a group's score = its two largest choices (default) or its largest; the chosen weights as they
-// are (default) or divided by their sum.
+// are (default) or divided by their sum, times a factor.  Expert numbers past the experts that have tensors are identity experts:
+// they get no position in the sort, and the combine takes the feed-forward's input row for them.
+//   route_plan_kernel  selection and sort in one launch for steps of few rows
 #include <algorithm>
 
 #include "common.h"
@@ -26,7 +28,8 @@ namespace pk {
 template <typename A>
 __device__ __forceinline__ void route_select_wave(float* s, float* ch, float* gs, const A* __restrict__ corr,
                                                   int32_t* __restrict__ out_e, float* __restrict__ out_w, int row, int lane, int E,
-                                                  int G, int keep, int top, int score, int group_kind = 0, int renorm = 0) {
+                                                  int G, int keep, int top, int score, int group_kind = 0, int renorm = 0,
+                                                  float factor = 1.0f) {
   if (score == PEGAINFER_SCORE_SOFTMAX) {            // s = exp(z - max) / sum over ALL experts, then the choice scores
     float mx = -INFINITY;
     for (int e = lane; e < E; e += 64) mx = fmaxf(mx, s[e]);
@@ -85,10 +88,10 @@ __device__ __forceinline__ void route_select_wave(float* s, float* ch, float* gs
     }
     __builtin_amdgcn_wave_barrier();
   }
-  if (renorm && lane == 0) {   // the chosen weights divided by their sum (in choice order)
+  if ((renorm || factor != 1.0f) && lane == 0) {   // the chosen weights divided by their sum (in choice order), times the factor
     float sum = 0.f;
     for (int k = 0; k < top; ++k) sum += out_w[(size_t)row * top + k];
-    const float inv = 1.0f / (sum + 1e-20f);
+    const float inv = factor * (renorm ? 1.0f / (sum + 1e-20f) : 1.0f);
     for (int k = 0; k < top; ++k) out_w[(size_t)row * top + k] *= inv;
   }
 }
@@ -144,71 +147,110 @@ __global__ __launch_bounds__(256) void route_kernel(const A* __restrict__ h, con
   route_select_wave(s, ch, gs, corr, out_e, out_w, row, lane, E, G, keep, top, score);
 }
 
-// The same selection from router logits that a GEMM has left in fp32 ([rows][E]): a wave per row, four rows per workgroup.
+// The same selection from router logits that a GEMM has left in fp32 ([rows][E] at a stride), by one wave with LDS of its own.
+struct RouteForm {
+  int E, G, keep, top, score, group_kind, renorm;
+  float factor;
+  int64_t logits_stride;
+};
 template <typename A>
-__global__ __launch_bounds__(256) void route_from_logits_kernel(const float* __restrict__ logits, const A* __restrict__ corr,
-                                                                int32_t* __restrict__ out_e, float* __restrict__ out_w, int E,
-                                                                int G, int keep, int top, int rows, int score,
-                                                                int64_t logits_stride, int group_kind, int renorm) {
-  extern __shared__ float sm[];
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int row = blockIdx.x * 4 + wave;
-  if (row >= rows) return;
-  float* s = sm + wave * (2 * E + G);
-  float* ch = s + E;
-  float* gs = s + 2 * E;
-  for (int e = lane; e < E; e += 64) {
-    const float z = logits[(size_t)row * logits_stride + e];
-    const float sc = score == PEGAINFER_SCORE_SOFTMAX ? z : sigmoid_f(z);
+__device__ __forceinline__ void route_row_from_logits(const float* __restrict__ logits, const A* __restrict__ corr, int32_t* out_e,
+                                                      float* out_w, const RouteForm& f, int row, int lane, float* s) {
+  float *ch = s + f.E, *gs = s + 2 * f.E;
+  for (int e = lane; e < f.E; e += 64) {
+    const float z = logits[(size_t)row * f.logits_stride + e];
+    const float sc = f.score == PEGAINFER_SCORE_SOFTMAX ? z : sigmoid_f(z);
     s[e] = sc;
     ch[e] = corr ? sc + ld(corr + e) : sc;
   }
   __builtin_amdgcn_wave_barrier();
-  route_select_wave(s, ch, gs, corr, out_e, out_w, row, lane, E, G, keep, top, score, group_kind, renorm);
+  route_select_wave(s, ch, gs, corr, out_e, out_w, row, lane, f.E, f.G, f.keep, f.top, f.score, f.group_kind, f.renorm, f.factor);
+}
+// a wave per row, four rows per workgroup
+template <typename A>
+__global__ __launch_bounds__(256) void route_from_logits_kernel(const float* __restrict__ logits, const A* __restrict__ corr,
+                                                                int32_t* __restrict__ out_e, float* __restrict__ out_w, int rows,
+                                                                RouteForm f) {
+  extern __shared__ float sm[];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int row = blockIdx.x * 4 + wave;
+  if (row >= rows) return;
+  route_row_from_logits(logits, corr, out_e, out_w, f, row, lane, sm + wave * (2 * f.E + f.G));
 }
 
-__global__ __launch_bounds__(256) void route_sort_kernel(const int32_t* __restrict__ expert, int n_pairs, int top, int E,
-                                                         int32_t* __restrict__ pos_pair, int32_t* __restrict__ pos_row,
-                                                         int32_t* __restrict__ tile_group, int32_t* __restrict__ tile_row0,
-                                                         int32_t* __restrict__ tile_rows, int32_t* __restrict__ n_tiles,
-                                                         int max_tiles, int per_tile) {
-  extern __shared__ int cnt[];   // [E] counts, then [E] cursors
-  int* cur = cnt + E;
+struct SortOut {
+  int32_t *pos_pair, *pos_row, *tile_group, *tile_row0, *tile_rows, *n_tiles;
+  int max_tiles, per_tile;
+};
+// Pairs whose expert number is E or more (identity experts) get no position.  One workgroup; cnt: [2 E] of LDS.
+__device__ __forceinline__ void route_sort_block(const int32_t* expert, int n_pairs, int top, int E, const SortOut& o, int* cnt) {
+  int* cur = cnt + E;            // [E] counts, then [E] cursors
   for (int e = threadIdx.x; e < E; e += 256) cnt[e] = 0;
   __syncthreads();
-  for (int p = threadIdx.x; p < n_pairs; p += 256) atomicAdd(&cnt[expert[p]], 1);
+  for (int p = threadIdx.x; p < n_pairs; p += 256) {
+    const int e = expert[p];
+    if (e < E) atomicAdd(&cnt[e], 1);
+  }
   __syncthreads();
   if (threadIdx.x == 0) {
     int off = 0, nt = 0;
     for (int e = 0; e < E; ++e) {
       const int c = cnt[e];
       cur[e] = off;
-      for (int r0 = 0; r0 < c && nt < max_tiles; r0 += per_tile, ++nt) {
-        tile_group[nt] = e;
-        tile_row0[nt] = off + r0;
-        tile_rows[nt] = min(per_tile, c - r0);
+      for (int r0 = 0; r0 < c && nt < o.max_tiles; r0 += o.per_tile, ++nt) {
+        o.tile_group[nt] = e;
+        o.tile_row0[nt] = off + r0;
+        o.tile_rows[nt] = min(o.per_tile, c - r0);
       }
       off += c;
     }
-    *n_tiles = nt;
+    *o.n_tiles = nt;
   }
   __syncthreads();
   for (int p = threadIdx.x; p < n_pairs; p += 256) {
-    const int at = atomicAdd(&cur[expert[p]], 1);
-    pos_pair[at] = p;
-    pos_row[at] = p / top;
+    const int e = expert[p];
+    if (e >= E) continue;
+    const int at = atomicAdd(&cur[e], 1);
+    o.pos_pair[at] = p;
+    o.pos_row[at] = p / top;
   }
 }
+__global__ __launch_bounds__(256) void route_sort_kernel(const int32_t* __restrict__ expert, int n_pairs, int top, int E, SortOut o) {
+  extern __shared__ int cnt[];
+  route_sort_block(expert, n_pairs, top, E, o, cnt);
+}
+// Few rows (decoding): selection and sort in one launch of one workgroup, which sees its own choices after a barrier.
+template <typename A>
+__global__ __launch_bounds__(256) void route_plan_kernel(const float* __restrict__ logits, const A* __restrict__ corr, int32_t* out_e,
+                                                         float* out_w, int rows, RouteForm f, int sort_experts, SortOut o) {
+  extern __shared__ float sm[];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  for (int row = wave; row < rows; row += 4) {
+    route_row_from_logits(logits, corr, out_e, out_w, f, row, lane, sm + wave * (2 * f.E + f.G));
+    __builtin_amdgcn_wave_barrier();
+  }
+  __threadfence_block();
+  __syncthreads();               // the choices are read by other waves of this workgroup; the selection's LDS is free
+  route_sort_block(out_e, rows * f.top, f.top, sort_experts, o, reinterpret_cast<int*>(sm));
+}
 
+// expert / same: pairs that chose an expert number of same_from or more take the row of `same` (the feed-forward's own input) instead
+// of a y_pairs row
 template <typename A>
 __global__ __launch_bounds__(256) void route_combine_kernel(const float* __restrict__ y, const float* __restrict__ w,
                                                             const A* __restrict__ add, A* __restrict__ out, int d, int top,
-                                                            const float* __restrict__ add_gate, int64_t add_gate_stride) {
+                                                            const float* __restrict__ add_gate, int64_t add_gate_stride,
+                                                            const int32_t* __restrict__ expert, int same_from,
+                                                            const A* __restrict__ same, int64_t same_stride) {
   const int row = blockIdx.x;
   const float gate = add && add_gate ? sigmoid_f(add_gate[(size_t)row * add_gate_stride]) : 1.0f;
   for (int i = blockIdx.y * 256 + threadIdx.x; i < d; i += gridDim.y * 256) {
     float a = add ? ld(add + (size_t)row * d + i) * gate : 0.f;
-    for (int c = 0; c < top; ++c) a = fmaf(w[(size_t)row * top + c], y[((size_t)row * top + c) * d + i], a);
+    for (int c = 0; c < top; ++c) {
+      const bool own = same && expert[(size_t)row * top + c] >= same_from;      // uniform over the workgroup
+      const float v = own ? ld(same + (size_t)row * same_stride + i) : y[((size_t)row * top + c) * d + i];
+      a = fmaf(w[(size_t)row * top + c], v, a);
+    }
     st(out + (size_t)row * d + i, a);
   }
 }
@@ -238,26 +280,51 @@ pegainfer_status_t pegainfer_route_topk(const void* h, const void* w_router, con
   return (pegainfer_status_t)hipGetLastError();
 }
 
+pegainfer_status_t pegainfer_route_plan(const pegainfer_route_plan_desc* q, pegainfer_stream_t stream) {
+  constexpr pegainfer_status_t bad = (pegainfer_status_t)hipErrorInvalidValue;
+  if (!q) return bad;
+  if (q->rows <= 0) return 0;
+  const int E = q->experts, groups = std::max(1, q->n_groups), keep = q->n_groups < 1 ? 1 : q->keep_groups, top = q->top;
+  if (!q->logits || !q->out_expert || !q->out_weight || E <= 0 || E % groups || top <= 0 || top > E || keep < 1 || keep > groups ||
+      q->logits_stride < E || (size_t)(2 * E + groups) * 16 > 60000 ||
+      (q->score_kind != PEGAINFER_SCORE_SIGMOID && q->score_kind != PEGAINFER_SCORE_SOFTMAX) ||
+      (q->group_kind != PEGAINFER_GROUP_TOP2_SUM && q->group_kind != PEGAINFER_GROUP_MAX))
+    return bad;
+  const int64_t pairs = (int64_t)q->rows * top;
+  const bool sorted = q->sort_experts > 0;
+  if (sorted && ((q->rows_per_tile != 64 && q->rows_per_tile != 128) || q->sort_experts > 7000 || pairs > 0x7FFFFFFF || !q->pos_pair ||
+                 !q->pos_row || !q->tile_group || !q->tile_row0 || !q->tile_rows || !q->n_tiles ||
+                 q->max_tiles < (pairs + q->rows_per_tile - 1) / q->rows_per_tile + q->sort_experts))
+    return bad;
+  const RouteForm f{E, groups, keep, top, q->score_kind, q->group_kind, q->renorm, q->factor, q->logits_stride};
+  const SortOut o{q->pos_pair, q->pos_row, q->tile_group, q->tile_row0, q->tile_rows, q->n_tiles, q->max_tiles, q->rows_per_tile};
+  const size_t smem = (size_t)4 * (2 * E + groups) * sizeof(float), sort_smem = (size_t)2 * std::max(0, q->sort_experts) * sizeof(int);
+  if (!by_dtype(q->dtype, [&](auto* t) {
+        using A = std::remove_pointer_t<decltype(t)>;
+        const A* corr = static_cast<const A*>(q->correction);
+        if (sorted && q->rows <= 16) {
+          route_plan_kernel<A><<<1, 256, std::max(smem, sort_smem), as_stream(stream)>>>(q->logits, corr, q->out_expert, q->out_weight,
+                                                                                        q->rows, f, q->sort_experts, o);
+          return;
+        }
+        route_from_logits_kernel<A><<<ceil_div(q->rows, 4), 256, smem, as_stream(stream)>>>(q->logits, corr, q->out_expert, q->out_weight,
+                                                                                            q->rows, f);
+        if (sorted)
+          route_sort_kernel<<<1, 256, sort_smem, as_stream(stream)>>>(q->out_expert, (int)pairs, top, q->sort_experts, o);
+      }))
+    return bad;
+  return (pegainfer_status_t)hipGetLastError();
+}
+
 pegainfer_status_t pegainfer_route_from_logits_ex(const float* logits, int64_t logits_stride, const void* correction,
                                                   int32_t* out_expert, float* out_weight, int32_t experts, int32_t n_groups,
                                                   int32_t keep_groups, int32_t top, int32_t rows, int32_t score_kind,
                                                   int32_t group_kind, int32_t renorm, int32_t dtype, pegainfer_stream_t stream) {
-  if (rows <= 0) return 0;
-  if (n_groups < 1) n_groups = 1;
-  if (experts <= 0 || experts % n_groups || top <= 0 || top > experts || keep_groups < 1 || keep_groups > n_groups ||
-      logits_stride < experts || (size_t)(2 * experts + n_groups) * 16 > 60000 ||
-      (score_kind != PEGAINFER_SCORE_SIGMOID && score_kind != PEGAINFER_SCORE_SOFTMAX) ||
-      (group_kind != PEGAINFER_GROUP_TOP2_SUM && group_kind != PEGAINFER_GROUP_MAX))
-    return (pegainfer_status_t)hipErrorInvalidValue;
-  const size_t smem = (size_t)4 * (2 * experts + n_groups) * sizeof(float);
-  if (!by_dtype(dtype, [&](auto* t) {
-        using A = std::remove_pointer_t<decltype(t)>;
-        route_from_logits_kernel<A><<<ceil_div(rows, 4), 256, smem, as_stream(stream)>>>(
-            logits, static_cast<const A*>(correction), out_expert, out_weight, experts, n_groups, keep_groups, top, rows, score_kind,
-            logits_stride, group_kind, renorm);
-      }))
-    return (pegainfer_status_t)hipErrorInvalidValue;
-  return (pegainfer_status_t)hipGetLastError();
+  pegainfer_route_plan_desc q{};
+  q.logits = logits; q.logits_stride = logits_stride; q.correction = correction; q.out_expert = out_expert; q.out_weight = out_weight;
+  q.experts = experts; q.n_groups = n_groups; q.keep_groups = keep_groups; q.top = top; q.rows = rows; q.score_kind = score_kind;
+  q.group_kind = group_kind; q.renorm = renorm; q.factor = 1.0f; q.dtype = dtype;
+  return pegainfer_route_plan(&q, stream);
 }
 
 pegainfer_status_t pegainfer_route_from_logits(const float* logits, const void* correction, int32_t* out_expert, float* out_weight,
@@ -283,21 +350,30 @@ pegainfer_status_t pegainfer_route_sort(const int32_t* expert, int32_t n_pairs, 
   if ((rows_per_tile != 64 && rows_per_tile != 128) || experts <= 0 || experts > 7000 ||
       max_tiles < (n_pairs + rows_per_tile - 1) / rows_per_tile + experts)
     return (pegainfer_status_t)hipErrorInvalidValue;
-  route_sort_kernel<<<1, 256, (size_t)2 * experts * sizeof(int), as_stream(stream)>>>(
-      expert, n_pairs, top, experts, pos_pair, pos_row, tile_group, tile_row0, tile_rows, n_tiles, max_tiles, rows_per_tile);
+  const SortOut o{pos_pair, pos_row, tile_group, tile_row0, tile_rows, n_tiles, max_tiles, rows_per_tile};
+  route_sort_kernel<<<1, 256, (size_t)2 * experts * sizeof(int), as_stream(stream)>>>(expert, n_pairs, top, experts, o);
   return (pegainfer_status_t)hipGetLastError();
 }
 
 pegainfer_status_t pegainfer_route_combine_gated(const float* y_pairs, const float* weight, const void* add,
                                                  const float* add_gate, int64_t add_gate_stride, void* out, int32_t d,
                                                  int32_t top, int32_t rows, int32_t dtype, pegainfer_stream_t stream) {
+  return pegainfer_route_combine_same(y_pairs, weight, nullptr, 0, nullptr, 0, add, add_gate, add_gate_stride, out, d, top, rows, dtype, stream);
+}
+
+pegainfer_status_t pegainfer_route_combine_same(const float* y_pairs, const float* weight, const int32_t* expert, int32_t same_from,
+                                                const void* same, int64_t same_stride, const void* add, const float* add_gate,
+                                                int64_t add_gate_stride, void* out, int32_t d, int32_t top, int32_t rows, int32_t dtype,
+                                                pegainfer_stream_t stream) {
   if (rows <= 0) return 0;
+  if (same && !expert) return (pegainfer_status_t)hipErrorInvalidValue;
   if (!by_dtype(dtype, [&](auto* t) {
         using A = std::remove_pointer_t<decltype(t)>;
         // few rows (decoding): the row is cut over several workgroups
         const dim3 grid(rows, rows >= 256 ? 1 : std::min(16, ceil_div(d, 256)));
-        route_combine_kernel<A><<<grid, 256, 0, as_stream(stream)>>>(y_pairs, weight, static_cast<const A*>(add),
-                                                                     static_cast<A*>(out), d, top, add_gate, add_gate_stride);
+        route_combine_kernel<A><<<grid, 256, 0, as_stream(stream)>>>(y_pairs, weight, static_cast<const A*>(add), static_cast<A*>(out), d,
+                                                                     top, add_gate, add_gate_stride, expert, same_from,
+                                                                     static_cast<const A*>(same), same_stride);
       }))
     return (pegainfer_status_t)hipErrorInvalidValue;
   return (pegainfer_status_t)hipGetLastError();

@@ -1,10 +1,12 @@
-// What the token-by-token recurrences share (recurrent.hip, decay_attn.hip): the layout of a workgroup - 16 value columns, a column's
+// What the token-by-token recurrences share (recurrent.hip, decay_attn.hip, gated_linear.hip): the layout of a workgroup - 16 value columns, a column's
 // state over the sixteen lanes of a DPP row - and the staging of 16 tokens' q | k | v through registers into LDS.
 #pragma once
 
 #include "common.h"
 
 namespace pk {
+
+__device__ __forceinline__ float logsigmoid_f(float x) { return fminf(x, 0.0f) - log1pf(expf(-fabsf(x))); }
 
 constexpr int kRecTokens = 16;   // tokens staged per round
 constexpr int kRecCols = 16;     // value columns per workgroup (four per wave)

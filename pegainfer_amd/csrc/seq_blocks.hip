@@ -12,7 +12,10 @@
 //   terms_rms_add_kernel    residual sum of up to three sublayer outputs, each optionally RMS-normed with a weight first, then
 //                           the RMS norm (a weight per channel) of what reads the stream next: one launch closes a layer whose
 //                           sublayers all read the same normed input, and opens the next
-//   glu_rows_kernel         act(gate) * up from two column ranges of a wider row (silu, relu or tanh-gelu)
+//                           (its stream may be read through a row index, or start as an embedding row plus the row of a table
+//                           addressed by the previous and the current token)
+//   glu_rows_kernel         act(gate) * up from two column ranges of a wider row (silu, relu, tanh-gelu or erf-gelu)
+//   act_rows_kernel         the same activations alone
 //   softcap_rows_kernel     cap * tanh(x / cap) on fp32 rows
 #include <algorithm>
 
@@ -392,16 +395,39 @@ __global__ __launch_bounds__(256) void scalar_rms_add_kernel(const float* x_in, 
 //   r = x_in + sum_t term_t                                  -> x_out (fp32; may alias x_in)
 //   n = r / sqrt(mean(r^2) + eps) * gain                     -> n_out (N: float or the storage type; optional)
 // NPT: values a thread keeps between the sum and the norm (d <= 256 * NPT), 0 = any d (the row is summed a second time).
+// gain_offset: added to every norm weight (1: weights stored around zero).  x_in rows may be picked through row_index, or be the
+// token's embedding row times a factor plus the row of a table addressed by (previous token, token).
 struct SumTerm { const void* y; int64_t stride; const void* bias; const void* w; float factor; };
 struct SumTerms { SumTerm t[3]; int n; };
+struct RowSource {
+  const float* x;
+  const int32_t* row_index;
+  const void* embed;
+  const uint32_t* ids;
+  float embed_scale;
+  const void* pairs;            // [buckets + 1][d]: row (prev * mul_prev + id * mul_cur) mod buckets; the last row without a previous token
+  const int32_t* prev;          // -1: none
+  int64_t mul_prev, mul_cur, buckets;
+};
 // VEC: d, the terms' strides and every pointer allow four values per load.
 template <typename A, typename N, int NPT, bool VEC>
-__global__ __launch_bounds__(256) void terms_rms_add_kernel(const float* x_in, SumTerms terms, float* x_out,
-                                                            const A* __restrict__ gain, float eps, N* __restrict__ n_out, int d) {
+__global__ __launch_bounds__(256) void terms_rms_add_kernel(RowSource src, SumTerms terms, float* x_out, const A* __restrict__ gain,
+                                                            float eps, float gain_offset, N* __restrict__ n_out, int d) {
   __shared__ float red[4];
   constexpr int V = VEC ? 4 : 1;
   const int row = blockIdx.x;
   const int64_t base = (int64_t)row * d;
+  const float* x_row = src.x ? src.x + (src.row_index ? (int64_t)src.row_index[row] * d : base) : nullptr;
+  const A *e_row = nullptr, *p_row = nullptr;
+  if (!src.x && src.embed) {
+    const uint32_t id = src.ids[row];
+    e_row = static_cast<const A*>(src.embed) + (int64_t)id * d;
+    if (src.pairs) {
+      const int32_t prev = src.prev[row];
+      const int64_t at = prev < 0 ? src.buckets : ((int64_t)prev * src.mul_prev + (int64_t)id * src.mul_cur) % src.buckets;
+      p_row = static_cast<const A*>(src.pairs) + at * d;
+    }
+  }
   auto load = [&](const auto* p, float* o) {
     if constexpr (VEC) ld4(p, o); else o[0] = ld(p);
   };
@@ -425,8 +451,18 @@ __global__ __launch_bounds__(256) void terms_rms_add_kernel(const float* x_in, S
     inv[t] = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)d + eps);
   }
   auto value = [&](int i, float* r) {      // V values from column i on
-    if (x_in) load(x_in + base + i, r);
-    else {
+    if (x_row) load(x_row + i, r);
+    else if (e_row) {
+      load(e_row + i, r);
+#pragma unroll
+      for (int u = 0; u < V; ++u) r[u] *= src.embed_scale;
+      if (p_row) {
+        float b[V];
+        load(p_row + i, b);
+#pragma unroll
+        for (int u = 0; u < V; ++u) r[u] += b[u];
+      }
+    } else {
 #pragma unroll
       for (int u = 0; u < V; ++u) r[u] = 0.f;
     }
@@ -443,7 +479,7 @@ __global__ __launch_bounds__(256) void terms_rms_add_kernel(const float* x_in, S
 #pragma unroll
       for (int u = 0; u < V; ++u) {
         float z = v[u] + (b ? bv[u] : 0.f);
-        if (w) z = z * inv[t] * wv[u];
+        if (w) z = z * inv[t] * (gain_offset + wv[u]);
         r[u] = fmaf(terms.t[t].factor, z, r[u]);
       }
     }
@@ -456,7 +492,7 @@ __global__ __launch_bounds__(256) void terms_rms_add_kernel(const float* x_in, S
       float g[V], o[V];
       load(gain + i, g);
 #pragma unroll
-      for (int u = 0; u < V; ++u) o[u] = r[u] * sc * g[u];
+      for (int u = 0; u < V; ++u) o[u] = r[u] * sc * (gain_offset + g[u]);
       if constexpr (VEC) st4(n_out + base + i, o); else st(n_out + base + i, o[0]);
     }
   };
@@ -506,11 +542,21 @@ __global__ __launch_bounds__(256) void glu_rows_kernel(const A* __restrict__ gat
   const int i = blockIdx.y * 256 + threadIdx.x;
   if (i >= I) return;
   const float g = ld(gate + (int64_t)row * in_stride + i), u = ld(up + (int64_t)row * in_stride + i);
-  float a;
-  if (act == 0) a = silu_f(g);
-  else if (act == 1) a = fmaxf(g, 0.f);
-  else a = 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-  st(out + (int64_t)row * out_stride + i, a * u);
+  st(out + (int64_t)row * out_stride + i, act_f(act, g) * u);
+}
+
+// out[row, i] = act(in[row, i]) (in place allowed); V values per thread
+template <typename A, int V>
+__global__ __launch_bounds__(256) void act_rows_kernel(const A* in, int64_t in_stride, A* out, int64_t out_stride, int I, int act) {
+  const int i = (blockIdx.y * 256 + threadIdx.x) * V;
+  if (i >= I) return;
+  const A* p = in + (int64_t)blockIdx.x * in_stride + i;
+  A* o = out + (int64_t)blockIdx.x * out_stride + i;
+  float v[V];
+  if constexpr (V == 4) ld4(p, v); else v[0] = ld(p);
+#pragma unroll
+  for (int u = 0; u < V; ++u) v[u] = act_f(act, v[u]);
+  if constexpr (V == 4) st4(o, v); else st(o, v[0]);
 }
 
 __global__ __launch_bounds__(256) void softcap_rows_kernel(const float* __restrict__ in, float* __restrict__ out, int64_t n, float cap) {
@@ -528,31 +574,44 @@ using namespace pk;
 pegainfer_status_t pegainfer_terms_rms_add(const float* x_in, const pegainfer_sum_term* terms, int32_t n_terms, float* x_out,
                                            const void* gain, float eps, void* n_out, int32_t n_dtype, int32_t d, int32_t rows,
                                            int32_t dtype, pegainfer_stream_t stream) {
-  if (rows <= 0) return 0;
-  if (d <= 0 || n_terms < 0 || n_terms > 3 || (n_terms > 0 && !terms) || (!x_in && n_terms == 0) || (!x_out && !n_out) ||
-      (n_out && !gain))
+  pegainfer_terms_rms_desc q{};
+  q.x_in = x_in; q.terms = terms; q.n_terms = n_terms; q.x_out = x_out; q.gain = gain; q.eps = eps;
+  q.n_out = n_out; q.n_dtype = n_dtype; q.d = d; q.rows = rows; q.dtype = dtype;
+  return pegainfer_terms_rms(&q, stream);
+}
+
+pegainfer_status_t pegainfer_terms_rms(const pegainfer_terms_rms_desc* q, pegainfer_stream_t stream) {
+  if (!q) return PK_BAD;
+  if (q->rows <= 0) return 0;
+  const int d = q->d, n_terms = q->n_terms;
+  const bool from_embed = !q->x_in && q->embed;
+  if (d <= 0 || n_terms < 0 || n_terms > 3 || (n_terms > 0 && !q->terms) || (!q->x_in && !from_embed && n_terms == 0) ||
+      (!q->x_out && !q->n_out) || (q->n_out && !q->gain) || (from_embed && !q->token_ids) ||
+      (from_embed && q->pair_table && (!q->prev_ids || q->buckets < 1)) || (q->row_index && q->x_out && q->x_out == q->x_in))
     return PK_BAD;
+  RowSource src{q->x_in, q->row_index, q->embed, q->token_ids, q->embed_scale, q->pair_table, q->prev_ids, q->mul_prev, q->mul_cur, q->buckets};
   SumTerms st_{};
   st_.n = n_terms;
   for (int t = 0; t < n_terms; ++t) {
-    if (!terms[t].y) return PK_BAD;
-    st_.t[t] = SumTerm{terms[t].y, terms[t].y_row_stride, terms[t].bias, terms[t].norm_w, terms[t].factor};
+    if (!q->terms[t].y) return PK_BAD;
+    st_.t[t] = SumTerm{q->terms[t].y, q->terms[t].y_row_stride, q->terms[t].bias, q->terms[t].norm_w, q->terms[t].factor};
   }
   bool ok = true;
-  const bool known = by_dtype(dtype, [&](auto* ta) {
+  const bool known = by_dtype(q->dtype, [&](auto* ta) {
     using A = std::remove_pointer_t<decltype(ta)>;
-    ok = by_dtype(n_out ? n_dtype : dtype, [&](auto* tn) {
+    ok = by_dtype(q->n_out ? q->n_dtype : q->dtype, [&](auto* tn) {
       using N = std::remove_pointer_t<decltype(tn)>;
-      bool vec = d % 4 == 0 && host_aligned16(x_in) && host_aligned16(x_out) && host_aligned16(gain) && host_aligned16(n_out);
+      bool vec = d % 4 == 0 && host_aligned16(q->x_in) && host_aligned16(q->x_out) && host_aligned16(q->gain) && host_aligned16(q->n_out) &&
+                 host_aligned16(q->embed) && host_aligned16(q->pair_table);
       for (int t = 0; t < n_terms; ++t)
-        vec = vec && terms[t].y_row_stride % 4 == 0 && host_aligned16(terms[t].y) && host_aligned16(terms[t].bias) && host_aligned16(terms[t].norm_w);
+        vec = vec && st_.t[t].stride % 4 == 0 && host_aligned16(st_.t[t].y) && host_aligned16(st_.t[t].bias) && host_aligned16(st_.t[t].w);
       auto go = [&](auto npt) {
-        if (vec)
-          terms_rms_add_kernel<A, N, decltype(npt)::value, true><<<rows, 256, 0, as_stream(stream)>>>(
-              x_in, st_, x_out, static_cast<const A*>(gain), eps, static_cast<N*>(n_out), d);
-        else
-          terms_rms_add_kernel<A, N, decltype(npt)::value, false><<<rows, 256, 0, as_stream(stream)>>>(
-              x_in, st_, x_out, static_cast<const A*>(gain), eps, static_cast<N*>(n_out), d);
+        auto launch = [&](auto kern) {
+          kern<<<q->rows, 256, 0, as_stream(stream)>>>(src, st_, q->x_out, static_cast<const A*>(q->gain), q->eps, q->gain_offset,
+                                                       static_cast<N*>(q->n_out), d);
+        };
+        if (vec) launch(terms_rms_add_kernel<A, N, decltype(npt)::value, true>);
+        else launch(terms_rms_add_kernel<A, N, decltype(npt)::value, false>);
       };
       if (d <= 1024) go(std::integral_constant<int, 4>());
       else if (d <= 4096) go(std::integral_constant<int, 16>());
@@ -563,10 +622,28 @@ pegainfer_status_t pegainfer_terms_rms_add(const float* x_in, const pegainfer_su
   return known && ok ? (pegainfer_status_t)hipGetLastError() : PK_BAD;
 }
 
+pegainfer_status_t pegainfer_act_rows(const void* in, int64_t in_row_stride, void* out, int64_t out_row_stride, int32_t I, int32_t rows,
+                                      int32_t act, int32_t dtype, pegainfer_stream_t stream) {
+  if (rows <= 0 || I <= 0) return 0;
+  if (act < 0 || act > PEGAINFER_ACT_GELU_ERF) return PK_BAD;
+  if (!by_dtype(dtype, [&](auto* t) {
+        using A = std::remove_pointer_t<decltype(t)>;
+        const bool vec = I % 4 == 0 && in_row_stride % 4 == 0 && out_row_stride % 4 == 0 && host_aligned16(in) && host_aligned16(out);
+        auto launch = [&](auto kern, int per) {
+          kern<<<dim3(rows, ceil_div(I, 256 * per)), 256, 0, as_stream(stream)>>>(static_cast<const A*>(in), in_row_stride,
+                                                                                  static_cast<A*>(out), out_row_stride, I, act);
+        };
+        if (vec) launch(act_rows_kernel<A, 4>, 4);
+        else launch(act_rows_kernel<A, 1>, 1);
+      }))
+    return PK_BAD;
+  return (pegainfer_status_t)hipGetLastError();
+}
+
 pegainfer_status_t pegainfer_glu_rows(const void* gate, const void* up, int64_t in_row_stride, void* out, int64_t out_row_stride,
                                       int32_t I, int32_t rows, int32_t act, int32_t dtype, pegainfer_stream_t stream) {
   if (rows <= 0 || I <= 0) return 0;
-  if (act < 0 || act > 2) return PK_BAD;
+  if (act < 0 || act > PEGAINFER_ACT_GELU_ERF) return PK_BAD;
   const dim3 grid(rows, ceil_div(I, 256));
   if (!by_dtype(dtype, [&](auto* t) {
         using A = std::remove_pointer_t<decltype(t)>;

@@ -50,5 +50,14 @@ __device__ __forceinline__ void ld4(const uint16_t* p, float* o) {
 __device__ __forceinline__ void st4(float* p, const float* o) { *reinterpret_cast<f32x4*>(p) = f32x4{o[0], o[1], o[2], o[3]}; }
 __device__ __forceinline__ void st4(uint16_t* p, const float* o) { *reinterpret_cast<u32x2*>(p) = u32x2{pack_bf2(o[0], o[1]), pack_bf2(o[2], o[3])}; }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+// the exact form of gelu: z times the normal distribution's share below z
+__device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+// an activation by its PEGAINFER_ACT_* number
+__device__ __forceinline__ float act_f(int act, float g) {
+  if (act == 0) return silu_f(g);
+  if (act == 1) return fmaxf(g, 0.f);
+  if (act == 2) return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+  return gelu_erf_f(g);
+}
 
 }  // namespace pk

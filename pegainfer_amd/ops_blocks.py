@@ -507,7 +507,7 @@ def _struct(name, fields):
 
 AttnOptions = _struct("AttnOptions", [("i", "maps"), ("f", "lambda_"), ("i", "block"), ("p", "sink"), ("i", "head_norm"), ("f", "norm_eps softcap"),
                                       ("i", "window keep_first"), ("p", "dist_bias"), ("i", "n_dist"), ("p", "dist_slope gate"),
-                                      ("l", "gate_stride"), ("i", "gate_kind n_split"), ("p", "workspace"), ("i", "plain")])
+                                      ("l", "gate_stride"), ("i", "gate_kind n_split"), ("p", "workspace"), ("i", "plain shared_tail")])
 LatentPrepDesc = _struct("LatentPrepDesc", [("p", "dkv"), ("l", "dkv_stride"), ("p", "c_norm_w ql"), ("l", "ql_stride"), ("p", "ql_norm_w ql_out"),
                                             ("i", "q_rank"), ("p", "q"), ("l", "q_stride"), ("p", "qc"), ("f", "eps"), ("p", "inv_freq"),
                                             ("i", "rot_dims rot_layout"), ("p", "positions token_req page_indptr page_ids cache"),

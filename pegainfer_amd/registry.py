@@ -1,9 +1,10 @@
 """Model registry: which engine serves a model folder, decided by its config.json.
 
 Hugging Face style configurations name their family in ``model_type`` / ``architectures`` (Qwen3, Qwen3.5); Duguzen,
-Feruzen, Ramalix, Kukulorn and Zofadra name it in ``architecture``.  ``load_engine`` builds the engine with the weights of the
+Feruzen, Ramalix, Kukulorn, Zofadra and Sopanex name it in ``architecture``.  ``load_engine`` builds the engine with the weights of the
 folder; ``scheduler_for`` puts the continuous-batching scheduler (include/pegainfer_scheduler.h) on top of it.
 """
+import importlib
 import json
 import os
 
@@ -23,51 +24,29 @@ def _qwen35(model_dir, cfg, **kw):
     return eng.load_safetensors(os.path.join(model_dir, "model.safetensors"))
 
 
-def _duguzen(model_dir, cfg, **kw):
-    from .duguzen import DuguzenEngine
-    return DuguzenEngine.from_pretrained(model_dir, max_tokens=kw.get("max_tokens", 4096), max_requests=kw.get("max_requests", 8),
-                                         dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
+# families over a runtime with one batched step function (step_engine.StepEngine); config.json names them in "architecture"
+STEP_FAMILIES = ("duguzen", "feruzen", "ramalix", "kukulorn", "zofadra", "sopanex")
 
 
-def _feruzen(model_dir, cfg, **kw):
-    from .feruzen import FeruzenEngine
-    return FeruzenEngine.from_pretrained(model_dir, max_tokens=kw.get("max_tokens", 4096), max_requests=kw.get("max_requests", 8),
-                                         dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
-
-
-def _ramalix(model_dir, cfg, **kw):
-    from .ramalix import RamalixEngine
-    return RamalixEngine.from_pretrained(model_dir, max_tokens=kw.get("max_tokens", 4096), max_requests=kw.get("max_requests", 8),
-                                         dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
-
-
-def _kukulorn(model_dir, cfg, **kw):
-    from .kukulorn import KukulornEngine
-    return KukulornEngine.from_pretrained(model_dir, max_tokens=kw.get("max_tokens", 4096), max_requests=kw.get("max_requests", 8),
-                                          dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
-
-
-def _zofadra(model_dir, cfg, **kw):
-    from .zofadra import ZofadraEngine
-    return ZofadraEngine.from_pretrained(model_dir, max_tokens=kw.get("max_tokens", 4096), max_requests=kw.get("max_requests", 8),
-                                         dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
+def _step_family(family):
+    def load(model_dir, cfg, **kw):
+        engine = getattr(importlib.import_module("." + family, __package__), family.capitalize() + "Engine")
+        return engine.from_pretrained(model_dir, max_tokens=kw.get("max_tokens", 4096), max_requests=kw.get("max_requests", 8),
+                                      dtype=kw.get("dtype", "bfloat16"), device=kw.get("device", 0))
+    return load
 
 
 # family -> (loader, dtypes it can be served in)
 REGISTRY = {
     "qwen3": (_qwen3, ("bfloat16",)),
     "qwen3_5": (_qwen35, ("bfloat16",)),
-    "duguzen": (_duguzen, ("bfloat16", "float32")),
-    "feruzen": (_feruzen, ("bfloat16", "float32")),
-    "ramalix": (_ramalix, ("bfloat16", "float32")),
-    "kukulorn": (_kukulorn, ("bfloat16", "float32")),
-    "zofadra": (_zofadra, ("bfloat16", "float32")),
+    **{f: (_step_family(f), ("bfloat16", "float32")) for f in STEP_FAMILIES},
 }
 
 
 def family_of(cfg):
     """the registry key of a parsed config.json, or None"""
-    if str(cfg.get("architecture", "")).lower() in ("duguzen", "feruzen", "ramalix", "kukulorn", "zofadra"):
+    if str(cfg.get("architecture", "")).lower() in STEP_FAMILIES:
         return str(cfg["architecture"]).lower()
     names = [str(cfg.get("model_type", ""))] + [str(a) for a in cfg.get("architectures", [])]
     low = " ".join(names).lower()

@@ -62,7 +62,8 @@ class Scheduler:
                   "FeruzenEngine": lib.pegainfer_sched_create_feruzen,
                   "RamalixEngine": lib.pegainfer_sched_create_ramalix,
                   "KukulornEngine": lib.pegainfer_sched_create_kukulorn,
-                  "ZofadraEngine": lib.pegainfer_sched_create_zofadra}.get(type(engine).__name__, lib.pegainfer_sched_create_qwen3)
+                  "ZofadraEngine": lib.pegainfer_sched_create_zofadra,
+                  "SopanexEngine": lib.pegainfer_sched_create_sopanex}.get(type(engine).__name__, lib.pegainfer_sched_create_qwen3)
         h = create(engine.h, seed, st.ctypes.data if st.size else None, int(st.size))
         return cls(h, keep=engine)
 
