@@ -12,7 +12,7 @@ import torch
 from . import ffi
 from .ops import _chk, _p, _stream
 
-EPI_NONE, EPI_RELU_SQ, EPI_SIGMOID_GATE = 0, 1, 2
+EPI_NONE, EPI_RELU_SQ, EPI_SIGMOID_GATE, EPI_GELU_ERF = 0, 1, 2, 3
 
 
 def _dt(t):
@@ -423,12 +423,15 @@ def terms_rms_add(x, terms, gain=None, eps=1e-6, out_dtype=None):
     return r, n
 
 
+ACTS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "gelu_erf": 3}
+
+
 def glu_rows(gate, up, act="relu"):
     """act(gate) * up; gate and up are [rows, I] views of rows with one stride (column ranges of a wider matrix)"""
     rows, I = gate.shape
     assert gate.stride(0) == up.stride(0)
     out = torch.empty((rows, I), dtype=gate.dtype, device=gate.device)
-    _chk(ffi.lib().pegainfer_glu_rows(_p(gate), _p(up), gate.stride(0), _p(out), I, I, rows, {"silu": 0, "relu": 1, "gelu_tanh": 2}[act],
+    _chk(ffi.lib().pegainfer_glu_rows(_p(gate), _p(up), gate.stride(0), _p(out), I, I, rows, ACTS[act],
                                       _dt(gate), _stream()), "glu_rows")
     return out
 
@@ -523,8 +526,9 @@ DecayAttentionDesc = _struct("DecayAttentionDesc", [("p", "proj"), ("l", "proj_s
 
 
 def paged_attention_opt(q, cache, page_stride, k_off, v_off, page_size, rg, page_indptr, page_ids, kv_heads, vdim, scale, window=0,
-                        dist_slope=None, softcap=0.0, n_split=1, plain=False):
-    """q fp32 [rows, heads, dim]; dist_slope fp32 [heads]: slope * distance is taken off the scores"""
+                        dist_slope=None, softcap=0.0, n_split=1, plain=False, sink=None, gate=None, factor=1.0, shared_tail=0):
+    """q fp32 [rows, heads, dim]; dist_slope fp32 [heads]: slope * distance is taken off the scores; gate: a [rows, heads] view in the
+    cache's type, one output gate logit per head; shared_tail: values of a key that are read from its value"""
     T, H, dim = q.shape
     out = torch.empty((T, H * vdim), dtype=cache.dtype, device=q.device)
     t = attention_tiles(rg.lens, H // kv_heads, q.device)
@@ -533,10 +537,11 @@ def paged_attention_opt(q, cache, page_stride, k_off, v_off, page_size, rg, page
         ws = torch.empty(ffi.lib().pegainfer_paged_attention_workspace(t[0].numel(), kv_heads, vdim, 1, n_split), dtype=torch.float32,
                          device=q.device)
     o = AttnOptions(window=int(window), dist_slope=_p(dist_slope), softcap=float(softcap), n_split=int(n_split), workspace=_p(ws),
-                    plain=int(bool(plain)))
+                    plain=int(bool(plain)), sink=_p(sink), gate=_p(gate), gate_stride=0 if gate is None else gate.stride(0),
+                    gate_kind=0 if gate is None else 2, shared_tail=int(shared_tail))
     _chk(ffi.lib().pegainfer_paged_attention_opt(_p(q), _p(cache), page_stride, k_off, v_off, page_size, _p(rg.positions), _p(rg.row_entry),
-                                                 _p(page_indptr), _p(page_ids), H, kv_heads, dim, vdim, float(scale), 1.0, _p(t[0]), _p(t[1]),
-                                                 _p(t[2]), _p(t[3]), t[0].numel(), _p(out), out.stride(0), ctypes.addressof(o), _dt(cache),
+                                                 _p(page_indptr), _p(page_ids), H, kv_heads, dim, vdim, float(scale), float(factor), _p(t[0]),
+                                                 _p(t[1]), _p(t[2]), _p(t[3]), t[0].numel(), _p(out), out.stride(0), ctypes.addressof(o), _dt(cache),
                                                  _stream()), "paged_attention_opt")
     return out
 
@@ -588,6 +593,28 @@ def stream_mix(x, streams, d, dtype, y=None, mix=None, out_w=None, mult=1.0, rea
     return new, n, sm
 
 
+def _chunk_tables(d, rg, scan_max, workspace, heads, dim, vdim, chunk=64):
+    """the chunk tables of a step's entries of more than scan_max rows, put into the descriptor d; returns the tensors behind them"""
+    row0, rows, first, slot, at = [], [], [0], [], 0
+    slots = rg.entry_slot.tolist()
+    for i, n in enumerate(rg.lens if scan_max > 0 else []):
+        if n > scan_max:
+            for k in range(0, n, chunk):
+                row0.append(at + k)
+                rows.append(min(chunk, n - k))
+            first.append(len(row0))
+            slot.append(slots[i])
+        at += n
+    if not slot:
+        return []
+    dev = rg.entry_slot.device
+    keep = [torch.tensor(v, dtype=torch.int32, device=dev) for v in (row0, rows, first, slot)]
+    keep.append(torch.full((int(workspace(len(row0), heads, dim, vdim)),), float("nan"), dtype=torch.float32, device=dev))
+    d.scan_max, d.chunk_row0, d.chunk_rows, d.n_chunks = scan_max, _p(keep[0]), _p(keep[1]), len(row0)
+    d.long_chunk0, d.long_slot, d.n_long, d.workspace = _p(keep[2]), _p(keep[3]), len(slot), _p(keep[4])
+    return keep
+
+
 def decay_attention(proj, offs, decay, state, heads, dim, vdim, rg, silu=True, scan_max=0):
     """proj rows [.. q at offs[0] | k at offs[1] | v at offs[2] ..]; decay: one number per head; state fp32 [slots, heads * dim * vdim];
     scan_max > 0: entries of more rows take the chunk form -> fp32 [rows, heads * vdim]"""
@@ -597,23 +624,107 @@ def decay_attention(proj, offs, decay, state, heads, dim, vdim, rg, silu=True, s
     d = DecayAttentionDesc(proj=_p(proj), proj_stride=proj.stride(0), q_off=offs[0], k_off=offs[1], v_off=offs[2], silu=int(bool(silu)),
                            decay_pow=_p(pw), pow_n=C + 1, state=_p(state), slot_stride=state.stride(0), o=_p(o), heads=heads, dim=dim,
                            vdim=vdim, entry_row0=_p(rg.entry_row0), entry_slot=_p(rg.entry_slot), n_entries=len(rg.lens), dtype=_dt(proj))
-    keep = []
-    if scan_max > 0:
-        row0, rows, first, slot, at = [], [], [0], [], 0
-        slots = rg.entry_slot.tolist()
-        for i, n in enumerate(rg.lens):
-            if n > scan_max:
-                for k in range(0, n, C):
-                    row0.append(at + k)
-                    rows.append(min(C, n - k))
-                first.append(len(row0))
-                slot.append(slots[i])
-            at += n
-        if slot:
-            keep = [torch.tensor(v, dtype=torch.int32, device=proj.device) for v in (row0, rows, first, slot)]
-            keep.append(torch.empty(int(ffi.lib().pegainfer_decay_attention_workspace(len(row0), heads, dim, vdim)), dtype=torch.float32,
-                                    device=proj.device))
-            d.scan_max, d.chunk_row0, d.chunk_rows, d.n_chunks = scan_max, _p(keep[0]), _p(keep[1]), len(row0)
-            d.long_chunk0, d.long_slot, d.n_long, d.workspace = _p(keep[2]), _p(keep[3]), len(slot), _p(keep[4])
+    keep = _chunk_tables(d, rg, scan_max, ffi.lib().pegainfer_decay_attention_workspace, heads, dim, vdim)  # noqa: F841 (alive until enqueued)
     _chk(ffi.lib().pegainfer_decay_attention(ctypes.addressof(d), _stream()), "decay_attention")
+    return o
+
+
+# ---- norms with offset gains, rows of token pairs, identity experts, values that are keys, gated linear attention ----
+TermsRmsDesc = _struct("TermsRmsDesc", [("p", "x_in row_index embed token_ids"), ("f", "embed_scale"), ("p", "pair_table prev_ids"),
+                                        ("l", "mul_prev mul_cur buckets"), ("p", "terms"), ("i", "n_terms"), ("p", "x_out gain"),
+                                        ("f", "eps gain_offset"), ("p", "n_out"), ("i", "n_dtype d rows dtype")])
+RoutePlanDesc = _struct("RoutePlanDesc", [("p", "logits"), ("l", "logits_stride"), ("p", "correction out_expert out_weight"),
+                                          ("i", "experts n_groups keep_groups top rows score_kind group_kind renorm"), ("f", "factor"),
+                                          ("i", "sort_experts"), ("p", "pos_pair pos_row tile_group tile_row0 tile_rows n_tiles"),
+                                          ("i", "max_tiles rows_per_tile dtype")])
+QkPrepDesc = _struct("QkPrepDesc", [("p", "proj"), ("i", "proj_dtype"), ("l", "proj_stride q_off k_off v_off"), ("i", "heads kv_heads dim vdim"),
+                                    ("p", "q_norm k_norm"), ("i", "norm_kind"), ("f", "eps"), ("p", "q_bias k_bias v_bias"), ("f", "qt_coef"),
+                                    ("i", "qt_every"), ("p", "inv_freq"), ("i", "rot_dims rot_layout"), ("f", "rot_amp"),
+                                    ("p", "positions row_entry page_indptr page_ids cache"), ("l", "page_stride k_cache_off v_cache_off"),
+                                    ("i", "page_size shared_tail"), ("p", "q_out q_out_stored"), ("i", "n_rows dtype")])
+GatedLinearDesc = _struct("GatedLinearDesc", [("p", "proj"), ("l", "proj_stride q_off k_off v_off"), ("f", "q_scale"), ("p", "z"), ("l", "z_stride"),
+                                              ("p", "z_bias"), ("f", "tau"), ("p", "state"), ("l", "slot_stride"), ("p", "o"),
+                                              ("i", "heads dim vdim"), ("p", "entry_row0 entry_slot"), ("i", "n_entries scan_max"),
+                                              ("p", "chunk_row0 chunk_rows"), ("i", "n_chunks"), ("p", "long_chunk0 long_slot"), ("i", "n_long"),
+                                              ("p", "workspace"), ("i", "dtype")])
+
+
+def terms_rms(dtype, d, x=None, row_index=None, embed=None, token_ids=None, embed_scale=1.0, pair_table=None, prev_ids=None, muls=(0, 0),
+              terms=(), gain=None, eps=1e-5, gain_offset=0.0, out_dtype=None):
+    """terms_rms_add with its options: gain_offset, x rows picked by row_index, or the stream started from embedding rows (and the rows of
+    pair_table [buckets + 1, d]) -> (stream fp32, normed row or None)"""
+    rows = row_index.numel() if row_index is not None else token_ids.numel() if x is None else x.shape[0]
+    arr = (SumTerm * max(1, len(terms)))()
+    for i, (y, bias, nw, f) in enumerate(terms):
+        arr[i] = SumTerm(_p(y), y.stride(0), _p(bias), _p(nw), float(f))
+    r = torch.empty((rows, d), dtype=torch.float32, device="cuda")
+    n = torch.empty((rows, d), dtype=out_dtype or dtype, device="cuda") if gain is not None else None
+    q = TermsRmsDesc(x_in=_p(x), row_index=_p(row_index), embed=_p(embed), token_ids=_p(token_ids), embed_scale=float(embed_scale),
+                     pair_table=_p(pair_table), prev_ids=_p(prev_ids), mul_prev=int(muls[0]), mul_cur=int(muls[1]),
+                     buckets=0 if pair_table is None else pair_table.shape[0] - 1, terms=ctypes.addressof(arr) if terms else None,
+                     n_terms=len(terms), x_out=_p(r), gain=_p(gain), eps=float(eps), gain_offset=float(gain_offset), n_out=_p(n),
+                     n_dtype=_dt(n) if n is not None else 0, d=d, rows=rows, dtype=0 if dtype == torch.bfloat16 else 1)
+    _chk(ffi.lib().pegainfer_terms_rms(ctypes.addressof(q), _stream()), "terms_rms")
+    return r, n
+
+
+def act_rows(x, act):
+    """x: a [rows, I] view of rows with one stride"""
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    _chk(ffi.lib().pegainfer_act_rows(_p(x), x.stride(0), _p(out), out.stride(0), x.shape[1], x.shape[0], ACTS[act], _dt(x), _stream()), "act_rows")
+    return out
+
+
+def route_plan(logits_f32, experts, top, sort_experts, correction=None, score="softmax", renorm=True, factor=1.0, rows_per_tile=64,
+               dtype=torch.bfloat16):
+    """selection and sort -> (expert [rows, top], weight, dict of the sort's arrays)"""
+    rows, dev = logits_f32.shape[0], logits_f32.device
+    P = rows * top
+    max_tiles = (P + rows_per_tile - 1) // rows_per_tile + sort_experts
+    i32 = lambda *n: torch.full(n, -7, dtype=torch.int32, device=dev)  # noqa: E731
+    e, w = i32(rows, top), torch.empty((rows, top), dtype=torch.float32, device=dev)
+    s = {"pos_pair": i32(P), "pos_row": i32(P), "tile_group": i32(max_tiles), "tile_row0": i32(max_tiles), "tile_rows": i32(max_tiles), "n_tiles": i32(1)}
+    q = RoutePlanDesc(logits=_p(logits_f32), logits_stride=logits_f32.stride(0), correction=_p(correction), out_expert=_p(e), out_weight=_p(w),
+                      experts=experts, n_groups=1, keep_groups=1, top=top, rows=rows, score_kind=1 if score == "softmax" else 0,
+                      renorm=int(bool(renorm)), factor=float(factor), sort_experts=sort_experts, max_tiles=max_tiles,
+                      rows_per_tile=rows_per_tile, dtype=0 if dtype == torch.bfloat16 else 1, **{k: _p(v) for k, v in s.items()})
+    _chk(ffi.lib().pegainfer_route_plan(ctypes.addressof(q), _stream()), "route_plan")
+    s["max_tiles"] = max_tiles
+    return e, w, s
+
+
+def route_combine_same(y_pairs, weight, expert, same_from, same, add=None, add_gate_f32=None):
+    """pairs of expert numbers >= same_from take their row of `same`"""
+    rows, top = weight.shape
+    d = same.shape[1]
+    out = torch.empty((rows, d), dtype=same.dtype, device=same.device)
+    _chk(ffi.lib().pegainfer_route_combine_same(_p(y_pairs), _p(weight), _p(expert), same_from, _p(same), same.stride(0), _p(add),
+                                                _p(add_gate_f32), 0 if add_gate_f32 is None else add_gate_f32.stride(0), _p(out), d, top, rows,
+                                                _dt(out), _stream()), "route_combine_same")
+    return out
+
+
+def qk_prep(proj, offs, heads, kv_heads, dim, vdim, rg, page_indptr, page_ids, cache, page_stride, k_off, v_off, page_size, inv_freq=None,
+            rot_dims=0, halves=True, rot_amp=1.0, shared_tail=0):
+    """queries -> fp32 [rows, heads, dim]; keys (without their last shared_tail values) and values -> the cache"""
+    q = torch.empty((proj.shape[0], heads, dim), dtype=torch.float32, device=proj.device)
+    p = QkPrepDesc(proj=_p(proj), proj_dtype=_dt(proj), proj_stride=proj.stride(0), q_off=offs[0], k_off=offs[1], v_off=offs[2], heads=heads,
+                   kv_heads=kv_heads, dim=dim, vdim=vdim, inv_freq=_p(inv_freq), rot_dims=rot_dims, rot_layout=int(bool(halves)),
+                   rot_amp=float(rot_amp), positions=_p(rg.positions), row_entry=_p(rg.row_entry), page_indptr=_p(page_indptr),
+                   page_ids=_p(page_ids), cache=_p(cache), page_stride=page_stride, k_cache_off=k_off, v_cache_off=v_off, page_size=page_size,
+                   shared_tail=shared_tail, q_out=_p(q), n_rows=proj.shape[0], dtype=_dt(cache))
+    _chk(ffi.lib().pegainfer_qk_prep(ctypes.addressof(p), _stream()), "qk_prep")
+    return q
+
+
+def gated_linear(proj, offs, z_f32, z_bias, tau, q_scale, state, heads, dim, vdim, rg, scan_max=0):
+    """proj rows [.. q at offs[0] | k at offs[1] | v at offs[2] ..]; z fp32 [rows, heads * dim]; state fp32 [slots, heads * dim * vdim];
+    scan_max > 0: entries of more rows take the chunk form -> fp32 [rows, heads * vdim]"""
+    o = torch.empty((proj.shape[0], heads * vdim), dtype=torch.float32, device=proj.device)
+    d = GatedLinearDesc(proj=_p(proj), proj_stride=proj.stride(0), q_off=offs[0], k_off=offs[1], v_off=offs[2], q_scale=float(q_scale),
+                        z=_p(z_f32), z_stride=z_f32.stride(0), z_bias=_p(z_bias), tau=float(tau), state=_p(state),
+                        slot_stride=state.stride(0), o=_p(o), heads=heads, dim=dim, vdim=vdim, entry_row0=_p(rg.entry_row0),
+                        entry_slot=_p(rg.entry_slot), n_entries=len(rg.lens), dtype=_dt(proj))
+    keep = _chunk_tables(d, rg, scan_max, ffi.lib().pegainfer_gated_linear_workspace, heads, dim, vdim)  # noqa: F841 (alive until enqueued)
+    _chk(ffi.lib().pegainfer_gated_linear(ctypes.addressof(d), _stream()), "gated_linear")
     return o
