@@ -662,13 +662,14 @@ def main():
     ap.add_argument("--ctx", type=int, default=1024, help="prompt length before the timed decode steps")
     ap.add_argument("--batch", type=int, default=1, help="requests decoded together per rank")
     ap.add_argument("--model", default="qwen3-4b", choices=["qwen3-4b", "qwen3-8b", "qwen3.5-4b", "duguzen", "feruzen", "ramalix", "kukulorn",
-                                                            "zofadra"],
+                                                            "zofadra", "sopanex"],
                     help="duguzen: prefill / decode throughput of the Duguzen design at real layer sizes beside Qwen3 at equal size "
                          "(pegainfer_amd/bench_duguzen.py; its own JSON line, not the headline metric); feruzen: the same for the "
                          "Feruzen design beside Qwen3.5 at equal size (pegainfer_amd/bench_feruzen.py); ramalix: the Ramalix design beside "
                          "Feruzen at equal size (pegainfer_amd/bench_ramalix.py); kukulorn: the Kukulorn design beside Feruzen at "
                          "equal size (pegainfer_amd/bench_kukulorn.py); zofadra: the Zofadra design beside Kukulorn and Duguzen at equal size "
-                         "(pegainfer_amd/bench_zofadra.py)")
+                         "(pegainfer_amd/bench_zofadra.py); sopanex: the Sopanex design beside Feruzen and Ramalix at equal size "
+                         "(pegainfer_amd/bench_sopanex.py)")
     ap.add_argument("--dz-size", default="mid", choices=["small", "mid", "large", "all"], help="layer sizes of --model duguzen")
     ap.add_argument("--fz-size", default="mid", choices=["small", "mid", "large", "all"], help="layer sizes of --model feruzen")
     ap.add_argument("--fz-only", default="both", choices=["both", "feruzen", "qwen35"], help="--model feruzen: which side to run")
@@ -684,6 +685,10 @@ def main():
     ap.add_argument("--zf-only", default="all", choices=["all", "zofadra", "kukulorn", "duguzen"], help="--model zofadra: which side to run")
     ap.add_argument("--zf-phase", default="all", choices=["all", "prefill", "decode"],
                     help="--model zofadra: prefill or decode (bs 1) alone, for a kernel trace of that phase")
+    ap.add_argument("--sx-size", default="mid", choices=["small", "mid", "large", "all"], help="layer sizes of --model sopanex")
+    ap.add_argument("--sx-only", default="all", choices=["all", "sopanex", "feruzen", "ramalix"], help="--model sopanex: which side to run")
+    ap.add_argument("--sx-phase", default="all", choices=["all", "prefill", "decode"],
+                    help="--model sopanex: prefill or decode (bs 1) alone, for a kernel trace of that phase")
     ap.add_argument("--decode-mode", type=int, choices=[0, 1], default=int(os.environ.get("PEGAINFER_DECODE_MODE", "1")),
                     help="0 = reference op sequence 1:1, 1 = fused MI355X decode kernels (bit-identical)")
     ap.add_argument("--split-policy", type=int, default=1)
@@ -734,6 +739,9 @@ def main():
     if args.model == "zofadra":
         from pegainfer_amd import bench_zofadra
         return bench_zofadra.run(args)
+    if args.model == "sopanex":
+        from pegainfer_amd import bench_sopanex
+        return bench_sopanex.run(args)
 
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         # plain `python bench.py --gpus N`: become the launcher - one process per GPU over RCCL, exactly what the

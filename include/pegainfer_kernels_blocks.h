@@ -262,7 +262,7 @@ pegainfer_status_t pegainfer_route_from_logits_ex(const float* logits, int64_t l
 /* Selection and, with sort_experts > 0, the sort of pegainfer_route_sort behind it, from router logits in fp32 (one launch for up to 16
  * rows).  As pegainfer_route_from_logits_ex, with the weights times `factor` at the end.  Only expert numbers below sort_experts get
  * positions: numbers from there on are identity experts, whose output is the feed-forward's own input
- * (pegainfer_route_combine_same). */
+ * (pegainfer_route_combine_same).  max_tiles >= min(pairs, ceil(pairs / rows_per_tile) + sort_experts): no more tiles than pairs. */
 typedef struct {
   const float* logits;
   int64_t logits_stride;
@@ -345,6 +345,31 @@ typedef struct {
   int32_t n_dtype, d, rows, dtype;
 } pegainfer_terms_rms_desc;
 pegainfer_status_t pegainfer_terms_rms(const pegainfer_terms_rms_desc* q, pegainfer_stream_t stream);
+/* ONE sublayer output, normed, joins the stream in place, and the next norm leaves its input:
+ *   x <- x + y / sqrt(mean(y^2) + eps) * (gain_offset + post);  n_out = x / sqrt(mean(x^2) + eps) * (gain_offset + gain)   (gain NULL: no n_out)
+ * y: rows of dtype at y_row_stride; or, with y_pairs given, the weighted sum of routed experts made on the way, in fp32
+ * (pegainfer_route_combine_same: y_pairs, weight, expert, top, same_from, same, add [rows][d], add_gate).  Everything a row needs is
+ * requested before the first sum and stays in registers.  d <= 32768. */
+typedef struct {
+  float* x;
+  const void* y;
+  int64_t y_row_stride;
+  const float* y_pairs;
+  const float* weight;
+  const int32_t* expert;
+  int32_t top, same_from;
+  const void* same;
+  int64_t same_stride;
+  const void* add;
+  const float* add_gate;
+  int64_t add_gate_stride;
+  const void* post;
+  const void* gain;
+  float eps, gain_offset;
+  void* n_out;
+  int32_t d, rows, dtype;
+} pegainfer_join_rms_desc;
+pegainfer_status_t pegainfer_join_rms(const pegainfer_join_rms_desc* q, pegainfer_stream_t stream);
 /* out[row, i] = act(gate[row, i]) * up[row, i], i < I; gate and up are column ranges of rows with stride in_row_stride (elements of
  * dtype).  act 0 = silu, 1 = relu, 2 = gelu (tanh form), 3 = gelu (exact form) */
 enum { PEGAINFER_ACT_SILU = 0, PEGAINFER_ACT_RELU = 1, PEGAINFER_ACT_GELU_TANH = 2, PEGAINFER_ACT_GELU_ERF = 3 };
@@ -476,6 +501,8 @@ pegainfer_status_t pegainfer_decay_attention(const pegainfer_decay_attention_des
  * Per row of `proj` (dtype): q at q_off, k at k_off (heads x dim), v at v_off (heads x vdim);  z: fp32 [rows][heads * dim] at z_stride,
  * z_bias [heads * dim] of dtype or NULL:
  *   a = sigmoid(z + z_bias)^(1 / tau);  S <- diag(a) S + k v^T;  y = S^T (q * q_scale)          -> o (fp32 [rows][heads * vdim])
+ * With z NULL the scan makes z itself from the low-rank values of the row, z = w_up proj[row, low_off ..] (w_up [heads * dim][rank_stride]
+ * of dtype, columns past rank zero; pegainfer_gated_linear_fused_ok): one launch less for steps of few rows; no chunk form then.
  * Scan and chunk form, tables and scan_max as pegainfer_decay_attention (pegainfer_gated_linear_chunked_ok, ..._workspace). */
 typedef struct {
   const void* proj;
@@ -485,6 +512,9 @@ typedef struct {
   int64_t z_stride;
   const void* z_bias;
   float tau;
+  const void* w_up;
+  int64_t low_off;
+  int32_t rank, rank_stride;
   float* state;
   int64_t slot_stride;
   float* o;
@@ -503,6 +533,7 @@ typedef struct {
   int32_t dtype;
 } pegainfer_gated_linear_desc;
 int32_t pegainfer_gated_linear_chunked_ok(int32_t dim, int32_t vdim);
+int32_t pegainfer_gated_linear_fused_ok(int32_t rank, int32_t rank_stride, const void* w_up);
 int64_t pegainfer_gated_linear_workspace(int32_t n_chunks, int32_t heads, int32_t dim, int32_t vdim);
 pegainfer_status_t pegainfer_gated_linear(const pegainfer_gated_linear_desc* d, pegainfer_stream_t stream);
 /* Per-head RMS norm of a memory's read-out, a weight, a gate and a constant factor:

@@ -41,7 +41,7 @@ __global__ __launch_bounds__(256) void qk_prep_paged_kernel(
     const int32_t* __restrict__ page_ids, A* __restrict__ cache, int64_t page_stride, int64_t k_cache_off, int64_t v_cache_off,
     int page_size, float* __restrict__ q_out, A* __restrict__ q_out_stored, const A* __restrict__ q_bias,
     const A* __restrict__ k_bias, const A* __restrict__ v_bias, float qt_coef, int qt_every, PrepForm pf) {
-  extern __shared__ float sm[];   // [4 waves][dim]
+  extern __shared__ float sm[];   // [4 waves][dim], then the row's cosines and sines [rot_dims / 2] each
   __shared__ float red[4];
   const int row = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int pos = positions[row], e = row_entry[row];
@@ -66,6 +66,13 @@ __global__ __launch_bounds__(256) void qk_prep_paged_kernel(
     inv_all_k = 1.0f / sqrtf(block_sum<4>(sk, red) / (float)(G * dim) + eps);
   }
   const int half = rot_dims >> 1;
+  float *s_cs = sm + 4 * dim, *s_sn = s_cs + half;   // every head turns by the same angles
+  for (int f = threadIdx.x; f < half; f += 256) {
+    const float ang = (float)pos * inv_freq[f];
+    s_cs[f] = cosf(ang) * pf.rot_amp;
+    s_sn[f] = sinf(ang) * pf.rot_amp;
+  }
+  __syncthreads();
   // the row's heads are dealt to the workgroups of its grid column, a wave per head
   for (int hh = blockIdx.y * 4 + wave; hh < H + G; hh += 4 * gridDim.y) {
     const bool is_q = hh < H;
@@ -101,12 +108,10 @@ __global__ __launch_bounds__(256) void qk_prep_paged_kernel(
         if (i < rot_dims) {
           if (pf.rot_halves) {
             const int f = i < half ? i : i - half;
-            const float ang = (float)pos * inv_freq[f];
-            const float cs = cosf(ang) * pf.rot_amp, sn = sinf(ang) * pf.rot_amp;
+            const float cs = s_cs[f], sn = s_sn[f];
             out = i < half ? buf[i] * cs - buf[i + half] * sn : buf[i] * cs + buf[i - half] * sn;
           } else {
-            const float ang = (float)pos * inv_freq[i >> 1];
-            const float cs = cosf(ang) * pf.rot_amp, sn = sinf(ang) * pf.rot_amp;
+            const float cs = s_cs[i >> 1], sn = s_sn[i >> 1];
             out = (i & 1) ? buf[i] * cs + buf[i - 1] * sn : buf[i] * cs - buf[i + 1] * sn;
           }
         }
@@ -795,7 +800,7 @@ pegainfer_status_t pegainfer_qk_prep(const pegainfer_qk_prep_desc* p, pegainfer_
       using I = std::remove_pointer_t<decltype(ti)>;
       // few rows (decoding): the heads of a row spread over several workgroups, four heads each; many rows fill the chip alone
       const int per_row = p->n_rows >= 512 ? 1 : std::min(16, ceil_div(heads + kv_heads, 4));
-      qk_prep_paged_kernel<A, I><<<dim3(p->n_rows, per_row), 256, (size_t)4 * dim * sizeof(float), as_stream(stream)>>>(
+      qk_prep_paged_kernel<A, I><<<dim3(p->n_rows, per_row), 256, ((size_t)4 * dim + p->rot_dims) * sizeof(float), as_stream(stream)>>>(
           static_cast<const I*>(p->proj), p->proj_stride, p->q_off, p->k_off, p->v_off, heads, kv_heads, dim, p->vdim,
           static_cast<const A*>(p->q_norm), static_cast<const A*>(p->k_norm), p->eps, p->inv_freq, p->rot_dims, p->positions, p->row_entry,
           p->page_indptr, p->page_ids, static_cast<A*>(p->cache), p->page_stride, p->k_cache_off, p->v_cache_off, p->page_size, p->q_out,

@@ -26,6 +26,34 @@
 
 namespace pk {
 
+// sigmoid(z)^p through x = p (min(z, 0) - log(1 + e^-|z|)).  A decay near one multiplies hundreds of tokens, so its error must not lean to
+// one side: there the logarithm comes from the series of 2 artanh(t / (2 + t)) and e^x from its own series around 1, whose last step is
+// the only rounding that counts; a decay further down is forgotten before the hardware exponential's last bit shows.
+__device__ __forceinline__ float sigmoid_power(float z, float p) {
+  constexpr float kLog2e = 1.44269504088896341f;
+  const float t = __builtin_amdgcn_exp2f(-fabsf(z) * kLog2e);
+  const float s = t / (2.0f + t), q = s * s;           // s <= 1/3
+  float l = 2.0f / 15.0f;
+  l = fmaf(l, q, 2.0f / 13.0f);
+  l = fmaf(l, q, 2.0f / 11.0f);
+  l = fmaf(l, q, 2.0f / 9.0f);
+  l = fmaf(l, q, 2.0f / 7.0f);
+  l = fmaf(l, q, 2.0f / 5.0f);
+  l = fmaf(l, q, 2.0f / 3.0f);
+  l = fmaf(l, q, 2.0f);
+  const float x = (fminf(z, 0.f) - l * s) * p;
+  float e = 1.0f / 362880.0f;                          // (e^x - 1) / x for -1/2 < x <= 0
+  e = fmaf(e, x, 1.0f / 40320.0f);
+  e = fmaf(e, x, 1.0f / 5040.0f);
+  e = fmaf(e, x, 1.0f / 720.0f);
+  e = fmaf(e, x, 1.0f / 120.0f);
+  e = fmaf(e, x, 1.0f / 24.0f);
+  e = fmaf(e, x, 1.0f / 6.0f);
+  e = fmaf(e, x, 0.5f);
+  e = fmaf(e, x, 1.0f);
+  return x > -0.5f ? fmaf(e, x, 1.0f) : __builtin_amdgcn_exp2f(x * kLog2e);
+}
+
 template <typename A>
 struct GatedIn {
   const A* proj;
@@ -35,11 +63,15 @@ struct GatedIn {
   int64_t z_stride;
   const A* z_bias;             // [heads * dim], or NULL
   float inv_tau;
-  // sigmoid(z)^(1 / tau) through the logarithm of the sigmoid: exact at both ends
-  __device__ __forceinline__ float decay(float zb) const { return expf(logsigmoid_f(zb) * inv_tau); }
+  // with z NULL: the scan makes the decay inputs itself, W_up [heads * dim][rank_stride] times the row's `rank` values at low_off
+  const A* w_up;
+  int64_t low_off;
+  int rank, rank_stride;
+  __device__ __forceinline__ float decay(float zb) const { return sigmoid_power(zb, inv_tau); }
 };
+constexpr int kLowRank = 256;                        // most values of a row's low-rank part that the scan takes
 
-template <int NS, typename A>
+template <int NS, typename A, bool FUSED>
 __global__ __launch_bounds__(256) void gated_scan_kernel(GatedIn<A> in, float* __restrict__ state, int64_t slot_stride,
                                                          float* __restrict__ o, int H, int dim, int vdim,
                                                          const int32_t* __restrict__ entry_row0,
@@ -47,6 +79,7 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(GatedIn<A> in, float* _
   constexpr int DP = kRecSlices * NS;
   __shared__ __attribute__((aligned(16))) float s_k[kRecTokens][DP], s_q[kRecTokens][DP], s_a[kRecTokens][DP];
   __shared__ float s_v[kRecTokens][kRecCols];
+  __shared__ __attribute__((aligned(16))) float s_low[FUSED ? kLowRank : 4];
   const int e = blockIdx.z, h = blockIdx.y, col0 = blockIdx.x * kRecCols;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, cl = wave * 4 + (lane >> 4);
   const int col = col0 + cl;
@@ -64,7 +97,7 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(GatedIn<A> in, float* _
 #pragma unroll
   for (int j = 0; j < NS; ++j) {
     const int d = part + 16 * j;
-    bias[j] = in.z_bias && d < dim ? ld(in.z_bias + (int64_t)h * dim + d) : 0.f;
+    bias[j] = !FUSED && in.z_bias && d < dim ? ld(in.z_bias + (int64_t)h * dim + d) : 0.f;
   }
   RoundFetch<NS> nxt;
   float znx[NS];
@@ -75,6 +108,7 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(GatedIn<A> in, float* _
     nxt.issue(tc, tid, dim, [=](int tt, int d) { return ld(qb + (int64_t)tt * in.stride + d); },
               [=](int tt, int d) { return ld(kb + (int64_t)tt * in.stride + d); },
               [=](int tt, int c) { return col0 + c < vdim ? ld(vb + (int64_t)tt * in.stride + c) : 0.f; });
+    if constexpr (FUSED) return;
 #pragma unroll
     for (int j = 0; j < NS; ++j) {
       const int d = part + 16 * j;
@@ -86,26 +120,53 @@ __global__ __launch_bounds__(256) void gated_scan_kernel(GatedIn<A> in, float* _
     const int tc = min(kRecTokens, len - t0);
     __syncthreads();
     nxt.land(tid, s_q, s_k, s_v);
+    // rows past the entry's end: no decay, k = v = 0 - a step that leaves S as it is
+    if constexpr (FUSED) {
 #pragma unroll
-    for (int j = 0; j < NS; ++j)                     // rows past the entry's end: no decay, k = v = 0 - a step that leaves S as it is
-      s_a[tt_l][part + 16 * j] = tt_l < tc ? in.decay(znx[j] + bias[j]) : 1.0f;
+      for (int j = 0; j < NS; ++j) s_a[tt_l][part + 16 * j] = 1.0f;
+      for (int tt = 0; tt < tc; ++tt) {              // two threads per channel, eight values of the rank at a time
+        const A* low = in.proj + (int64_t)(row0 + t0 + tt) * in.stride + in.low_off;
+        __syncthreads();
+        if (tid < in.rank_stride) s_low[tid] = tid < in.rank ? ld(low + tid) : 0.f;
+        __syncthreads();
+        for (int d = tid >> 1; d < dim; d += 128) {
+          const A* wr = in.w_up + ((int64_t)h * dim + d) * in.rank_stride;
+          float sum = 0.f;
+          for (int c = (tid & 1) * 8; c < in.rank_stride; c += 16) {
+            float wv[8];
+            Vec8<A>::load(wr + c, wv);
+#pragma unroll
+            for (int u = 0; u < 8; ++u) sum = fmaf(wv[u], s_low[c + u], sum);
+          }
+          sum += __shfl_xor(sum, 1, kWave);
+          if (!(tid & 1)) s_a[tt][d] = in.decay(sum + (in.z_bias ? ld(in.z_bias + (int64_t)h * dim + d) : 0.f));
+        }
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < NS; ++j) s_a[tt_l][part + 16 * j] = tt_l < tc ? in.decay(znx[j] + bias[j]) : 1.0f;
+    }
     __syncthreads();
     if (t0 + kRecTokens < len) fetch(t0 + kRecTokens);
     float okeep = 0.f;
-    for (int t4 = 0; t4 < tc; t4 += 4) {             // no sum of a token feeds the state: four read-outs are in flight together
+    auto token = [&](int tt) {
+      const float vv = s_v[tt][cl];
+      float y0 = 0.f, y1 = 0.f;
 #pragma unroll
-      for (int uu = 0; uu < 4; ++uu) {
-        const int tt = t4 + uu;
-        const float vv = s_v[tt][cl];
-        float y0 = 0.f, y1 = 0.f;
+      for (int i = 0; i < NS; ++i) {
+        const float kk = s_k[tt][r * NS + i], qq = s_q[tt][r * NS + i], aa = s_a[tt][r * NS + i];
+        S[i] = fmaf(vv, kk, aa * S[i]);
+        if (i & 1) y1 = fmaf(S[i], qq, y1); else y0 = fmaf(S[i], qq, y0);
+      }
+      const float y = row16_sum(y0 + y1) * in.q_scale;
+      okeep = tt == r ? y : okeep;
+    };
+    if (tc == 1) {
+      token(0);
+    } else {
+      for (int t4 = 0; t4 < tc; t4 += 4) {           // no sum of a token feeds the state: four read-outs are in flight together
 #pragma unroll
-        for (int i = 0; i < NS; ++i) {
-          const float kk = s_k[tt][r * NS + i], qq = s_q[tt][r * NS + i], aa = s_a[tt][r * NS + i];
-          S[i] = fmaf(vv, kk, aa * S[i]);
-          if (i & 1) y1 = fmaf(S[i], qq, y1); else y0 = fmaf(S[i], qq, y0);
-        }
-        const float y = row16_sum(y0 + y1) * in.q_scale;
-        okeep = tt == r ? y : okeep;
+        for (int uu = 0; uu < 4; ++uu) token(t4 + uu);
       }
     }
     if (r < tc && col < vdim) o[(int64_t)(row0 + t0 + r) * ((int64_t)H * vdim) + (int64_t)h * vdim + col] = okeep;
@@ -400,6 +461,10 @@ int32_t pegainfer_gated_linear_chunked_ok(int32_t dim, int32_t vdim) {
          gated_out_lds(dim, vdim) + kGatedStatic <= kLdsMost;
 }
 
+int32_t pegainfer_gated_linear_fused_ok(int32_t rank, int32_t rank_stride, const void* w_up) {
+  return rank > 0 && rank <= rank_stride && rank_stride <= kLowRank && rank_stride % 8 == 0 && host_aligned16(w_up);
+}
+
 int64_t pegainfer_gated_linear_workspace(int32_t n_chunks, int32_t heads, int32_t dim, int32_t vdim) {
   return (int64_t)n_chunks * heads * pad_channels(dim) * (pad_values(vdim) + 1);
 }
@@ -409,10 +474,11 @@ pegainfer_status_t pegainfer_gated_linear(const pegainfer_gated_linear_desc* q, 
   if (!q) return bad;
   if (q->n_entries <= 0) return 0;
   const int H = q->heads, dim = q->dim, vdim = q->vdim;
-  if (H <= 0 || H > 65535 || dim <= 0 || dim > 256 || vdim <= 0 || q->n_entries > 65535 || !(q->tau > 0.f) || !q->proj || !q->z ||
+  if (H <= 0 || H > 65535 || dim <= 0 || dim > 256 || vdim <= 0 || q->n_entries > 65535 || !(q->tau > 0.f) || !q->proj ||
       !q->state || !q->o || !q->entry_row0 || !q->entry_slot)
     return bad;
-  const bool chunks = q->n_chunks > 0 && q->n_long > 0;
+  const bool chunks = q->n_chunks > 0 && q->n_long > 0, fused = !q->z;
+  if (fused && (chunks || !q->w_up || !pegainfer_gated_linear_fused_ok(q->rank, q->rank_stride, q->w_up))) return bad;
   if (chunks && (!pegainfer_gated_linear_chunked_ok(dim, vdim) || !q->workspace || !q->chunk_row0 || !q->chunk_rows || !q->long_chunk0 ||
                  !q->long_slot || q->scan_max <= 0 || q->n_long > 65535))
     return bad;
@@ -421,11 +487,15 @@ pegainfer_status_t pegainfer_gated_linear(const pegainfer_gated_linear_desc* q, 
   const bool known = by_dtype(q->dtype, [&](auto* t) {
     using A = std::remove_pointer_t<decltype(t)>;
     const GatedIn<A> in{static_cast<const A*>(q->proj), q->proj_stride, q->q_off, q->k_off, q->v_off, q->q_scale, q->z, q->z_stride,
-                        static_cast<const A*>(q->z_bias), 1.0f / q->tau};
+                        static_cast<const A*>(q->z_bias), 1.0f / q->tau, static_cast<const A*>(q->w_up), q->low_off, q->rank, q->rank_stride};
     if (q->n_entries > (chunks ? q->n_long : 0))
       ok = by_slices(dim, [&](auto ns) {
-        gated_scan_kernel<decltype(ns)::value, A><<<dim3(ceil_div(vdim, kRecCols), H, q->n_entries), 256, 0, st>>>(
-            in, q->state, q->slot_stride, q->o, H, dim, vdim, q->entry_row0, q->entry_slot, chunks ? q->scan_max : 0);
+        auto scan = [&](auto kern) {
+          kern<<<dim3(ceil_div(vdim, kRecCols), H, q->n_entries), 256, 0, st>>>(in, q->state, q->slot_stride, q->o, H, dim, vdim, q->entry_row0,
+                                                                                q->entry_slot, chunks ? q->scan_max : 0);
+        };
+        if (fused) scan(gated_scan_kernel<decltype(ns)::value, A, true>);
+        else scan(gated_scan_kernel<decltype(ns)::value, A, false>);
       });
     if (!ok || !chunks) return;
     float* total = q->workspace + (int64_t)q->n_chunks * H * pad_channels(dim) * pad_values(vdim);

@@ -9,7 +9,8 @@
 //              right: W_a2 (W_a1 h) in fp32, the recurrence over the request's fp32 state, norm * gate * right_scale (one launch);
 //              both leave their heads side by side in one row, and ONE GEMM over [W_o | W_o] gives the sum
 //   ff       : [router ; shared gate] h in fp32, selection and sort by expert, the experts' two GEMMs (gelu in the first one's
-//              epilogue), the shared expert, weighted sum with the input's own row for identity experts
+//              epilogue), the shared expert; the weighted sum, with the input's own row for identity experts, is made in the launch that
+//              norms it, adds it to the stream and norms for the next layer
 //   logits   : W_head norm(x) on the wanted rows, fp32 out
 // Cache: page-first [page][layer][k: slot, kv head, rotated values | v: slot, kv head, dim] - the values are the unrotated keys, so the
 // part of a key that the rotation does not reach is read from them.
@@ -24,6 +25,7 @@ using namespace pstep;
 constexpr int kSplitGroups = 512;   // most (tile, kv head, key split) workgroups of an attention launch that cuts its keys
 constexpr int kMaxSplits = 16;
 constexpr int kFewTiles = 128;      // launches of fewer workgroups deal their keys to several
+constexpr int kFusedRows = 8;       // steps of at most so many rows make the decay inputs inside the scan
 constexpr int kScanMax = 32;        // longest entry whose recurrence runs token by token
 constexpr int kSyntheticRank = 32;  // of the decays' two-step projection when no tensor tells it
 constexpr float kGainOffset = 1.0f; // the stream's norm weights are stored around zero
@@ -83,7 +85,7 @@ class Model : public StepModel {
         return set_error("config: embedding.bigram needs positive buckets and multipliers of at most 2^31");
     }
     const Json* ls = j.get("layers");
-    if (D <= 0 || V <= 0 || !ls || ls->kind != Json::Arr || ls->arr.empty()) return set_error("config: width / vocab / layers missing");
+    if (D <= 0 || D > 32768 || V <= 0 || !ls || ls->kind != Json::Arr || ls->arr.empty()) return set_error("config: width / vocab / layers missing");
     for (size_t i = 0; i < ls->arr.size(); ++i) {
       LayerCfg c;
       if (parse_layer(ls->arr[i], (int)i, &c)) return -1;
@@ -321,13 +323,17 @@ class Model : public StepModel {
     d.eps = eps; d.gain_offset = kGainOffset; d.n_dtype = dtype; d.d = D; d.rows = rows; d.dtype = dtype;
     return d;
   }
-  // the end of a sublayer and the start of the next: y, normed, joins the stream, and `next` (NULL: nothing follows) leaves h
+  // the end of a sublayer and the start of the next: its output, normed, joins the stream, and `next` (NULL: nothing follows) leaves h
+  pegainfer_join_rms_desc join_desc(const StepCtx& s, const void* post, const void* next) const {
+    pegainfer_join_rms_desc d{};
+    d.x = x; d.post = post; d.gain = next; d.n_out = next ? h : nullptr;
+    d.eps = eps; d.gain_offset = kGainOffset; d.d = D; d.rows = s.T; d.dtype = dtype;
+    return d;
+  }
   int join(const StepCtx& s, const void* post, const void* next) {
-    pegainfer_sum_term t{y, D, nullptr, post, 1.0f};
-    pegainfer_terms_rms_desc d = norm_desc(s.T);
-    d.x_in = x; d.x_out = x; d.terms = &t; d.n_terms = 1;
-    if (next) { d.gain = next; d.n_out = h; }
-    PSTEP_K(pegainfer_terms_rms(&d, S()));
+    pegainfer_join_rms_desc d = join_desc(s, post, next);
+    d.y = y; d.y_row_stride = D;
+    PSTEP_K(pegainfer_join_rms(&d, S()));
     return 0;
   }
   int attention(const StepCtx& s, const LayerCfg& c, const LayerW& w) {
@@ -357,11 +363,16 @@ class Model : public StepModel {
   int memory(const StepCtx& s, const LayerCfg& c, const LayerW& w) {
     const MemCfg& m = c.right;
     const int rd = m.heads * m.dim;
-    if (linear_strided(w.a2, at(proj, (size_t)m.o_a), dtype, c.proj_rows, z32, PEGAINFER_DTYPE_F32, rd, s.T, pad8(m.rank))) return -1;
+    const int rp = pad8(m.rank);
+    // few rows: the scan makes the decay inputs itself (its workgroups read W_a2 once per row)
+    const bool fused = s.T <= kFusedRows && s.chunks.n_long == 0 && !plain_kernels && pegainfer_gated_linear_fused_ok(m.rank, rp, w.a2);
+    if (!fused && linear_strided(w.a2, at(proj, (size_t)m.o_a), dtype, c.proj_rows, z32, PEGAINFER_DTYPE_F32, rd, s.T, rp)) return -1;
     pegainfer_gated_linear_desc d{};
     d.proj = proj; d.proj_stride = c.proj_rows; d.q_off = m.o_q; d.k_off = m.o_k; d.v_off = m.o_v;
     d.q_scale = (float)(1.0 / std::sqrt((double)m.dim));
-    d.z = z32; d.z_stride = rd; d.z_bias = w.a2_bias; d.tau = m.tau;
+    if (fused) { d.w_up = w.a2; d.low_off = m.o_a; d.rank = m.rank; d.rank_stride = rp; }
+    else { d.z = z32; d.z_stride = rd; }
+    d.z_bias = w.a2_bias; d.tau = m.tau;
     d.state = state + m.st_off; d.slot_stride = state_layout.floats_per_slot(); d.o = o32;
     d.heads = m.heads; d.dim = m.dim; d.vdim = m.vdim;
     d.entry_row0 = s.row0; d.entry_slot = s.slot; d.n_entries = s.n;
@@ -377,8 +388,8 @@ class Model : public StepModel {
                                     at(mix, (size_t)c.mix_right), c.mix_cols, m.heads, m.vdim, s.T, dtype, S()));
     return 0;
   }
-  // h -> y
-  int feed_forward(const StepCtx& s, const LayerCfg& c, const LayerW& w) {
+  // h -> the stream, and h of the next layer
+  int feed_forward(const StepCtx& s, const LayerCfg& c, const LayerW& w, const void* next) {
     const MoeCfg& f = c.moe;
     const int T = s.T, P = T * f.top, all = f.experts + f.identity;
     const bool tuned = dtype == PEGAINFER_DTYPE_BF16 && !plain_kernels && T > 8;      // many rows in bf16
@@ -391,7 +402,7 @@ class Model : public StepModel {
     r.sort_experts = f.experts;
     r.pos_pair = pos_pair; r.pos_row = pos_row;
     r.tile_group = tiles; r.tile_row0 = tiles + max_tiles; r.tile_rows = tiles + 2 * max_tiles; r.n_tiles = tiles + 3 * max_tiles;
-    r.max_tiles = (P + per_tile - 1) / per_tile + f.experts; r.rows_per_tile = per_tile; r.dtype = dtype;
+    r.max_tiles = std::min(P, (P + per_tile - 1) / per_tile + f.experts); r.rows_per_tile = per_tile; r.dtype = dtype;
     PSTEP_K(pegainfer_route_plan(&r, S()));
     pegainfer_gemm_desc g{};
     g.tile_group = r.tile_group; g.tile_row0 = r.tile_row0; g.tile_rows = r.tile_rows; g.n_tiles = r.n_tiles; g.max_tiles = r.max_tiles;
@@ -421,8 +432,11 @@ class Model : public StepModel {
       }
       if (linear(w.down_s, act_s, y_s, D, T, f.shared_ff)) return -1;
     }
-    PSTEP_K(pegainfer_route_combine_same(y_pairs, route_w, route_e, f.experts, f.identity ? h : nullptr, D, f.shared_ff ? y_s : nullptr,
-                                         logits_r + all, all + 1, y, D, f.top, T, dtype, S()));
+    pegainfer_join_rms_desc j = join_desc(s, w.norm2b, next);
+    j.y_pairs = y_pairs; j.weight = route_w; j.expert = route_e; j.top = f.top; j.same_from = f.experts;
+    if (f.identity) { j.same = h; j.same_stride = D; }
+    if (f.shared_ff) { j.add = y_s; j.add_gate = logits_r + all; j.add_gate_stride = all + 1; }
+    PSTEP_K(pegainfer_join_rms(&j, S()));
     return 0;
   }
   int run_step(const StepCtx& s) override {
@@ -438,8 +452,8 @@ class Model : public StepModel {
       const LayerW& w = weights[i];
       const void* next = i + 1 < layers.size() ? weights[i + 1].norm1 : nullptr;
       if (linear(w.proj, h, proj, c.proj_rows, s.T, D) || attention(s, c, w) || memory(s, c, w) || linear(w.o, mix, y, D, s.T, c.mix_cols)) return -1;
-      if (c.moe.ff && (join(s, w.norm1b, w.norm2) || feed_forward(s, c, w) || join(s, w.norm2b, next))) return -1;
-      if (!c.moe.ff && join(s, w.norm1b, next)) return -1;
+      if (join(s, w.norm1b, c.moe.ff ? w.norm2 : next)) return -1;
+      if (c.moe.ff && feed_forward(s, c, w, next)) return -1;
       if (tap_on) PSTEP_HIP(hipMemcpyAsync(tap_at((int)i), x, (size_t)s.T * D * 4, hipMemcpyDeviceToDevice, stream));
     }
     if (s.W > 0) {

@@ -182,12 +182,23 @@ struct SortOut {
   int32_t *pos_pair, *pos_row, *tile_group, *tile_row0, *tile_rows, *n_tiles;
   int max_tiles, per_tile;
 };
-// Pairs whose expert number is E or more (identity experts) get no position.  One workgroup; cnt: [2 E] of LDS.
+// Pairs whose expert number is E or more (identity experts) get no position.  One workgroup of N threads; cnt: [2 E] of LDS.
+template <int N>
 __device__ __forceinline__ void route_sort_block(const int32_t* expert, int n_pairs, int top, int E, const SortOut& o, int* cnt) {
   int* cur = cnt + E;            // [E] counts, then [E] cursors
-  for (int e = threadIdx.x; e < E; e += 256) cnt[e] = 0;
+  for (int e = threadIdx.x; e < E; e += N) cnt[e] = 0;
   __syncthreads();
-  for (int p = threadIdx.x; p < n_pairs; p += 256) {
+  constexpr int kKeep = 4;       // a thread's first choices stay in registers between the two walks
+  int mine[kKeep];
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int p = threadIdx.x + N * k;
+    mine[k] = p < n_pairs ? expert[p] : E;
+  }
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k)
+    if (mine[k] < E) atomicAdd(&cnt[mine[k]], 1);
+  for (int p = threadIdx.x + N * kKeep; p < n_pairs; p += N) {
     const int e = expert[p];
     if (e < E) atomicAdd(&cnt[e], 1);
   }
@@ -207,17 +218,20 @@ __device__ __forceinline__ void route_sort_block(const int32_t* expert, int n_pa
     *o.n_tiles = nt;
   }
   __syncthreads();
-  for (int p = threadIdx.x; p < n_pairs; p += 256) {
-    const int e = expert[p];
-    if (e >= E) continue;
+  auto place = [&](int p, int e) {
+    if (e >= E) return;
     const int at = atomicAdd(&cur[e], 1);
     o.pos_pair[at] = p;
     o.pos_row[at] = p / top;
-  }
+  };
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) place(threadIdx.x + N * k, mine[k]);
+  for (int p = threadIdx.x + N * kKeep; p < n_pairs; p += N) place(p, expert[p]);
 }
-__global__ __launch_bounds__(256) void route_sort_kernel(const int32_t* __restrict__ expert, int n_pairs, int top, int E, SortOut o) {
+constexpr int kSortThreads = 1024;
+__global__ __launch_bounds__(kSortThreads) void route_sort_kernel(const int32_t* __restrict__ expert, int n_pairs, int top, int E, SortOut o) {
   extern __shared__ int cnt[];
-  route_sort_block(expert, n_pairs, top, E, o, cnt);
+  route_sort_block<kSortThreads>(expert, n_pairs, top, E, o, cnt);
 }
 // Few rows (decoding): selection and sort in one launch of one workgroup, which sees its own choices after a barrier.
 template <typename A>
@@ -231,7 +245,7 @@ __global__ __launch_bounds__(256) void route_plan_kernel(const float* __restrict
   }
   __threadfence_block();
   __syncthreads();               // the choices are read by other waves of this workgroup; the selection's LDS is free
-  route_sort_block(out_e, rows * f.top, f.top, sort_experts, o, reinterpret_cast<int*>(sm));
+  route_sort_block<256>(out_e, rows * f.top, f.top, sort_experts, o, reinterpret_cast<int*>(sm));
 }
 
 // expert / same: pairs that chose an expert number of same_from or more take the row of `same` (the feed-forward's own input) instead
@@ -294,7 +308,7 @@ pegainfer_status_t pegainfer_route_plan(const pegainfer_route_plan_desc* q, pega
   const bool sorted = q->sort_experts > 0;
   if (sorted && ((q->rows_per_tile != 64 && q->rows_per_tile != 128) || q->sort_experts > 7000 || pairs > 0x7FFFFFFF || !q->pos_pair ||
                  !q->pos_row || !q->tile_group || !q->tile_row0 || !q->tile_rows || !q->n_tiles ||
-                 q->max_tiles < (pairs + q->rows_per_tile - 1) / q->rows_per_tile + q->sort_experts))
+                 q->max_tiles < std::min<int64_t>(pairs, (pairs + q->rows_per_tile - 1) / q->rows_per_tile + q->sort_experts)))
     return bad;
   const RouteForm f{E, groups, keep, top, q->score_kind, q->group_kind, q->renorm, q->factor, q->logits_stride};
   const SortOut o{q->pos_pair, q->pos_row, q->tile_group, q->tile_row0, q->tile_rows, q->n_tiles, q->max_tiles, q->rows_per_tile};
@@ -310,7 +324,7 @@ pegainfer_status_t pegainfer_route_plan(const pegainfer_route_plan_desc* q, pega
         route_from_logits_kernel<A><<<ceil_div(q->rows, 4), 256, smem, as_stream(stream)>>>(q->logits, corr, q->out_expert, q->out_weight,
                                                                                             q->rows, f);
         if (sorted)
-          route_sort_kernel<<<1, 256, sort_smem, as_stream(stream)>>>(q->out_expert, (int)pairs, top, q->sort_experts, o);
+          route_sort_kernel<<<1, kSortThreads, sort_smem, as_stream(stream)>>>(q->out_expert, (int)pairs, top, q->sort_experts, o);
       }))
     return bad;
   return (pegainfer_status_t)hipGetLastError();
@@ -351,7 +365,7 @@ pegainfer_status_t pegainfer_route_sort(const int32_t* expert, int32_t n_pairs, 
       max_tiles < (n_pairs + rows_per_tile - 1) / rows_per_tile + experts)
     return (pegainfer_status_t)hipErrorInvalidValue;
   const SortOut o{pos_pair, pos_row, tile_group, tile_row0, tile_rows, n_tiles, max_tiles, rows_per_tile};
-  route_sort_kernel<<<1, 256, (size_t)2 * experts * sizeof(int), as_stream(stream)>>>(expert, n_pairs, top, experts, o);
+  route_sort_kernel<<<1, kSortThreads, (size_t)2 * experts * sizeof(int), as_stream(stream)>>>(expert, n_pairs, top, experts, o);
   return (pegainfer_status_t)hipGetLastError();
 }
 

@@ -23,6 +23,7 @@
 namespace pk {
 
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.0f ? x : log1pf(expf(x)); }
+__device__ __forceinline__ float logsigmoid_f(float x) { return fminf(x, 0.0f) - log1pf(expf(-fabsf(x))); }
 
 // Per row, before the recurrence: q and k heads made unit vectors in place (x / sqrt(sum(x^2) + 1e-6), q also * dim^-1/2),
 // gates[row] = [g: heads | beta: heads].  One workgroup per row, a wave per head.

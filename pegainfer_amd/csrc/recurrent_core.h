@@ -6,8 +6,6 @@
 
 namespace pk {
 
-__device__ __forceinline__ float logsigmoid_f(float x) { return fminf(x, 0.0f) - log1pf(expf(-fabsf(x))); }
-
 constexpr int kRecTokens = 16;   // tokens staged per round
 constexpr int kRecCols = 16;     // value columns per workgroup (four per wave)
 constexpr int kRecSlices = 16;   // lanes that share one column

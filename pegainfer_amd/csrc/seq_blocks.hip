@@ -14,6 +14,8 @@
 //                           sublayers all read the same normed input, and opens the next
 //                           (its stream may be read through a row index, or start as an embedding row plus the row of a table
 //                           addressed by the previous and the current token)
+//   join_rms_kernel         one normed output joins the stream in place and the next norm follows, with everything a row needs in
+//                           registers from the start; the output may be the weighted sum of routed experts, made on the way
 //   glu_rows_kernel         act(gate) * up from two column ranges of a wider row (silu, relu, tanh-gelu or erf-gelu)
 //   act_rows_kernel         the same activations alone
 //   softcap_rows_kernel     cap * tanh(x / cap) on fp32 rows
@@ -534,6 +536,95 @@ __global__ __launch_bounds__(256) void terms_rms_add_kernel(RowSource src, SumTe
   }
 }
 
+// One sublayer output, normed, joins the stream in place; the next norm leaves its input.  N threads, NPT values each (d <= N * NPT): what
+// the row needs is requested at once and stays in registers, so a step of few rows pays one memory latency and two sums.  ROUTED: the
+// output is the weighted sum of routed experts, made here (n_out may be the buffer `same` lies in: a row is read before it is written).
+template <typename A>
+struct JoinSource {
+  const A* y; int64_t y_stride;
+  const float *pairs, *weight; const int32_t* expert; int top, same_from;
+  const A* same; int64_t same_stride;
+  const A* add; const float* add_gate; int64_t add_gate_stride;
+};
+template <typename A, int N, int NPT, bool VEC, bool ROUTED>
+__global__ __launch_bounds__(N) void join_rms_kernel(float* __restrict__ x, JoinSource<A> src, const A* __restrict__ post,
+                                                     const A* __restrict__ gain, float eps, float gain_offset, A* n_out, int d) {
+  __shared__ float red[N / 64];
+  constexpr int V = VEC ? 4 : 1, NV = NPT / V;
+  const int row = blockIdx.x;
+  float* xr = x + (int64_t)row * d;
+  float y[NV][V], xv[NV][V], pw[NV][V], gw[NV][V];
+  auto load = [&](const auto* p, float* o) {
+    if constexpr (VEC) ld4(p, o); else o[0] = ld(p);
+  };
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (threadIdx.x + N * k) * V;
+#pragma unroll
+    for (int u = 0; u < V; ++u) { y[k][u] = 0.f; xv[k][u] = 0.f; }
+    if (i >= d) continue;
+    load(xr + i, xv[k]);
+    load(post + i, pw[k]);
+    if (gain) load(gain + i, gw[k]);
+    if constexpr (!ROUTED) {
+      load(src.y + (int64_t)row * src.y_stride + i, y[k]);
+    } else if (src.add) {
+      load(src.add + (int64_t)row * d + i, y[k]);
+    }
+  }
+  if constexpr (ROUTED) {
+    const float g = src.add && src.add_gate ? sigmoid_f(src.add_gate[(int64_t)row * src.add_gate_stride]) : 1.0f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k)
+#pragma unroll
+      for (int u = 0; u < V; ++u) y[k][u] *= g;
+#pragma unroll 4
+    for (int c = 0; c < src.top; ++c) {
+      const int64_t at = (int64_t)row * src.top + c;
+      const float w = src.weight[at];
+      const bool own = src.same && src.expert[at] >= src.same_from;       // uniform over the workgroup
+#pragma unroll
+      for (int k = 0; k < NV; ++k) {
+        const int i = (threadIdx.x + N * k) * V;
+        if (i >= d) continue;
+        float v[V];
+        if (own) load(src.same + (int64_t)row * src.same_stride + i, v); else load(src.pairs + at * d + i, v);
+#pragma unroll
+        for (int u = 0; u < V; ++u) y[k][u] = fmaf(w, v[u], y[k][u]);
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k)
+#pragma unroll
+    for (int u = 0; u < V; ++u) ss = fmaf(y[k][u], y[k][u], ss);
+  const float inv = 1.0f / sqrtf(block_sum<N / 64>(ss, red) / (float)d + eps);
+  ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (threadIdx.x + N * k) * V;
+    if (i >= d) continue;
+#pragma unroll
+    for (int u = 0; u < V; ++u) {
+      xv[k][u] += y[k][u] * inv * (gain_offset + pw[k][u]);
+      ss = fmaf(xv[k][u], xv[k][u], ss);
+    }
+    if constexpr (VEC) st4(xr + i, xv[k]); else xr[i] = xv[k][0];
+  }
+  if (!gain) return;                       // uniform over the grid
+  const float sc = 1.0f / sqrtf(block_sum<N / 64>(ss, red) / (float)d + eps);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = (threadIdx.x + N * k) * V;
+    if (i >= d) continue;
+    float o[V];
+#pragma unroll
+    for (int u = 0; u < V; ++u) o[u] = xv[k][u] * sc * (gain_offset + gw[k][u]);
+    if constexpr (VEC) st4(n_out + (int64_t)row * d + i, o); else st(n_out + (int64_t)row * d + i, o[0]);
+  }
+}
+
 // out[row, i] = act(gate[row, i]) * up[row, i]; gate and up are column ranges of rows with one stride
 template <typename A>
 __global__ __launch_bounds__(256) void glu_rows_kernel(const A* __restrict__ gate, const A* __restrict__ up, int64_t in_stride,
@@ -620,6 +711,49 @@ pegainfer_status_t pegainfer_terms_rms(const pegainfer_terms_rms_desc* q, pegain
     });
   });
   return known && ok ? (pegainfer_status_t)hipGetLastError() : PK_BAD;
+}
+
+pegainfer_status_t pegainfer_join_rms(const pegainfer_join_rms_desc* q, pegainfer_stream_t stream) {
+  if (!q) return PK_BAD;
+  if (q->rows <= 0) return 0;
+  const int d = q->d;
+  const bool routed = q->y_pairs != nullptr;
+  if (d <= 0 || d > 32768 || !q->x || !q->post || (!routed && !q->y) || (q->gain && !q->n_out) ||
+      (routed && (!q->weight || q->top <= 0 || (q->same && !q->expert))))
+    return PK_BAD;
+  if (!by_dtype(q->dtype, [&](auto* t) {
+        using A = std::remove_pointer_t<decltype(t)>;
+        const JoinSource<A> src{static_cast<const A*>(q->y), q->y_row_stride, q->y_pairs, q->weight, q->expert, q->top, q->same_from,
+                                static_cast<const A*>(q->same), q->same_stride, static_cast<const A*>(q->add), q->add_gate, q->add_gate_stride};
+        const bool vec = d % 4 == 0 && q->y_row_stride % 4 == 0 && q->same_stride % 4 == 0 && host_aligned16(q->x) && host_aligned16(q->y) &&
+                         host_aligned16(q->y_pairs) && host_aligned16(q->same) && host_aligned16(q->add) && host_aligned16(q->post) &&
+                         host_aligned16(q->gain) && host_aligned16(q->n_out);
+        auto launch = [&](auto kern, int threads) {
+          kern<<<q->rows, threads, 0, as_stream(stream)>>>(q->x, src, static_cast<const A*>(q->post), static_cast<const A*>(q->gain), q->eps,
+                                                          q->gain_offset, static_cast<A*>(q->n_out), d);
+        };
+        auto shape = [&](auto n, auto npt) {
+          constexpr int N = decltype(n)::value, NPT = decltype(npt)::value;
+          if (routed) {
+            if (vec) launch(join_rms_kernel<A, N, NPT, true, true>, N);
+            else launch(join_rms_kernel<A, N, NPT, false, true>, N);
+          } else {
+            if (vec) launch(join_rms_kernel<A, N, NPT, true, false>, N);
+            else launch(join_rms_kernel<A, N, NPT, false, false>, N);
+          }
+        };
+        const std::integral_constant<int, 256> narrow;
+        const std::integral_constant<int, 1024> wide;
+        const bool few = q->rows < 128;              // few rows: a row over more threads
+        if (d <= 1024) shape(narrow, std::integral_constant<int, 4>());
+        else if (few && d <= 4096) shape(wide, std::integral_constant<int, 4>());
+        else if (d <= 2048) shape(narrow, std::integral_constant<int, 8>());
+        else if (d <= 4096) shape(narrow, std::integral_constant<int, 16>());
+        else if (d <= 8192) shape(wide, std::integral_constant<int, 8>());
+        else shape(wide, std::integral_constant<int, 32>());
+      }))
+    return PK_BAD;
+  return (pegainfer_status_t)hipGetLastError();
 }
 
 pegainfer_status_t pegainfer_act_rows(const void* in, int64_t in_row_stride, void* out, int64_t out_row_stride, int32_t I, int32_t rows,

@@ -643,8 +643,8 @@ QkPrepDesc = _struct("QkPrepDesc", [("p", "proj"), ("i", "proj_dtype"), ("l", "p
                                     ("p", "positions row_entry page_indptr page_ids cache"), ("l", "page_stride k_cache_off v_cache_off"),
                                     ("i", "page_size shared_tail"), ("p", "q_out q_out_stored"), ("i", "n_rows dtype")])
 GatedLinearDesc = _struct("GatedLinearDesc", [("p", "proj"), ("l", "proj_stride q_off k_off v_off"), ("f", "q_scale"), ("p", "z"), ("l", "z_stride"),
-                                              ("p", "z_bias"), ("f", "tau"), ("p", "state"), ("l", "slot_stride"), ("p", "o"),
-                                              ("i", "heads dim vdim"), ("p", "entry_row0 entry_slot"), ("i", "n_entries scan_max"),
+                                              ("p", "z_bias"), ("f", "tau"), ("p", "w_up"), ("l", "low_off"), ("i", "rank rank_stride"), ("p", "state"),
+                                              ("l", "slot_stride"), ("p", "o"), ("i", "heads dim vdim"), ("p", "entry_row0 entry_slot"), ("i", "n_entries scan_max"),
                                               ("p", "chunk_row0 chunk_rows"), ("i", "n_chunks"), ("p", "long_chunk0 long_slot"), ("i", "n_long"),
                                               ("p", "workspace"), ("i", "dtype")])
 
@@ -666,6 +666,25 @@ def terms_rms(dtype, d, x=None, row_index=None, embed=None, token_ids=None, embe
                      n_dtype=_dt(n) if n is not None else 0, d=d, rows=rows, dtype=0 if dtype == torch.bfloat16 else 1)
     _chk(ffi.lib().pegainfer_terms_rms(ctypes.addressof(q), _stream()), "terms_rms")
     return r, n
+
+
+JoinRmsDesc = _struct("JoinRmsDesc", [("p", "x y"), ("l", "y_row_stride"), ("p", "y_pairs weight expert"), ("i", "top same_from"), ("p", "same"),
+                                      ("l", "same_stride"), ("p", "add add_gate"), ("l", "add_gate_stride"), ("p", "post gain"),
+                                      ("f", "eps gain_offset"), ("p", "n_out"), ("i", "d rows dtype")])
+
+
+def join_rms(x_f32, post, gain=None, eps=1e-5, gain_offset=0.0, y=None, y_pairs=None, weight=None, expert=None, same_from=0, same=None, add=None,
+             add_gate_f32=None):
+    """x (in place) += rms_norm(y) * (gain_offset + post); -> rms_norm(x) * (gain_offset + gain) or None.  y: rows of the weights' type, or the
+    weighted sum of routed experts from y_pairs fp32 [rows * top, d]"""
+    rows, d = x_f32.shape
+    n = torch.empty((rows, d), dtype=post.dtype, device=post.device) if gain is not None else None
+    q = JoinRmsDesc(x=_p(x_f32), y=_p(y), y_row_stride=0 if y is None else y.stride(0), y_pairs=_p(y_pairs), weight=_p(weight), expert=_p(expert),
+                    top=0 if weight is None else weight.shape[1], same_from=same_from, same=_p(same), same_stride=0 if same is None else same.stride(0),
+                    add=_p(add), add_gate=_p(add_gate_f32), add_gate_stride=0 if add_gate_f32 is None else add_gate_f32.stride(0), post=_p(post),
+                    gain=_p(gain), eps=float(eps), gain_offset=float(gain_offset), n_out=_p(n), d=d, rows=rows, dtype=_dt(post))
+    _chk(ffi.lib().pegainfer_join_rms(ctypes.addressof(q), _stream()), "join_rms")
+    return n
 
 
 def act_rows(x, act):
@@ -717,12 +736,14 @@ def qk_prep(proj, offs, heads, kv_heads, dim, vdim, rg, page_indptr, page_ids, c
     return q
 
 
-def gated_linear(proj, offs, z_f32, z_bias, tau, q_scale, state, heads, dim, vdim, rg, scan_max=0):
-    """proj rows [.. q at offs[0] | k at offs[1] | v at offs[2] ..]; z fp32 [rows, heads * dim]; state fp32 [slots, heads * dim * vdim];
-    scan_max > 0: entries of more rows take the chunk form -> fp32 [rows, heads * vdim]"""
+def gated_linear(proj, offs, z_f32, z_bias, tau, q_scale, state, heads, dim, vdim, rg, scan_max=0, w_up=None, low_off=0, rank=0):
+    """proj rows [.. q at offs[0] | k at offs[1] | v at offs[2] ..]; z fp32 [rows, heads * dim], or None: w_up [heads * dim, rank padded to 8]
+    times the row's rank values at low_off; state fp32 [slots, heads * dim * vdim]; scan_max > 0: entries of more rows take the chunk form
+    -> fp32 [rows, heads * vdim]"""
     o = torch.empty((proj.shape[0], heads * vdim), dtype=torch.float32, device=proj.device)
     d = GatedLinearDesc(proj=_p(proj), proj_stride=proj.stride(0), q_off=offs[0], k_off=offs[1], v_off=offs[2], q_scale=float(q_scale),
-                        z=_p(z_f32), z_stride=z_f32.stride(0), z_bias=_p(z_bias), tau=float(tau), state=_p(state),
+                        z=_p(z_f32), z_stride=0 if z_f32 is None else z_f32.stride(0), z_bias=_p(z_bias), tau=float(tau), w_up=_p(w_up),
+                        low_off=low_off, rank=rank, rank_stride=0 if w_up is None else w_up.stride(0), state=_p(state),
                         slot_stride=state.stride(0), o=_p(o), heads=heads, dim=dim, vdim=vdim, entry_row0=_p(rg.entry_row0),
                         entry_slot=_p(rg.entry_slot), n_entries=len(rg.lens), dtype=_dt(proj))
     keep = _chunk_tables(d, rg, scan_max, ffi.lib().pegainfer_gated_linear_workspace, heads, dim, vdim)  # noqa: F841 (alive until enqueued)

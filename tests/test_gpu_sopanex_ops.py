@@ -56,6 +56,41 @@ def test_normed_output_joins_the_stream_and_the_next_norm_reads_it(dtype, d):
 
 
 @BOTH
+@pytest.mark.parametrize("rows", [1, 6, 200])
+@pytest.mark.parametrize("d", [50, 1024, 1030, 2048, 4096, 4100, 8192, 9000])
+def test_one_launch_joins_norms_and_sums_routed_experts(dtype, rows, d):
+    if rows == 200 and d > 2048:
+        rows = 130
+    g = torch.Generator().manual_seed(d + rows)
+    x, y = torch.randn(rows, d, generator=g) * 2, draw(rows, d, seed=1, scale=3.0)
+    post, gain = draw(d, seed=2, scale=0.3), draw(d, seed=3, scale=0.3)
+    xs = x.cuda()
+    n = B().join_rms(xs, dev(post, dtype), dev(gain, dtype), eps=1e-3, gain_offset=1.0, y=dev(y, dtype))
+    ref = x.double() + R.zrms(y.double(), post.double(), 1e-3)
+    close(xs, ref, "float32", tol32=3e-6)
+    close(n, R.zrms(ref, gain.double(), 1e-3), dtype, tol16=1e-2)
+    E, I, top = 3, 2, 3
+    e = torch.stack([torch.randperm(E + I, generator=g)[:top] for _ in range(rows)]).int()
+    wt, yp = torch.rand(rows, top, generator=g), torch.randn(rows * top, d, generator=g)
+    yp[(e.view(-1) >= E)] = float("nan")                         # rows no expert has written
+    h, add, gate = draw(rows, d, seed=11), draw(rows, d, seed=12), torch.randn(rows, 4, generator=g)
+    own = (e >= E)[:, :, None]
+    routed = (wt.double()[:, :, None] * torch.where(own, h.double()[:, None], yp.double().view(rows, top, d))).sum(1)
+    for extra in (False, True):
+        xs = x.cuda()
+        kw = dict(add=dev(add, dtype), add_gate_f32=gate.cuda()[:, 2]) if extra else {}
+        n = B().join_rms(xs, dev(post, dtype), None if extra else dev(gain, dtype), eps=1e-5, gain_offset=1.0, y_pairs=yp.cuda(), weight=wt.cuda(),
+                         expert=e.cuda(), same_from=E, same=dev(h, dtype), **kw)
+        t = routed + add.double() * torch.sigmoid(gate[:, 2:3].double()) if extra else routed
+        ref = x.double() + R.zrms(t, post.double(), 1e-5)
+        close(xs, ref, "float32", tol32=3e-6)
+        if extra:
+            assert n is None
+        else:
+            close(n, R.zrms(ref, gain.double(), 1e-5), dtype, tol16=1e-2)
+
+
+@BOTH
 @pytest.mark.parametrize("buckets,muls", [(1, (3, 2)), (29, (3, 17)), (301, (65537, 2147483647))])
 def test_stream_starts_from_embedding_and_token_pair_rows(dtype, buckets, muls):
     d, toks = 72, [39, 0, 7, 7, 38]
@@ -360,3 +395,25 @@ def test_channels_that_forget_at_once_and_remember_again(dtype):
         assert torch.isfinite(outs[0]).all()
         close(outs[0], ref, "float32", tol32=1e-5)
         close(state[0], end, "float32", tol32=1e-5)
+
+
+@BOTH
+@pytest.mark.parametrize("m,rank", [(SIZES[0], 6), (SIZES[2], 5), (SIZES[3], 24), (SIZES[4], 96), (SIZES[6], 250)], ids=lambda v: str(v) if isinstance(v, int) else "")
+def test_scan_makes_the_decay_inputs_itself(dtype, m, rank):
+    """one to four tokens of two requests, the low-rank values inside the rows: the same outputs and states as with the inputs given"""
+    Bk = B()
+    H, dk, dv = m["heads"], m["dim"], m["vdim"]
+    rp, wq = (rank + 7) // 8 * 8, H * (2 * dk + dv)
+    up = torch.zeros(H * dk, rp)
+    up[:, :rank] = draw(H * dk, rank, seed=50, scale=2 * rank ** -0.5)
+    bias = draw(H * dk, seed=51)
+    for lens in ([1, 1], [3, 1], [4, 4]):
+        x = draw(sum(lens), wq + 3 + rp, seed=52)                 # values past the rank are not read as inputs
+        z = x[:, wq + 3:wq + 3 + rank].double() @ up[:, :rank].double().T
+        start = torch.randn(2, H * dk * dv, generator=torch.Generator().manual_seed(53)).cuda()
+        rg, offs = Bk.Ragged(lens), [0, H * dk, 2 * H * dk]
+        sa, sb = start.clone(), start.clone()
+        a = Bk.gated_linear(dev(x, dtype), offs, z.float().cuda(), dev(bias, dtype), m["tau"], 0.5, sa, H, dk, dv, rg)
+        b = Bk.gated_linear(dev(x, dtype), offs, None, dev(bias, dtype), m["tau"], 0.5, sb, H, dk, dv, rg, w_up=dev(up, dtype), low_off=wq + 3, rank=rank)
+        close(b, a.cpu(), "float32", tol32=1e-5)
+        close(sb, sa.cpu(), "float32", tol32=1e-5)
