@@ -695,7 +695,11 @@ typedef struct {
   float* workspace;
   int32_t plain;
   int32_t shared_tail;       /* > 0: the last shared_tail values of a key are its value's (see pegainfer_qk_prep); one map, vdim == dim */
+  int32_t tile_rows;         /* 32 or 64: the tiles hold ntok * nqh <= tile_rows rows and run on the kernel for prompts (bf16 cache, one map,
+                                unsplit, pegainfer_paged_attention_rows_ok); otherwise <= 16 */
 } pegainfer_attn_options;
+int32_t pegainfer_paged_attention_rows_ok(int32_t dim, int32_t vdim, int32_t shared_tail, int64_t page_stride, int64_t v_cache_off,
+                                          int32_t page_size);
 pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cache, int64_t page_stride, int64_t k_cache_off,
                                                  int64_t v_cache_off, int32_t page_size, const int32_t* positions,
                                                  const int32_t* row_entry, const int32_t* page_indptr, const int32_t* page_ids,

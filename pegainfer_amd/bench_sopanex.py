@@ -4,6 +4,7 @@ memory - and softmax-routed experts with a shared one) and Ramalix (attention wi
 same router with a gated shared expert).  Random weights, bf16, one GPU.
 `python bench.py --model sopanex [--sx-size mid]` prints one JSON line; the default bench workload is untouched."""
 import json
+import sys
 
 from .bench_ramalix import SIZES, measure, ramalix_config
 
@@ -48,6 +49,7 @@ def run(args):
             if args.sx_only in ("all", side):
                 res[name][side if side == "sopanex" else side + "_equal_size"] = measure(cls, cfg, s, args.ctx, args.ctx, batches,
                                                                                        max(2, args.warmup), phase)
+                print("%s, %s: done" % (name, side), file=sys.stderr, flush=True)
     print(json.dumps({"metric": "sopanex_layer_throughput_beside_feruzen_and_ramalix", "unit": "tokens/s", "dtype": "bf16",
                       "data": "synthetic", "n_gpus": 1, "prompt_len": args.ctx, "decode_ctx": args.ctx, "results": res}))
     return 0

@@ -12,6 +12,8 @@
 //                              (AttnForm): keys restricted to the query's own run of `block` positions, a per-head sink
 //                              logit in the denominator, two softmax maps over the same values combined as
 //                              map 1 - lambda * map 2, an RMS norm of the head's output
+//   paged_attention_mfma_kernel  the same tiles on the matrix cores, for a bf16 cache
+//   paged_attention_rows_kernel  prompts over a bf16 cache: 32 or 64 rows per workgroup, the next tile's values on their way
 // Keys are always visited in tiles of 64 from position 0, whatever the step's shape, so a row's arithmetic does not depend on
 // how its prompt was cut or on what else runs in the step.
 #include <algorithm>
@@ -682,6 +684,244 @@ static size_t mfma_attention_lds(int maps, int dim, int ncb) {
   return std::max(tiles, fold);
 }
 
+// Prompts: the same attention with 16 RG rows per workgroup (32 or 64), for a bf16 cache, one map, sizes in multiples of 8.
+// Two waves per 16 rows, each on 32 of a tile's 64 keys, two softmax streams per row folded once at the end.  The next tile is on its way
+// while one is multiplied: its values are requested into registers a whole tile ahead (its page numbers two tiles ahead, through LDS)
+// and land in the other half of a double buffer, so a tile costs one barrier.  Products on v_mfma_f32_16x16x32_bf16: S^T = K Q^T leaves
+// lane l with the scores of row l % 16, and O^T = V^T P^T takes them as they are - which of its 32 keys sits in which place of the product
+// is free, so a lane's two runs of four keys are its eight places - and leaves the outputs of row l % 16 in the same lane: the running
+// maximum's factors need no exchange.  Values lie transposed in LDS as pairs of keys (dword: column, key pair), the pair number XORed with
+// bits of the column: writes along a row and reads along 16 columns both spread over the banks.
+template <int P, int RG>
+__global__ __launch_bounds__(RG * 128) void paged_attention_rows_kernel(
+    const float* __restrict__ q, const uint16_t* __restrict__ cache, int64_t page_stride, int64_t k_cache_off, int64_t v_cache_off,
+    int page_size, const int32_t* __restrict__ positions, const int32_t* __restrict__ row_entry,
+    const int32_t* __restrict__ page_indptr, const int32_t* __restrict__ page_ids, int H, int G, int dim, int vdim, float scale,
+    float factor, const int32_t* __restrict__ tile_row0, const int32_t* __restrict__ tile_ntok,
+    const int32_t* __restrict__ tile_qh0, const int32_t* __restrict__ tile_nqh, uint16_t* __restrict__ out, int64_t out_stride,
+    AttnForm form) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char smraw[];
+  constexpr int N = RG * 128, NCB = P / 16, CH = P / 8, KS = P + 8, KU = 64 * CH / N, VU = (32 * CH + N - 1) / N;
+  constexpr float kLog2e = 1.44269504088896341f;
+  uint16_t* s_k = reinterpret_cast<uint16_t*>(smraw);                 // [2][64][KS]
+  uint32_t* s_v = reinterpret_cast<uint32_t*>(s_k + 2 * kAttKeys * KS);   // [2][P][32]
+  __shared__ int s_pg[2][kAttKeys];
+  const int tile = gridDim.x - 1 - blockIdx.x, g = blockIdx.y;        // the longest rows of keys first
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
+  const int rg = wave % RG, kh = wave / RG;
+  const int row0 = tile_row0[tile], ntok = tile_ntok[tile], qh0 = tile_qh0[tile], nqh = tile_nqh[tile];
+  const int nrows = ntok * nqh, per_group = H / G;
+  const int32_t* pages = page_ids + page_indptr[row_entry[row0]];
+  const int kmax = positions[row0 + ntok - 1] + 1;
+  const int lo0 = attn_row_lo(form, positions[row0]);                 // rows of a tile are in position order: the lowest run start
+  auto next_tile = [&](int k) {                                       // the next tile that any row sees
+    k += kAttKeys;
+    return k >= form.keep_first && k + kAttKeys <= lo0 ? (lo0 / kAttKeys) * kAttKeys : k;
+  };
+  const int kfirst = form.keep_first > 0 ? 0 : (lo0 / kAttKeys) * kAttKeys;
+  const int kw = form.k_keep;
+  // this wave's rows
+  const int lr = rg * 16 + l15;
+  const bool mine = lr < nrows;
+  const int rpos = mine ? positions[row0 + lr / nqh] : -1, rlo = mine ? attn_row_lo(form, rpos) : 0;
+  const int rqh = g * per_group + qh0 + (mine ? lr % nqh : 0);
+  const float rsl = form.dist_slope ? form.dist_slope[rqh] : 0.f;
+  const int last = rg * 16 < nrows ? positions[row0 + min(rg * 16 + 15, nrows - 1) / nqh] : -1;    // uniform: no later key concerns the wave
+  bf16x8_t qf[P / 32];
+  {
+    const float* qr = q + ((int64_t)(row0 + (mine ? lr / nqh : 0)) * H + rqh) * dim;
+#pragma unroll
+    for (int st = 0; st < P / 32; ++st) {
+      const int c = st * 32 + lg * 8;
+      float t[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (mine && c < dim) Vec8<float>::load(qr + c, t);
+      qf[st] = __builtin_bit_cast(bf16x8_t, u32x4{pack_bf2(t[0], t[1]), pack_bf2(t[2], t[3]), pack_bf2(t[4], t[5]), pack_bf2(t[6], t[7])});
+    }
+  }
+  for (int i = tid; i < 2 * kAttKeys * KS / 8; i += N) reinterpret_cast<u32x4*>(s_k)[i] = u32x4{0u, 0u, 0u, 0u};   // columns past dim stay zero
+  u32x4 rk[KU], rv[VU][2];
+  auto page_of = [&](int k0) { return k0 + tid < kmax ? pages[(k0 + tid) / page_size] : 0; };      // threads 0 .. 63
+  auto request = [&](int k0, int b) {      // the tile's values into registers; keys past the context's end as zeros
+    const u32x4 zero = {0u, 0u, 0u, 0u};
+#pragma unroll
+    for (int i = 0; i < KU; ++i) {
+      const int c = (tid % CH) * 8, j = tid / CH + (N / CH) * i, p = k0 + j;
+      rk[i] = zero;
+      if (p < kmax && c < dim) {
+        const int64_t slot = (int64_t)(p % page_size) * G + g;
+        const uint16_t* pg = cache + (int64_t)s_pg[b][j] * page_stride;
+        rk[i] = *reinterpret_cast<const u32x4*>(c < kw ? pg + k_cache_off + slot * kw + c : pg + v_cache_off + slot * vdim + c);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < VU; ++i) {
+      const int unit = tid + N * i, c = (unit % CH) * 8, jp = unit / CH;
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        const int j = 2 * jp + t, p = k0 + j;
+        rv[i][t] = zero;
+        if (jp < 32 && p < kmax && c < vdim)
+          rv[i][t] = *reinterpret_cast<const u32x4*>(cache + (int64_t)s_pg[b][j] * page_stride + v_cache_off + ((int64_t)(p % page_size) * G + g) * vdim + c);
+      }
+    }
+  };
+  auto v_at = [](int col, int jp) { return col * 32 + (jp ^ (((col ^ (col >> 3)) & 7) << 2)); };
+  auto land = [&](int b) {
+    uint16_t* kb = s_k + b * kAttKeys * KS;
+    uint32_t* vb = s_v + b * P * 32;
+#pragma unroll
+    for (int i = 0; i < KU; ++i) {
+      const int c = (tid % CH) * 8, j = tid / CH + (N / CH) * i;
+      if (c < dim) *reinterpret_cast<u32x4*>(kb + j * KS + c) = rk[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VU; ++i) {
+      const int unit = tid + N * i, c = (unit % CH) * 8, jp = unit / CH;
+      if (jp < 32) {
+        const uint32_t a[4] = {rv[i][0].x, rv[i][0].y, rv[i][0].z, rv[i][0].w}, d[4] = {rv[i][1].x, rv[i][1].y, rv[i][1].z, rv[i][1].w};
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          vb[v_at(c + 2 * u, jp)] = (a[u] & 0xFFFFu) | (d[u] << 16);
+          vb[v_at(c + 2 * u + 1, jp)] = (a[u] >> 16) | (d[u] & 0xFFFF0000u);
+        }
+      }
+    }
+  };
+  float mrun = -INFINITY, lrun = 0.f;
+  f32x4 o[NCB];
+#pragma unroll
+  for (int cb = 0; cb < NCB; ++cb) o[cb] = f32x4{0.f, 0.f, 0.f, 0.f};
+  auto multiply = [&](int k0, int b) {
+    const int kb = k0 + 32 * kh;
+    if (kb > last || kb >= kmax) return;             // uniform over the wave
+    const uint16_t* ka = s_k + b * kAttKeys * KS + (32 * kh + l15) * KS + lg * 8;
+    f32x4 sc[2] = {};
+#pragma unroll
+    for (int st = 0; st < P / 32; ++st)
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+        sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4*>(ka + 16 * t * KS + st * 32)),
+                                                         qf[st], sc[t], 0, 0, 0);
+    float tmax = -INFINITY;
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int kp = kb + 16 * t + 4 * lg + r;
+        sc[t][r] = kp <= rpos && (kp >= rlo || kp < form.keep_first) ? attn_score(form, sc[t][r], scale, rpos, kp, rqh, H, rsl) : -INFINITY;
+        tmax = fmaxf(tmax, sc[t][r]);
+      }
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, kWave));
+    const float mnew = fmaxf(mrun, tmax), mref = mnew == -INFINITY ? 0.f : mnew;
+    const float corr = __builtin_amdgcn_exp2f((mrun - mref) * kLog2e);           // a row that has met no key yet: 0, and nothing to scale
+    uint32_t pb[4];
+    float psum = 0.f;
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; r += 2) {
+        const uint32_t w = pack_bf2(__builtin_amdgcn_exp2f((sc[t][r] - mref) * kLog2e), __builtin_amdgcn_exp2f((sc[t][r + 1] - mref) * kLog2e));
+        pb[2 * t + (r >> 1)] = w;
+        psum += bf_lo(w) + bf_hi(w);                 // the sum of the weights as they are multiplied
+      }
+    psum += __shfl_xor(psum, 16, kWave);
+    psum += __shfl_xor(psum, 32, kWave);
+    lrun = lrun * corr + psum;
+    if (__any(mnew != mrun)) {
+#pragma unroll
+      for (int cb = 0; cb < NCB; ++cb) { o[cb].x *= corr; o[cb].y *= corr; o[cb].z *= corr; o[cb].w *= corr; }
+    }
+    mrun = mnew;
+    const bf16x8_t pf = __builtin_bit_cast(bf16x8_t, u32x4{pb[0], pb[1], pb[2], pb[3]});
+    const uint32_t* vb = s_v + b * P * 32;
+#pragma unroll
+    for (int cb = 0; cb < NCB; ++cb) {
+      const int col = 16 * cb + l15, jp = 16 * kh + 2 * lg;
+      const u32x2 v0 = *reinterpret_cast<const u32x2*>(vb + v_at(col, jp)), v1 = *reinterpret_cast<const u32x2*>(vb + v_at(col, jp + 8));
+      o[cb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, u32x4{v0.x, v0.y, v1.x, v1.y}), pf, o[cb], 0, 0, 0);
+    }
+  };
+  int k0 = kfirst, k1 = next_tile(k0);
+  if (tid < kAttKeys) {
+    s_pg[0][tid] = page_of(k0);
+    s_pg[1][tid] = page_of(k1);
+  }
+  __syncthreads();
+  request(k0, 0);
+  land(0);
+  __syncthreads();
+  request(k1, 1);
+  for (int b = 0;; b ^= 1) {
+    const int k2 = next_tile(k1);
+    const int pg = tid < kAttKeys ? page_of(k2) : 0;
+    multiply(k0, b);
+    if (k1 >= kmax) break;                           // uniform over the workgroup
+    land(b ^ 1);
+    if (tid < kAttKeys) s_pg[b][tid] = pg;
+    __syncthreads();
+    k0 = k1;
+    k1 = k2;
+    request(k1, b);                                  // k1 may lie past the end: zeros, no access
+  }
+  __syncthreads();                                   // the tiles' LDS is free
+  f32x4* f_o = reinterpret_cast<f32x4*>(smraw);      // [RG][NCB][64]
+  float* f_ml = reinterpret_cast<float*>(f_o + RG * NCB * 64);        // [RG][64][2]
+  if (kh == 1) {
+#pragma unroll
+    for (int cb = 0; cb < NCB; ++cb) f_o[(rg * NCB + cb) * 64 + lane] = o[cb];
+    f_ml[(rg * 64 + lane) * 2] = mrun;
+    f_ml[(rg * 64 + lane) * 2 + 1] = lrun;
+  }
+  __syncthreads();
+  if (kh == 1 || rg * 16 >= nrows) return;
+  const float m1 = f_ml[(rg * 64 + lane) * 2], l1 = f_ml[(rg * 64 + lane) * 2 + 1];
+  float mall = fmaxf(mrun, m1), sink = -INFINITY;
+  if (form.sink && mine) {
+    sink = bf2f(static_cast<const uint16_t*>(form.sink)[rqh]);
+    mall = fmaxf(mall, sink);
+  }
+  const float w0 = mrun == -INFINITY ? 0.f : expf(mrun - mall), w1 = m1 == -INFINITY ? 0.f : expf(m1 - mall);
+  const float l = lrun * w0 + l1 * w1 + (sink == -INFINITY ? 0.f : expf(sink - mall));
+  const float i0 = w0 / l, i1 = w1 / l;
+  float ss = 0.f;
+#pragma unroll
+  for (int cb = 0; cb < NCB; ++cb) {
+    const f32x4 t = f_o[(rg * NCB + cb) * 64 + lane];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      o[cb][r] = o[cb][r] * i0 + t[r] * i1;
+      if (16 * cb + 4 * lg + r < vdim) ss = fmaf(o[cb][r], o[cb][r], ss);
+    }
+  }
+  float post = factor;
+  if (form.head_norm) {
+    ss += __shfl_xor(ss, 16, kWave);
+    ss += __shfl_xor(ss, 32, kWave);
+    post = factor / sqrtf(ss / (float)vdim + form.norm_eps);
+  }
+  if (!mine) return;
+  const int row = row0 + lr / nqh;
+  const uint16_t* gate = static_cast<const uint16_t*>(form.gate) + (int64_t)row * form.gate_stride;
+  if (form.gate_kind == 2) post *= sigmoid_f(bf2f(gate[rqh]));
+  uint16_t* dst = out + (int64_t)row * out_stride + (int64_t)rqh * vdim;
+#pragma unroll
+  for (int cb = 0; cb < NCB; ++cb) {
+    const int c = 16 * cb + 4 * lg;
+    if (c >= vdim) continue;                         // vdim is a multiple of 8
+    float v[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      v[r] = o[cb][r] * post;
+      if (form.gate_kind == 1) v[r] *= sigmoid_f(bf2f(gate[(int64_t)rqh * vdim + c + r]));
+    }
+    st4(dst + c, v);
+  }
+}
+static size_t rows_attention_lds(int p, int rg) {
+  return std::max((size_t)2 * kAttKeys * (p + 8) * 2 + (size_t)2 * p * 32 * 4, (size_t)rg * 64 * (p / 16 * 16 + 8));
+}
+
 // The states that the splits of a tile have left, brought to their common maximum and summed in split order, then finished like
 // an unsplit row.
 template <typename A, int MAPS>
@@ -902,6 +1142,32 @@ pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cac
   form.gate_kind = gate_kind;
   form.k_keep = qd - opt->shared_tail;
   bool ok = true;
+  if (opt->tile_rows > kAttRows) {    // tables cut for the prompts' kernel
+    if ((opt->tile_rows != 32 && opt->tile_rows != 64) || maps != 1 || n_split != 1 || plain || dtype != kDtBf16 || out_stride % 4 ||
+        !host_aligned16(out) || !host_aligned16(q) || !host_aligned16(cache) || k_cache_off % 8 ||
+        !pegainfer_paged_attention_rows_ok(dim, vdim, opt->shared_tail, page_stride, v_cache_off, page_size))
+      return PK_BAD;
+    auto launch = [&](auto kern, int p, int rg) {
+      const size_t lds = rows_attention_lds(p, rg);
+      if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) {
+        ok = false;
+        return;
+      }
+      kern<<<dim3(n_tiles, kv_heads), rg * 128, lds, as_stream(stream)>>>(
+          q, static_cast<const uint16_t*>(cache), page_stride, k_cache_off, v_cache_off, page_size, positions, row_entry, page_indptr, page_ids,
+          heads, kv_heads, dim, vdim, scale, factor, tile_row0, tile_ntok, tile_qh0, tile_nqh, static_cast<uint16_t*>(out), out_stride, form);
+    };
+    auto by_size = [&](auto rg) {
+      constexpr int RG = decltype(rg)::value;
+      const int most = std::max(dim, vdim);
+      if (most <= 64) launch(paged_attention_rows_kernel<64, RG>, 64, RG);
+      else if (most <= 128) launch(paged_attention_rows_kernel<128, RG>, 128, RG);
+      else launch(paged_attention_rows_kernel<256, RG>, 256, RG);
+    };
+    if (opt->tile_rows == 64) by_size(std::integral_constant<int, 4>());
+    else by_size(std::integral_constant<int, 2>());
+    return ok ? (pegainfer_status_t)hipGetLastError() : PK_BAD;
+  }
   if (dtype == kDtBf16 && !plain) {   // bf16 cache: the matrix-core kernel; same tiles, same splits, same merge
     const int ncb = vdim <= 32 ? 2 : vdim <= 64 ? 4 : vdim <= 128 ? 8 : 16;
     const size_t lds = mfma_attention_lds(maps, dim, ncb);
@@ -961,6 +1227,12 @@ pegainfer_status_t pegainfer_paged_attention_opt(const float* q, const void* cac
     }
   });
   return known && ok ? (pegainfer_status_t)hipGetLastError() : PK_BAD;
+}
+
+int32_t pegainfer_paged_attention_rows_ok(int32_t dim, int32_t vdim, int32_t shared_tail, int64_t page_stride, int64_t v_cache_off,
+                                          int32_t page_size) {
+  return dim > 0 && dim <= 256 && dim % 8 == 0 && vdim > 0 && vdim <= 256 && vdim % 8 == 0 && shared_tail % 8 == 0 && page_stride % 8 == 0 &&
+         v_cache_off % 8 == 0 && page_size > 0;
 }
 
 int64_t pegainfer_paged_attention_workspace(int32_t n_tiles, int32_t kv_heads, int32_t vdim, int32_t maps, int32_t n_split) {

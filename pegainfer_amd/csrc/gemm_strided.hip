@@ -343,7 +343,9 @@ static void rows_form_launch(const pegainfer_gemm_desc& d, hipStream_t s) {
                             hipFuncSetAttribute(reinterpret_cast<const void*>(kern8), hipFuncAttributeMaxDynamicSharedMemorySize, 152 * 1024),
                             true);
   (void)once;
-  const int row_tiles = d.tile_group ? d.max_tiles : ceil_div(d.rows, R), groups = d.tile_group ? 1 : d.groups;
+  // the tiles that a table's bound allows for and that are empty come last: an even grid width would send the others' workgroups, in
+  // their round robin over the XCDs, to some of the eight only
+  const int row_tiles = d.tile_group ? d.max_tiles | 1 : ceil_div(d.rows, R), groups = d.tile_group ? 1 : d.groups;
   // 32 outputs per workgroup unless that leaves most compute units without one
   const bool fine = (long)row_tiles * groups * ceil_div(d.m, 32) < device_cus();
   dim3 grid(row_tiles, ceil_div(d.m, fine ? 8 : 32), groups);

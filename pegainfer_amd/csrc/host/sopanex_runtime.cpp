@@ -130,9 +130,10 @@ class Model : public StepModel {
       return set_error("config: unsupported linear attention sizes in layer " + li);
     c->mix_right = pad8(a.heads * a.dim);
     c->mix_cols = pad8(c->mix_right + m.heads * m.vdim);
-    c->tiles = group_tiles(a.heads / a.kv);
     c->k_off = add_cache((int64_t)a.kv * a.rot_dims);
     c->v_off = add_cache((int64_t)a.kv * a.dim);
+    const bool wide = dtype == PEGAINFER_DTYPE_BF16 && pegainfer_paged_attention_rows_ok(a.dim, a.dim, a.tail(), 0, 0, kPageSize);
+    c->tiles = group_tiles(a.heads / a.kv, wide ? a.kv : 0);
     m.st_off = state_layout.reserve("l" + li + ".memory", (int64_t)m.heads * m.dim * m.vdim);
     if (pegainfer_gated_linear_chunked_ok(m.dim, m.vdim)) scan_max = kScanMax;
     if (mlp && mlp->kind == Json::Obj) {
@@ -351,7 +352,8 @@ class Model : public StepModel {
     pegainfer_attn_options o{};
     o.sink = w.sink;
     o.gate = at(proj, (size_t)a.o_g); o.gate_stride = c.proj_rows; o.gate_kind = PEGAINFER_GATE_PER_HEAD;
-    o.n_split = wgs >= kFewTiles ? 1 : std::max(1, std::min(kMaxSplits, kSplitGroups / wgs));
+    o.tile_rows = t.rows;
+    o.n_split = wgs >= kFewTiles || t.rows > kGroupRows ? 1 : std::max(1, std::min(kMaxSplits, kSplitGroups / wgs));
     o.workspace = part;
     o.plain = plain_kernels ? 1 : 0;
     o.shared_tail = a.tail();
@@ -424,7 +426,7 @@ class Model : public StepModel {
     d.y_row_index = pos_pair;
     PSTEP_K(pegainfer_gemm_strided(&d, S()));
     if (f.shared_ff) {
-      if (tuned) {
+      if (dtype == PEGAINFER_DTYPE_BF16 && !plain_kernels && T > 1) {   // a tuned route and the activation; one row: both in one launch
         if (linear(w.up_s, h, act_s, f.shared_ff, T, D)) return -1;
         PSTEP_K(pegainfer_act_rows(act_s, f.shared_ff, act_s, f.shared_ff, f.shared_ff, T, PEGAINFER_ACT_GELU_ERF, dtype, S()));
       } else if (linear_strided(w.up_s, h, dtype, D, act_s, dtype, f.shared_ff, T, D, PEGAINFER_EPI_GELU_ERF)) {

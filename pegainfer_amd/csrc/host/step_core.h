@@ -76,14 +76,17 @@ inline bool ends_with(const std::string& s, const char* suf) {
 
 constexpr int kPageSize = 16;       // tokens per cache page, as in the other runtimes
 constexpr int kGroupRows = 16;      // (token, query head) rows of one workgroup of the paged attention
+constexpr int kWideGroups = 256;    // a step whose 64- (32-) row tiles give so many workgroups takes those
 constexpr int kFlatRows = 64;       // flattened (token, head) rows of one workgroup of the latent attention
 
 // A table of row tiles on the device.  Group tiles: runs of tokens of one entry times a run of the query heads of one key/value
-// head, at most kGroupRows rows (rows of four arrays: first token row, tokens, first query head, query heads).  Flat tiles: runs of
+// head, at most kGroupRows rows - or 32 or 64 in prompts, where a model asks for it - (rows of four arrays: first token row, tokens, first
+// query head, query heads).  Flat tiles: runs of
 // <= kFlatRows flattened rows token * heads + head of one entry (two arrays: first row, rows).
 struct TileTable {
   const int32_t* at = nullptr;
   int count = 0;
+  int rows = kGroupRows;        // group tiles: the most rows of a tile
   const int32_t* col(int k) const { return at + (size_t)k * count; }
 };
 // Long entries (more than scan_max rows) cut into chunks, for recurrences with a chunk form.
@@ -316,7 +319,12 @@ class StepModel {
       for (int i = 0; i < W; ++i) mb[o_want + i] = want[i];
     }
     std::vector<std::pair<size_t, int>> group_at, flat_at;    // (offset, tiles)
-    for (int per : group_heads) group_at.push_back(put_group_tiles(&mb, lens, n, per));
+    std::vector<int> group_rows;
+    for (auto& gt : group_sets) {
+      const int rows = gt.wide_kv > 0 && !plain_kernels ? wide_rows(lens, n, (int)T, gt) : kGroupRows;
+      group_rows.push_back(rows);
+      group_at.push_back(put_group_tiles(&mb, lens, n, gt.per, rows));
+    }
     for (int heads : flat_heads) flat_at.push_back(put_flat_tiles(&mb, lens, n, heads));
     size_t o_chunks[4] = {0, 0, 0, 0};
     if (scan_max > 0) put_chunks(&mb, ids, lens, n, &c.chunks, o_chunks);
@@ -330,8 +338,8 @@ class StepModel {
     c.tokens = reinterpret_cast<const uint32_t*>(md + o_tok);
     c.prev = md + o_prev; c.pos = md + o_pos; c.entry = md + o_ent; c.row0 = md + o_row0; c.slot = md + o_slot; c.page_indptr = md + o_ind;
     c.want = md + o_want; c.pages = md + o_pages;
-    for (auto& g : group_at) c.group_tiles.push_back(TileTable{md + g.first, g.second});
-    for (auto& f : flat_at) c.flat_tiles.push_back(TileTable{md + f.first, f.second});
+    for (size_t k = 0; k < group_at.size(); ++k) c.group_tiles.push_back(TileTable{md + group_at[k].first, group_at[k].second, group_rows[k]});
+    for (auto& f : flat_at) c.flat_tiles.push_back(TileTable{md + f.first, f.second, kFlatRows});
     if (c.chunks.n_long > 0) {
       c.chunks.row0 = md + o_chunks[0]; c.chunks.rows = md + o_chunks[1];
       c.chunks.long_chunk0 = md + o_chunks[2]; c.chunks.long_slot = md + o_chunks[3];
@@ -420,7 +428,11 @@ class StepModel {
   float* state = nullptr;
   std::vector<void*> step_owned, want_owned, owned;
   float* logits32 = nullptr;         // [wanted, V]: run_step leaves them here
-  std::vector<int> group_heads, flat_heads;   // distinct parameters of the tile tables a model's launches read
+  // distinct parameters of the tile tables a model's launches read.  wide_kv: key/value heads of a layer whose prompts may take wider
+  // group tiles (0: never)
+  struct GroupSet { int per, wide_kv; bool operator==(const GroupSet& o) const { return per == o.per && wide_kv == o.wide_kv; } };
+  std::vector<GroupSet> group_sets;
+  std::vector<int> flat_heads;
   int scan_max = 0;                  // > 0: entries with more rows go into the chunk table
   bool graphs_on = true;
   std::map<std::string, std::vector<uint16_t>> staged;
@@ -442,13 +454,14 @@ class StepModel {
     page_stride += kPageSize * per_token;
     return off;
   }
-  static int index_of(std::vector<int>* v, int x) {
+  template <typename X>
+  static int index_of(std::vector<X>* v, X x) {
     const auto it = std::find(v->begin(), v->end(), x);
     if (it != v->end()) return (int)(it - v->begin());
     v->push_back(x);
     return (int)v->size() - 1;
   }
-  int group_tiles(int heads_per_kv) { return index_of(&group_heads, heads_per_kv); }
+  int group_tiles(int heads_per_kv, int wide_kv = 0) { return index_of(&group_sets, GroupSet{heads_per_kv, wide_kv}); }
   int flat_tiles(int heads) { return index_of(&flat_heads, heads); }
 
   template <typename T>
@@ -672,14 +685,24 @@ class StepModel {
     for (auto& c : cols) mb->insert(mb->end(), c.begin(), c.end());
     return {at, (int)cols[0].size()};
   }
-  static std::pair<size_t, int> put_group_tiles(std::vector<int32_t>* mb, const int32_t* lens, int n, int per) {
+  // the widest tiles that still fill the chip and are at least half full
+  static int wide_rows(const int32_t* lens, int n, int T, const GroupSet& g) {
+    for (int rows : {64, 32}) {
+      const int tpt = std::max(1, rows / g.per), cuts = (g.per + rows - 1) / rows;
+      long tiles = 0;
+      for (int i = 0; i < n; ++i) tiles += (long)((lens[i] + tpt - 1) / tpt) * cuts;
+      if (tiles * g.wide_kv >= kWideGroups && (long)T * g.per * 2 >= tiles * rows) return rows;
+    }
+    return kGroupRows;
+  }
+  static std::pair<size_t, int> put_group_tiles(std::vector<int32_t>* mb, const int32_t* lens, int n, int per, int rows) {
     std::vector<std::vector<int32_t>> c(4);
     auto add = [&](int row0, int ntok, int qh0, int nqh) { c[0].push_back(row0); c[1].push_back(ntok); c[2].push_back(qh0); c[3].push_back(nqh); };
     int r0 = 0;
     for (int i = 0; i < n; r0 += lens[i++]) {
-      const int tpt = std::max(1, kGroupRows / per);
+      const int tpt = std::max(1, rows / per);
       for (int t0 = 0; t0 < lens[i]; t0 += tpt)
-        for (int q0 = 0; q0 < per; q0 += kGroupRows) add(r0 + t0, std::min(tpt, lens[i] - t0), q0, std::min(kGroupRows, per - q0));
+        for (int q0 = 0; q0 < per; q0 += rows) add(r0 + t0, std::min(tpt, lens[i] - t0), q0, std::min(rows, per - q0));
     }
     return put_columns(mb, c);
   }

@@ -155,7 +155,8 @@ class Model : public StepModel {
       c->proj_rows = pad8(c->o_v + c->kv * c->vdim);
       c->k_off = add_cache((int64_t)c->kv * c->dim);
       c->v_off = add_cache((int64_t)c->kv * c->vdim);
-      c->tiles = group_tiles(c->heads / c->kv);
+      const bool wide = dtype == PEGAINFER_DTYPE_BF16 && pegainfer_paged_attention_rows_ok(c->dim, c->vdim, 0, 0, 0, kPageSize);
+      c->tiles = group_tiles(c->heads / c->kv, wide ? c->kv : 0);
     } else if (ty->str == "lightning") {
       c->type = kLightning;
       const Json* g = mx->get("decay");
@@ -382,7 +383,8 @@ class Model : public StepModel {
     pegainfer_attn_options o{};
     o.window = c.window;
     o.dist_slope = w.slopes;
-    o.n_split = wgs >= kFewTiles ? 1 : std::max(1, std::min(kMaxSplits, kSplitGroups / wgs));
+    o.tile_rows = t.rows;
+    o.n_split = wgs >= kFewTiles || t.rows > kGroupRows ? 1 : std::max(1, std::min(kMaxSplits, kSplitGroups / wgs));
     o.workspace = part;
     o.plain = plain_kernels ? 1 : 0;
     PSTEP_K(pegainfer_paged_attention_opt(qf, cache, page_stride, c.k_off, c.v_off, kPageSize, s.pos, s.entry, s.page_indptr, s.pages, c.heads,

@@ -282,19 +282,15 @@ def head_rms_gate(o_f32, w, gate, gate_kind, factor, eps, heads, vdim, out=None)
     return out
 
 
-def attention_tiles(lens, per_group, device="cuda"):
+def attention_tiles(lens, per_group, device="cuda", rows=16):
     """row tiles of pegainfer_paged_attention for entries of `lens` rows: runs of token rows times runs of the per_group query
-    heads of a key/value head, at most 16 rows each"""
+    heads of a key/value head, at most `rows` rows each"""
     row0, ntok, qh0, nqh, at = [], [], [], [], 0
     for n in lens:
-        if per_group <= 16:
-            tpt = 16 // per_group
-            for t0 in range(0, n, tpt):
-                row0.append(at + t0); ntok.append(min(tpt, n - t0)); qh0.append(0); nqh.append(per_group)  # noqa: E702
-        else:
-            for t0 in range(n):
-                for q0 in range(0, per_group, 16):
-                    row0.append(at + t0); ntok.append(1); qh0.append(q0); nqh.append(min(16, per_group - q0))  # noqa: E702
+        tpt = max(1, rows // per_group)
+        for t0 in range(0, n, tpt):
+            for q0 in range(0, per_group, rows):
+                row0.append(at + t0); ntok.append(min(tpt, n - t0)); qh0.append(q0); nqh.append(min(rows, per_group - q0))  # noqa: E702
         at += n
     return tuple(torch.tensor(v, dtype=torch.int32, device=device) for v in (row0, ntok, qh0, nqh))
 
@@ -510,7 +506,7 @@ def _struct(name, fields):
 
 AttnOptions = _struct("AttnOptions", [("i", "maps"), ("f", "lambda_"), ("i", "block"), ("p", "sink"), ("i", "head_norm"), ("f", "norm_eps softcap"),
                                       ("i", "window keep_first"), ("p", "dist_bias"), ("i", "n_dist"), ("p", "dist_slope gate"),
-                                      ("l", "gate_stride"), ("i", "gate_kind n_split"), ("p", "workspace"), ("i", "plain shared_tail")])
+                                      ("l", "gate_stride"), ("i", "gate_kind n_split"), ("p", "workspace"), ("i", "plain shared_tail tile_rows")])
 LatentPrepDesc = _struct("LatentPrepDesc", [("p", "dkv"), ("l", "dkv_stride"), ("p", "c_norm_w ql"), ("l", "ql_stride"), ("p", "ql_norm_w ql_out"),
                                             ("i", "q_rank"), ("p", "q"), ("l", "q_stride"), ("p", "qc"), ("f", "eps"), ("p", "inv_freq"),
                                             ("i", "rot_dims rot_layout"), ("p", "positions token_req page_indptr page_ids cache"),
@@ -526,19 +522,19 @@ DecayAttentionDesc = _struct("DecayAttentionDesc", [("p", "proj"), ("l", "proj_s
 
 
 def paged_attention_opt(q, cache, page_stride, k_off, v_off, page_size, rg, page_indptr, page_ids, kv_heads, vdim, scale, window=0,
-                        dist_slope=None, softcap=0.0, n_split=1, plain=False, sink=None, gate=None, factor=1.0, shared_tail=0):
+                        dist_slope=None, softcap=0.0, n_split=1, plain=False, sink=None, gate=None, factor=1.0, shared_tail=0, tile_rows=16):
     """q fp32 [rows, heads, dim]; dist_slope fp32 [heads]: slope * distance is taken off the scores; gate: a [rows, heads] view in the
     cache's type, one output gate logit per head; shared_tail: values of a key that are read from its value"""
     T, H, dim = q.shape
     out = torch.empty((T, H * vdim), dtype=cache.dtype, device=q.device)
-    t = attention_tiles(rg.lens, H // kv_heads, q.device)
+    t = attention_tiles(rg.lens, H // kv_heads, q.device, tile_rows)
     ws = None
     if n_split > 1:
         ws = torch.empty(ffi.lib().pegainfer_paged_attention_workspace(t[0].numel(), kv_heads, vdim, 1, n_split), dtype=torch.float32,
                          device=q.device)
     o = AttnOptions(window=int(window), dist_slope=_p(dist_slope), softcap=float(softcap), n_split=int(n_split), workspace=_p(ws),
                     plain=int(bool(plain)), sink=_p(sink), gate=_p(gate), gate_stride=0 if gate is None else gate.stride(0),
-                    gate_kind=0 if gate is None else 2, shared_tail=int(shared_tail))
+                    gate_kind=0 if gate is None else 2, shared_tail=int(shared_tail), tile_rows=tile_rows if tile_rows > 16 else 0)
     _chk(ffi.lib().pegainfer_paged_attention_opt(_p(q), _p(cache), page_stride, k_off, v_off, page_size, _p(rg.positions), _p(rg.row_entry),
                                                  _p(page_indptr), _p(page_ids), H, kv_heads, dim, vdim, float(scale), float(factor), _p(t[0]),
                                                  _p(t[1]), _p(t[2]), _p(t[3]), t[0].numel(), _p(out), out.stride(0), ctypes.addressof(o), _dt(cache),

@@ -205,6 +205,26 @@ def test_a_long_prompt_matches_its_portions_and_the_restatement():
         eng.close()
 
 
+def test_prompts_long_enough_for_wide_attention_tiles():
+    """1500 tokens and eight key/value heads: 64-row tiles, beside short portions of other requests in the same step, against the restatement"""
+    cfg = C.base(64, 70, [C.layer((16, 8, 16, 0.25, C.rot(8, 1000.0, (4.0, 300, 16.0, 1.0))), (2, 16, 16, 16.0, 4), (1.1, 0.8), C.moe(16, 4, 2, 2, 1.3, 24)),
+                          C.layer((8, 8, 24, 0.2, C.rot(24, 500.0)), (1, 16, 24, 4.0, 4))], bigram=(29, 3, 17))
+    w = C.weights_for(cfg, 27, "bfloat16")
+    toks, other = C.tokens_for(cfg, 1500, 12), C.tokens_for(cfg, 40, 13)
+    want = [0, 1, 15, 16, 62, 63, 64, 65, 127, 128, 700, 1023, 1024, 1490, 1499]
+    ref, ref_o = C.oracle_logits(cfg, w, toks)[want], C.oracle_logits(cfg, w, other)
+    for dtype in ("bfloat16", "float32"):
+        eng = C.engine_for(cfg, w, dtype, max_tokens=3200, max_requests=3)
+        a, b = eng.new_request(), eng.new_request()
+        check(eng.step([(a, toks)], want=want), ref, dtype)
+        eng.step([(b, other[:7])], want=[])
+        c = eng.new_request()
+        lg = eng.step([(b, other[7:40]), (c, toks)], want=[32] + [33 + p for p in want])
+        check(lg[:1], ref_o[39:], dtype)
+        check(lg[1:], ref, dtype)
+        eng.close()
+
+
 def test_graph_replays_of_decode_steps_match_eager_steps():
     """single-token steps are replayed from a captured graph: several replays, with prompt steps and synchronisations of other
     requests between them, against the same steps run eagerly (the per-layer tap switches the capture off)"""

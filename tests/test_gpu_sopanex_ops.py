@@ -188,7 +188,8 @@ PAGES = [7, 2, 11, 0, 5, 9, 3, 12, 1, 10, 4, 6, 8, 13, 14, 15, 16, 17, 18, 19, 2
 PORTIONS = [15, 1, 1, 6, 2, 23, 15, 1, 1, 15] + [1] * 70
 
 
-def attend(qkg, H, G, d, dtype, plan, scale, rot=None, sink=None, gate=True, n_split=1, plain=False, factor=1.0, tail=None):
+def attend(qkg, H, G, d, dtype, plan, scale, rot=None, sink=None, gate=True, n_split=1, plain=False, factor=1.0, tail=None,
+           tile_rows=16):
     """rows [q | k | gate logits] -> the heads' outputs of every row; tail: key values read from the values (None: all the rotation leaves)"""
     Bk = B()
     dims = rot["dims"] if rot else 0
@@ -204,7 +205,7 @@ def attend(qkg, H, G, d, dtype, plan, scale, rot=None, sink=None, gate=True, n_s
                        rot_dims=dims, rot_amp=amp, shared_tail=tail)
         outs.append(Bk.paged_attention_opt(q, pc.cache, pc.page_stride, pc.offs[0], pc.offs[1], 16, rg, pc.indptr, pc.pids, G, d, scale,
                                            sink=None if sink is None else dev(sink, dtype), gate=x[:, (H + G) * d:] if gate else None,
-                                           n_split=n_split, plain=plain, factor=factor, shared_tail=tail))
+                                           n_split=n_split, plain=plain, factor=factor, shared_tail=tail, tile_rows=tile_rows))
         at += n
     return torch.cat(outs)
 
@@ -238,18 +239,63 @@ def test_attention_whole_in_portions_and_split(dtype, layer):
         close(attend(x, H, G, d, dtype, [n], m["scale"], plain=True, **kw), ref, dtype, **tol)
 
 
+@pytest.mark.parametrize("tile_rows", [32, 64])
+@pytest.mark.parametrize("heads", [(6, 2, 24, 16, 0.25), (4, 4, 16, 16, 0.3), (5, 1, 32, 8, 0.2), (20, 1, 72, 32, 0.12), (70, 1, 8, 8, 0.4), (4, 2, 136, 64, 0.08),
+                                   (2, 1, 256, 128, 0.06), (3, 1, 64, 0, 0.1), (4, 1, 128, 64, 0.1)], ids=lambda h: "x".join(map(str, h[:3])))
+def test_prompts_on_wide_tiles(heads, tile_rows):
+    """the kernel for prompts (bf16): lengths around its 64-key tiles, portions behind a cached prefix, the 16-row kernel's cache"""
+    H, G, d, dims, scale = heads
+    ro = C.rot(dims, 300.0, (3.0, 60, 6.0, 0.5)) if dims else None
+    sink = draw(H, seed=14, scale=1.5)
+    m = {"heads": H, "kv_heads": G, "dim": d, "scale": scale, "rot": ro}
+    for n, plan in ((1, [1]), (31, [31]), (64, [64]), (65, [65]), (129, [129]), (200, [200]), (200, [63, 2, 66, 69]), (330, [330]), (330, [1, 128, 201])):
+        x = draw(n, (H + G) * d + H, seed=n)
+        ref = attend_ref(x, m, sink)
+        close(attend(x, H, G, d, "bfloat16", plan, scale, rot=ro, sink=sink, tile_rows=tile_rows), ref, "bfloat16", tol16=6e-2)
+    close(attend(x, H, G, d, "bfloat16", plan, scale, rot=ro, sink=sink, tile_rows=tile_rows, tail=0, factor=0.5), ref * 0.5, "bfloat16", tol16=6e-2)
+
+
+@pytest.mark.parametrize("tile_rows", [32, 64])
+@pytest.mark.parametrize("window", [0, 1, 2, 31, 32, 33, 64, 65, 100, 200])
+@pytest.mark.parametrize("hot", [0, 31, 32, 63, 64, 130])
+def test_a_marked_key_on_wide_tiles_up_to_the_windows_edge(tile_rows, window, hot):
+    """every later row reads the one key that stands out while its window (0: none) reaches it; two heads read different values of it"""
+    Bk = B()
+    n, d = 300, 16
+    q, k = torch.zeros(n, 2 * d), torch.zeros(n, d)
+    q[:, 8], q[:, d + 8] = 8.0, 8.0
+    k[hot, 8], k[hot, 3] = 5.0, 1.0
+    x = dev(torch.cat([q, k], 1), "bfloat16")
+    pc = Paged(PAGES, [d, d], "bfloat16")
+    for plan in ([n], [hot + 1, n - hot - 1]):
+        outs, at = [], 0
+        for c in plan:
+            rg = Bk.Ragged([c], starts=[at])
+            qq = Bk.qk_prep(x[at:at + c], [0, 2 * d, 2 * d], 2, 1, d, d, rg, pc.indptr, pc.pids, pc.cache, pc.page_stride, pc.offs[0], pc.offs[1], 16)
+            outs.append(Bk.paged_attention_opt(qq, pc.cache, pc.page_stride, pc.offs[0], pc.offs[1], 16, rg, pc.indptr, pc.pids, 1, d, 1.0,
+                                               window=window, tile_rows=tile_rows))
+            at += c
+        got = torch.cat(outs).double().cpu()
+        i = torch.arange(n)
+        seen = (i >= hot) & ((i - hot < window) if window else (i >= 0))
+        for h in range(2):
+            assert (got[seen][:, h * d + 3] > 0.99).all() and (got[~seen][:, h * d + 3] == 0).all(), (window, hot, h)
+
+
 @BOTH
 @pytest.mark.parametrize("hot", [0, 1, 15, 16, 63, 64, 101, 300])
 def test_one_far_key_stands_out_among_hundreds(dtype, hot):
     """value 3 of every query asks for the one key that has it: later rows read that key as their value, and its unrotated form at that"""
     n, d = 420, 16
-    ro = C.rot(4, 50.0, (4.0, 100, 8.0, 1.0))
+    ro = C.rot(8, 50.0, (4.0, 100, 8.0, 1.0))
     x = torch.zeros(n, 2 * d)
     x[:, 10] = 8.0                                   # asked for in the part the rotation leaves
     x[hot, d + 10] = 5.0
     x[hot, d + 1] = 2.0                              # a value inside the rotated part must come out as projected
-    for plan, split in (([n], 1), ([hot + 1, n - hot - 1], 1), ([400] + [1] * 20, 7)):
-        got = attend(x, 1, 1, d, dtype, plan, 1.0, rot=ro, gate=False, n_split=split).double().cpu()
+    for plan, split, rows in (([n], 1, 16), ([hot + 1, n - hot - 1], 1, 16), ([400] + [1] * 20, 7, 16), ([n], 1, 64), ([hot + 1, n - hot - 1], 1, 32)):
+        if rows > 16 and dtype == "float32":
+            continue
+        got = attend(x, 1, 1, d, dtype, plan, 1.0, rot=ro, gate=False, n_split=split, tile_rows=rows).double().cpu()
         assert (got[hot:, 10] > 4.9).all() and ((got[hot:, 1] - 2.0).abs() < 0.05).all(), hot
         assert (got[:hot].abs() < 1e-6).all()
 
