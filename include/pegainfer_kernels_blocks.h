@@ -322,7 +322,7 @@ pegainfer_status_t pegainfer_terms_rms_add(const float* x_in, const pegainfer_su
                                            const void* gain, float eps, void* n_out, int32_t n_dtype, int32_t d, int32_t rows,
                                            int32_t dtype, pegainfer_stream_t stream);
 /* The same with its options in a struct (zeroed = as above):
- *   gain_offset  is added to every norm weight, the terms' and the gain: 1 for weights stored around zero;
+ *   gain_offset  is added to every norm weight, the terms' and the gain: 1 for weights kept as offsets from one;
  *   row_index    x_in's row of an output row (x_out must then be another buffer);
  *   embed        with x_in NULL the stream starts as embed[token_ids[row]] * embed_scale, plus, when pair_table ([buckets + 1][d]) is
  *                given, its row (prev_ids[row] * mul_prev + token_ids[row] * mul_cur) mod buckets - row `buckets` where prev_ids is

@@ -3,8 +3,8 @@
  *
  * Sopanex: a decoder whose layers are listed one by one in config.json ("layers": type, mixer sizes, feed-forward or none) over an
  * fp32 residual stream that starts as the token's embedding row times a constant plus, when "embedding.bigram" is given, the row of a
- * table addressed by the previous and the current token.  Every sublayer has an RMS norm before and after it, with weights stored
- * around zero: x <- x + norm_b(f(norm(x))).  Mixer "parallel": two mixers that read the same input, left_scale * left + right_scale *
+ * table addressed by the previous and the current token.  Every sublayer has an RMS norm before and after it, with weights kept as
+ * offsets from one: x <- x + norm_b(f(norm(x))).  Mixer "parallel": two mixers that read the same input, left_scale * left + right_scale *
  * right.  Left: softmax attention over grouped key/value heads whose values are the unrotated keys, rotation of the first rot.dims values
  * (value i with value i + rot.dims / 2; optional long-context scaling by a ramp over the dimensions), a sink logit per head and a sigmoid
  * gate per head.  Right: gated linear attention, a decay per (head, key channel) and token from a two-step projection, the read-out

@@ -4,7 +4,7 @@ One function per mechanism, one whole sequence at a time, float64 on the CPU, no
 the recurrence is a Python loop over the tokens from position 0, every attention sees whole score rows.
 
 Notation (n tokens, width D, p = a token's position counted from 0):
-  zrms(x, w)      : x / sqrt(mean(x^2) + eps) * (1 + w)                          a gain stored around zero
+  zrms(x, w)      : x / sqrt(mean(x^2) + eps) * (1 + w)                          a gain kept as its offset from one
   start           : x_t = embed[t] * embedding.scale + bigram[row(t-1, t)],  row = (prev * mul_prev + cur * mul_cur) mod buckets;
                     the first token of a sequence reads the table's extra last row
   sublayer f      : x <- x + zrms(f(zrms(x, norm<q>)), norm<q>b)                 q = 1 mixer, 2 feed-forward (a layer may have no second)

@@ -13,7 +13,7 @@ LAYERS = 8
 
 def sopanex_config(s):
     left = {"heads": s["heads"], "kv_heads": s["kv"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
-            "rot": {"base": 5e5, "dims": 64, "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+            "rot": {"base": 1e6, "dims": 64, "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
     right = {"heads": s["lin_k"], "dim": 128, "vdim": 128, "tau": 16.0, "rank": s["rank"]}
     moe = {"kind": "moe", "expert": {"ff": s["eff"]}, "router": {"experts": s["experts"], "identity": s["experts"] // 4, "top": s["top"], "scale": 2.0},
            "shared": {"ff": s["sff"]}}
@@ -26,7 +26,7 @@ def feruzen_config(s):
     """the same heads side by side: attention of equal sizes beside a matrix memory of equal sizes, the same expert sizes (gated: three matrices)"""
     moe = {"kind": "moe", "expert": {"ff": s["eff"], "limit": 7.0}, "router": {"experts": s["experts"], "top": s["top"]},
            "shared": {"ff": s["sff"], "limit": 7.0}}
-    par = {"left": {"heads": s["heads"], "kv_heads": s["kv"], "dim": 128, "vdim": 128, "rot": {"base": 5e5, "dims": 64}, "scale": 128 ** -0.5},
+    par = {"left": {"heads": s["heads"], "kv_heads": s["kv"], "dim": 128, "vdim": 128, "rot": {"base": 1e6, "dims": 64}, "scale": 128 ** -0.5},
            "right": {"heads": s["lin_k"], "dim": 128, "vdim": 128, "gate_cap": 15.0}, "left_scale": 1.0, "right_scale": 1.0}
     return {"architecture": "Feruzen", "width": s["width"], "vocab": s["vocab"], "norm": {"eps": 1e-5, "groups": 1}, "canon": {"taps": 4},
             "layers": [{"type": "parallel", "mixer": par, "mlp": moe}] * LAYERS}

@@ -28,7 +28,7 @@ constexpr int kFewTiles = 128;      // launches of fewer workgroups deal their k
 constexpr int kFusedRows = 8;       // steps of at most so many rows make the decay inputs inside the scan
 constexpr int kScanMax = 32;        // longest entry whose recurrence runs token by token
 constexpr int kSyntheticRank = 32;  // of the decays' two-step projection when no tensor tells it
-constexpr float kGainOffset = 1.0f; // the stream's norm weights are stored around zero
+constexpr float kGainOffset = 1.0f; // the stream's norm weights are kept as offsets from one
 
 struct AttnCfg {
   int heads = 0, kv = 0, dim = 0, rot_dims = 0;

@@ -397,7 +397,7 @@ __global__ __launch_bounds__(256) void scalar_rms_add_kernel(const float* x_in, 
 //   r = x_in + sum_t term_t                                  -> x_out (fp32; may alias x_in)
 //   n = r / sqrt(mean(r^2) + eps) * gain                     -> n_out (N: float or the storage type; optional)
 // NPT: values a thread keeps between the sum and the norm (d <= 256 * NPT), 0 = any d (the row is summed a second time).
-// gain_offset: added to every norm weight (1: weights stored around zero).  x_in rows may be picked through row_index, or be the
+// gain_offset: added to every norm weight (1: weights kept as offsets from one).  x_in rows may be picked through row_index, or be the
 // token's embedding row times a factor plus the row of a table addressed by (previous token, token).
 struct SumTerm { const void* y; int64_t stride; const void* bias; const void* w; float factor; };
 struct SumTerms { SumTerm t[3]; int n; };

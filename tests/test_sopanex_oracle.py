@@ -142,7 +142,7 @@ PLANTED = {
     "values are the rotated keys": lambda: ("shared_kv_attention", lambda h, w, p, m: _rotated_values(h, w, p, m)),
     "no sink": lambda: ("softmax_with_sink", lambda s, sink: _orig["softmax_with_sink"](s, sink - 1e9)),
     "amplitude left out": lambda: ("turn_frequencies", lambda rot: (_orig["turn_frequencies"](rot)[0], 1.0)),
-    "gain not around zero": lambda: ("zrms", lambda x, w, eps: R.rms(x, eps) * w),
+    "gain without its offset": lambda: ("zrms", lambda x, w, eps: R.rms(x, eps) * w),
     "decay of a whole head": lambda: ("channel_decays", lambda h, w, p, m: _orig["channel_decays"](h, w, p, m).mean(-1, keepdim=True).expand(-1, -1, m["dim"])),
     "first token reads row 0": lambda: ("bigram_rows", lambda t, bg: [0] + _orig["bigram_rows"](t, bg)[1:]),
     "correction weighs too": lambda: ("router", lambda h, w, p, r: _weighing(h, w, p, r)),
